@@ -38,8 +38,8 @@ template <typename T>
 __global__ void bigram_embed_kernel(const T* __restrict__ table, const T* __restrict__ pairs, const int* __restrict__ ids,
                                     const int* __restrict__ positions, const int* __restrict__ seq_of_token,
                                     const int* __restrict__ q_start, float* __restrict__ state,
-                                    const int* __restrict__ state_slots, float* __restrict__ out, int hidden, int buckets,
-                                    int mul_prev, int mul_cur) {
+                                    const int* __restrict__ state_slots, const T* __restrict__ places, int n_places,
+                                    float* __restrict__ out, int hidden, int buckets, int mul_prev, int mul_cur) {
   __shared__ int row_s;
   const int n = blockIdx.x;
   if (threadIdx.x == 0) {
@@ -55,12 +55,20 @@ __global__ void bigram_embed_kernel(const T* __restrict__ table, const T* __rest
   const T* row = table + static_cast<size_t>(ids[n]) * hidden;
   const T* pair = pairs + static_cast<size_t>(row_s) * hidden;
   float* o = out + static_cast<size_t>(n) * hidden;
-  for (int i = threadIdx.x; i < hidden; i += blockDim.x) o[i] = to_float(row[i]) + to_float(pair[i]);
+  if (!places) {
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x) o[i] = to_float(row[i]) + to_float(pair[i]);
+    return;
+  }
+  // a learned row per position; the engine takes no request that is longer than the table
+  const T* place = places + static_cast<size_t>(min(positions[n], n_places - 1)) * hidden;
+  for (int i = threadIdx.x; i < hidden; i += blockDim.x) o[i] = (to_float(row[i]) + to_float(pair[i])) + to_float(place[i]);
 }
 
 extern "C" int pyre_bigram_embed(const void* table, const void* pairs, int dt, const int* ids, const int* positions,
                                  const int* seq_of_token, const int* q_start, float* state, const int* state_slots,
-                                 float* out, int n, int hidden, int buckets, int mul_prev, int mul_cur, hipStream_t stream) {
+                                 const void* places, int n_places, float* out, int n, int hidden, int buckets, int mul_prev,
+                                 int mul_cur, hipStream_t stream) {
+  PYRE_REQUIRE(!places || n_places > 0, "bigram_embed: a table of positions needs rows");
   PYRE_REQUIRE(known_dtype(dt), "bigram_embed: unknown table dtype %d", dt);
   PYRE_REQUIRE(n >= 0 && hidden > 0 && buckets > 0 && mul_prev >= 0 && mul_cur >= 0, "bigram_embed: bad sizes");
   PYRE_REQUIRE(state && state_slots && q_start && seq_of_token && positions, "bigram_embed: the step's arrays and the state are needed");
@@ -68,7 +76,7 @@ extern "C" int pyre_bigram_embed(const void* table, const void* pairs, int dt, c
   PYRE_DISPATCH(dt, T,
                 hipLaunchKernelGGL(bigram_embed_kernel<T>, dim3(n), dim3(256), 0, stream, static_cast<const T*>(table),
                                    static_cast<const T*>(pairs), ids, positions, seq_of_token, q_start, state, state_slots,
-                                   out, hidden, buckets, mul_prev, mul_cur));
+                                   static_cast<const T*>(places), n_places, out, hidden, buckets, mul_prev, mul_cur));
   return check_launch("bigram_embed");
 }
 

@@ -5,10 +5,12 @@
 //                    adds the bias, turns the first `rot` elements of every query and key head by position
 //                    (element e with e + rot/2), stores the queries, the turned keys as keys and the keys
 //                    as they were before turning as values (k, v [pages, nkv, page, d]).
-//   latent_write     attention over one compressed row per token: stores the queries and, if the layer
-//                    makes the row itself, the row divided by its root mean square, times a gain
-//                    (c [pages, 1, page, rank]).
-//   head_matmul      out[n, h, :] = x[n, h, :] W[h] for every head h, W [heads, din, dout]: the products
+//   latent_rows      attention over one compressed row per token: what an input product holds for it. Queries, either
+//                    split into their unturned part (rows) and their turned part (turned by position, straight into the
+//                    wide queries that the attention kernels read), or a compressed row of queries, divided by its root
+//                    mean square, times a gain; the token's row [c | r]: c divided by its root mean square, times a
+//                    gain, r turned by position, into its page; the sigmoids of a gate.
+//   head_matmul      out[n, h, :] = W[h] x[n, h, :] (times a gate) for every head h, W [heads, dout, din]: the products
 //                    that carry a query into the compressed row's space and a weighted row out of it.
 //
 // All arithmetic is float32; roundings happen at the stores of 16-bit outputs only.
@@ -78,30 +80,6 @@ __global__ __launch_bounds__(kThreads) void rope_tied_write_kernel(Proj proj, vo
   }
 }
 
-template <typename TC>
-__global__ __launch_bounds__(kThreads) void latent_write_kernel(Proj proj, void* __restrict__ q_out, int q_dt,
-                                                                TC* __restrict__ c_cache, const void* __restrict__ gain,
-                                                                int gain_dt, float eps, const int* __restrict__ slots,
-                                                                int q_width, int rank, int page_size, int write) {
-  __shared__ float scratch[16];
-  const int n = blockIdx.x;
-  for (int i = threadIdx.x; i < q_width; i += kThreads)
-    store_from_float(q_out, q_dt, static_cast<size_t>(n) * q_width + i, proj_at(proj, n, i));
-  if (!write) return;
-  const int slot = slots[n];
-  float ss = 0.f;
-  for (int i = threadIdx.x; i < rank; i += kThreads) {
-    const float v = proj_at(proj, n, q_width + i);
-    ss += v * v;
-  }
-  ss = block_sum(ss, scratch);
-  if (slot < 0) return;
-  const float inv = 1.f / sqrtf(ss / static_cast<float>(rank) + eps);
-  TC* dst = c_cache + static_cast<size_t>(slot) * rank;  // pages of [1, page, rank]: slot = page * page_size + offset
-  for (int i = threadIdx.x; i < rank; i += kThreads)
-    dst[i] = from_float<TC>(proj_at(proj, n, q_width + i) * inv * load_as_float(gain, gain_dt, i));
-}
-
 // The same with a wave per token and head, four elements a lane and an element's partial sums asked for together:
 // head sizes, the number of turned elements of each half, the product's width, first column and stride are multiples
 // of four; queries, caches and bias share one element type.
@@ -155,80 +133,300 @@ __global__ __launch_bounds__(kWave) void rope_tied_write_vec_kernel(const TP* __
   Vec4<TC>::store(v_cache + at, x);
 }
 
-// Block (n, 0) norms and stores the compressed row, blocks (n, 1 ...) pass 1,024 query columns each: four elements a
-// thread (all widths, first column and strides are multiples of four; gain and cache share one element type).
-template <typename TP, typename TC>
-__global__ __launch_bounds__(kThreads) void latent_write_vec_kernel(const TP* __restrict__ proj, int count, size_t stride, int ld,
-                                                                    int col0, TC* __restrict__ q_out, TC* __restrict__ c_cache,
-                                                                    const TC* __restrict__ gain, float eps,
-                                                                    const int* __restrict__ slots, int q_width, int rank,
-                                                                    int write) {
-  __shared__ float scratch[16];
-  const int n = blockIdx.x, e = 4 * threadIdx.x;
-  const TP* in = proj + static_cast<size_t>(n) * ld + col0;
-  if (blockIdx.y > 0) {
-    const int c = (blockIdx.y - 1) * 4 * kThreads + e;
-    if (c < q_width) Vec4<TC>::store(q_out + static_cast<size_t>(n) * q_width + c, sum_partials4(in + c, stride, count));
-    return;
+// One product's columns for attention over a compressed row, any of the parts present. A token's blocks: one for the
+// row, one for the compressed queries, then blocks of kThreads * W columns for the split queries and for the gate.
+// W = 4: four columns a thread (sizes, first columns, strides and turned halves are multiples of four).
+struct LatentRows {
+  const void* proj;
+  size_t stride;
+  int count, ld;
+  const float* cos_t;
+  const float* sin_t;
+  const int* positions;
+  // split queries: heads of [dim | rot] at column q0; q_out [n][heads * dim], turned parts to wide [n][heads][rank + rot]
+  int heads, dim, q0;
+  void* q_out;
+  void* wide;
+  // compressed queries: q_rank columns at q0, normed into q_out [n][q_rank]
+  int q_rank;
+  const float* q_gain;
+  // the row: rank + rot columns at r0, into cache [pages][1][page][rank + rot] at slots
+  int rank, rot, neighbours, r0;
+  void* cache;
+  const float* gain;
+  const int* slots;
+  // the gate: gate_width columns at g0, float32 [n][gate_width]
+  int gate_width, g0;
+  float* gate;
+  float eps;
+  int row_blocks, norm_blocks, query_blocks;
+};
+
+template <typename TP, int W>
+__device__ inline void columns(const LatentRows& a, int n, int col, float (&v)[W]) {
+  const TP* src = static_cast<const TP*>(a.proj) + static_cast<size_t>(n) * a.ld + col;
+  if constexpr (W == 4) {
+    const float4 x = sum_partials4(src, a.stride, a.count);
+    v[0] = x.x, v[1] = x.y, v[2] = x.z, v[3] = x.w;
+  } else {
+    v[0] = 0.f;
+    for (int p = 0; p < a.count; ++p) v[0] += to_float(src[p * a.stride]);
   }
-  if (!write) return;
-  float4 v = {0.f, 0.f, 0.f, 0.f};
-  if (e < rank) v = sum_partials4(in + q_width + e, stride, count);
-  const float ss = block_sum((v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w), scratch);
-  const int slot = slots[n];
-  if (slot < 0 || e >= rank) return;
-  const float inv = 1.f / sqrtf(ss / static_cast<float>(rank) + eps);
-  const float4 g = Vec4<TC>::load(gain + e);
-  Vec4<TC>::store(c_cache + static_cast<size_t>(slot) * rank + e, float4{v.x * inv * g.x, v.y * inv * g.y, v.z * inv * g.z, v.w * inv * g.w});
 }
 
-// A block: kRows tokens of one head against 64 columns of W[h]. Thread (c, part) walks a quarter of the head's
-// elements for column c of every token; the four parts are added through LDS in their order.
-constexpr int kRows = 16;
-constexpr int kCols = 64;
-template <typename TX, typename TW, typename TO>
-__global__ __launch_bounds__(kThreads) void head_matmul_kernel(const TX* __restrict__ x, int x_ld, const TW* __restrict__ w,
-                                                               TO* __restrict__ out, int out_ld, int n, int din, int dout) {
-  extern __shared__ float lds[];  // xs [kRows][din], then sums [3][kRows][kCols]
-  float* xs = lds;
-  float* sums = lds + kRows * din;
-  const int h = blockIdx.y, n0 = blockIdx.x * kRows, rows = min(kRows, n - n0);
-  const int c = threadIdx.x % kCols, part = threadIdx.x / kCols, col = blockIdx.z * kCols + c;
-  for (int i = threadIdx.x; i < kRows * din; i += kThreads) {
-    const int r = i / din, e = i % din;
-    xs[i] = r < rows ? to_float(x[static_cast<size_t>(n0 + r) * x_ld + h * din + e]) : 0.f;
+template <typename T, int W>
+__device__ inline void put(T* dst, const float (&v)[W]) {
+  if constexpr (W == 4) Vec4<T>::store(dst, float4{v[0], v[1], v[2], v[3]});
+  else *dst = from_float<T>(v[0]);
+}
+
+// Elements e .. e + W - 1 of a part of `rot` turned elements that starts at column col, turned.
+template <typename TP, int W>
+__device__ inline void turned(const LatentRows& a, int n, int col, int e, float (&out)[W]) {
+  const int half = a.rot / 2;
+  const size_t at = static_cast<size_t>(a.positions[n]) * half;
+  float x[W], lost;
+  columns<TP, W>(a, n, col + e, x);
+  if (!a.neighbours) {  // element j with j + half; the W elements lie in one half
+    const bool low = e < half;
+    const int j = low ? e : e - half;
+    float y[W];
+    columns<TP, W>(a, n, col + (low ? e + half : e - half), y);
+#pragma unroll
+    for (int u = 0; u < W; ++u) {
+      const float c = a.cos_t[at + j + u], s = a.sin_t[at + j + u];
+      if (low) rotate_pair(x[u], y[u], c, s, out[u], lost);
+      else rotate_pair(y[u], x[u], c, s, lost, out[u]);
+    }
+  } else if constexpr (W == 4) {
+#pragma unroll
+    for (int u = 0; u < W; u += 2) rotate_pair(x[u], x[u + 1], a.cos_t[at + (e + u) / 2], a.sin_t[at + (e + u) / 2], out[u], out[u + 1]);
+  } else {
+    float y[W];
+    columns<TP, W>(a, n, col + (e ^ 1), y);
+    const float c = a.cos_t[at + e / 2], s = a.sin_t[at + e / 2];
+    if (e & 1) rotate_pair(y[0], x[0], c, s, lost, out[0]);
+    else rotate_pair(x[0], y[0], c, s, out[0], lost);
   }
+}
+
+template <typename TP, typename T, int W>
+__global__ __launch_bounds__(kThreads) void latent_rows_kernel(const LatentRows a) {
+  __shared__ float scratch[16];
+  const int n = blockIdx.x, tid = threadIdx.x;
+  int b = blockIdx.y;
+  if (b < a.row_blocks + a.norm_blocks) {  // a normed part: the row, or the compressed queries
+    const bool row = b < a.row_blocks;
+    const int width = row ? a.rank : a.q_rank, col = row ? a.r0 : a.q0;
+    const float* gain = row ? a.gain : a.q_gain;
+    const int slot = row ? a.slots[n] : 0;
+    T* dst = row ? static_cast<T*>(a.cache) + static_cast<size_t>(max(slot, 0)) * (a.rank + a.rot)
+                 : static_cast<T*>(a.q_out) + static_cast<size_t>(n) * a.q_rank;
+    float first[W], ss = 0.f;  // the thread's first columns stay in registers; wider parts are summed again below
+    for (int i = W * tid; i < width; i += W * kThreads) {
+      float v[W];
+      columns<TP, W>(a, n, col + i, v);
+#pragma unroll
+      for (int u = 0; u < W; ++u) {
+        ss += v[u] * v[u];
+        if (i == W * tid) first[u] = v[u];
+      }
+    }
+    ss = block_sum(ss, scratch);
+    if (row && slot < 0) return;
+    const float inv = 1.f / sqrtf(ss / static_cast<float>(width) + a.eps);
+    for (int i = W * tid; i < width; i += W * kThreads) {
+      float v[W];
+      if (i == W * tid) {
+#pragma unroll
+        for (int u = 0; u < W; ++u) v[u] = first[u];
+      } else {
+        columns<TP, W>(a, n, col + i, v);
+      }
+#pragma unroll
+      for (int u = 0; u < W; ++u) v[u] *= inv * gain[i + u];
+      put<T, W>(dst + i, v);
+    }
+    if (row)
+      for (int e = W * tid; e < a.rot; e += W * kThreads) {
+        float v[W];
+        turned<TP, W>(a, n, a.r0 + a.rank, e, v);
+        put<T, W>(dst + a.rank + e, v);
+      }
+    return;
+  }
+  b -= a.row_blocks + a.norm_blocks;
+  if (b < a.query_blocks) {
+    const int per = a.dim + a.rot, i = W * (b * kThreads + tid);
+    if (i >= a.heads * per) return;
+    const int head = i / per, e = i % per;
+    float v[W];
+    if (e < a.dim) {
+      columns<TP, W>(a, n, a.q0 + i, v);
+      put<T, W>(static_cast<T*>(a.q_out) + (static_cast<size_t>(n) * a.heads + head) * a.dim + e, v);
+    } else {
+      turned<TP, W>(a, n, a.q0 + head * per + a.dim, e - a.dim, v);
+      put<T, W>(static_cast<T*>(a.wide) + (static_cast<size_t>(n) * a.heads + head) * (a.rank + a.rot) + a.rank + (e - a.dim), v);
+    }
+    return;
+  }
+  b -= a.query_blocks;
+  const int i = W * (b * kThreads + tid);
+  if (i >= a.gate_width) return;
+  float v[W];
+  columns<TP, W>(a, n, a.g0 + i, v);
+#pragma unroll
+  for (int u = 0; u < W; ++u) v[u] = 1.f / (1.f + expf(-v[u]));
+  put<float, W>(a.gate + static_cast<size_t>(n) * a.gate_width + i, v);
+}
+
+// ---------------------------------------------------------------------------------------------
+typedef __attribute__((ext_vector_type(16))) float f32x16;
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+struct HeadProduct {
+  const void* x;   // token n, head h at x + n * x_token + h * x_head
+  const void* w;   // [heads][dout][din]
+  void* out;
+  const float* gate;  // [n][heads * dout] or null
+  long x_token, x_head, out_token, out_head;
+  int n, heads, din, dout;
+};
+
+template <typename T>
+__device__ inline f32x16 mfma_unit(uint4 a, uint4 b, f32x16 acc) {
+  if constexpr (sizeof(T) == 2) {
+    acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), acc, 0, 0, 0);
+  } else {
+    const f32x4 af = __builtin_bit_cast(f32x4, a), bf = __builtin_bit_cast(f32x4, b);
+#pragma unroll
+    for (int u = 0; u < 4; ++u) acc = __builtin_amdgcn_mfma_f32_32x32x2f32(af[u], bf[u], acc, 0, 0, 0);
+  }
+  return acc;
+}
+
+template <typename T>
+__device__ inline void head_store(const HeadProduct& a, int token, int head, int h, int col0, const f32x16& acc) {
+  if (token >= a.n) return;
+  T* dst = static_cast<T*>(a.out) + token * a.out_token + head * a.out_head;
+  const float* gate = a.gate ? a.gate + (static_cast<size_t>(token) * a.heads + head) * a.dout : nullptr;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int d = col0 + 8 * j + 4 * h;
+    float v[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) v[u] = d + u < a.dout ? acc[4 * j + u] * (gate ? gate[d + u] : 1.f) : 0.f;
+    if (d + 3 < a.dout && reinterpret_cast<uintptr_t>(dst + d) % (4 * sizeof(T)) == 0) {
+      Vec4<T>::store(dst + d, float4{v[0], v[1], v[2], v[3]});
+    } else {
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+        if (d + u < a.dout) dst[d + u] = from_float<T>(v[u]);
+    }
+  }
+}
+
+// On the matrix cores: rows of the tile are columns of the output (W's rows), its columns are tokens, so that a lane
+// holds neighbouring outputs of one token. A lane's operands are 16-byte units of W's rows and of x, straight from
+// memory (both are small and shared by many blocks). FEW: a block is one tile of 32 outputs and 32 tokens whose
+// inner product its four waves share (parts added through LDS, in order); else a wave has R x C such tiles.
+template <typename T>
+__global__ __launch_bounds__(kThreads) void head_matmul_few_kernel(const HeadProduct a) {
+  constexpr int E = 16 / sizeof(T);
+  __shared__ __attribute__((aligned(16))) float parts[3][4][64][4];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, h = lane >> 5, c = lane & 31;
+  const int head = blockIdx.y, col0 = blockIdx.z * 32, token = blockIdx.x * 32 + c;
+  const int steps = (a.din + 2 * E - 1) / (2 * E), per = (steps + 3) / 4, s0 = wave * per, s1 = min(steps, s0 + per);
+  const T* wrow = static_cast<const T*>(a.w) + (static_cast<size_t>(head) * a.dout + min(col0 + c, a.dout - 1)) * a.din + E * h;
+  const T* xrow = static_cast<const T*>(a.x) + min(token, a.n - 1) * a.x_token + head * a.x_head + E * h;
+  f32x16 acc;
+#pragma unroll
+  for (int i = 0; i < 16; ++i) acc[i] = 0.f;
+  const uint4 zero = {0u, 0u, 0u, 0u};
+  for (int s = s0; s < s1; s += 4) {
+    uint4 wv[4], xv[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const bool in = s + u < s1 && 2 * E * (s + u) + E * h < a.din;
+      wv[u] = in ? *reinterpret_cast<const uint4*>(wrow + 2 * E * (s + u)) : zero;
+      xv[u] = in ? *reinterpret_cast<const uint4*>(xrow + 2 * E * (s + u)) : zero;
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) acc = mfma_unit<T>(wv[u], xv[u], acc);
+  }
+  if (wave > 0)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) *reinterpret_cast<f32x4*>(parts[wave - 1][j][lane]) = f32x4{acc[4 * j], acc[4 * j + 1], acc[4 * j + 2], acc[4 * j + 3]};
   __syncthreads();
-  const int per = (din + 3) / 4, e0 = part * per, e1 = min(din, e0 + per);
-  const TW* wh = w + static_cast<size_t>(h) * din * dout + min(col, dout - 1);
-  float acc[kRows];
+  if (wave > 0) return;
 #pragma unroll
-  for (int r = 0; r < kRows; ++r) acc[r] = 0.f;
-  int e = e0;
-  for (; e + 8 <= e1; e += 8) {  // eight of W's rows on their way together
-    float wv[8];
+  for (int w = 0; w < 3; ++w)
 #pragma unroll
-    for (int u = 0; u < 8; ++u) wv[u] = to_float(wh[static_cast<size_t>(e + u) * dout]);
+    for (int j = 0; j < 4; ++j) {
+      const f32x4 p = *reinterpret_cast<const f32x4*>(parts[w][j][lane]);
 #pragma unroll
-    for (int u = 0; u < 8; ++u)
+      for (int u = 0; u < 4; ++u) acc[4 * j + u] += p[u];
+    }
+  head_store<T>(a, token, head, h, col0, acc);
+}
+
+template <typename T>
+__global__ __launch_bounds__(kThreads) void head_matmul_many_kernel(const HeadProduct a) {
+  constexpr int E = 16 / sizeof(T), R = 2, C = 2;  // tiles of outputs, tiles of tokens of a wave
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, h = lane >> 5, c = lane & 31;
+  const int head = blockIdx.y, col0 = blockIdx.z * 64 * R + (wave & 1) * 32 * R, tok0 = blockIdx.x * 64 * C + (wave >> 1) * 32 * C;
+  const int steps = (a.din + 2 * E - 1) / (2 * E);
+  if (col0 >= a.dout || tok0 >= a.n) return;
+  const T* wrow[R];
+  const T* xrow[C];
 #pragma unroll
-      for (int r = 0; r < kRows; ++r) acc[r] = fmaf(xs[r * din + e + u], wv[u], acc[r]);
+  for (int r = 0; r < R; ++r)
+    wrow[r] = static_cast<const T*>(a.w) + (static_cast<size_t>(head) * a.dout + min(col0 + 32 * r + c, a.dout - 1)) * a.din + E * h;
+#pragma unroll
+  for (int t = 0; t < C; ++t) xrow[t] = static_cast<const T*>(a.x) + min(tok0 + 32 * t + c, a.n - 1) * a.x_token + head * a.x_head + E * h;
+  f32x16 acc[R][C];
+#pragma unroll
+  for (int r = 0; r < R; ++r)
+#pragma unroll
+    for (int t = 0; t < C; ++t)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) acc[r][t][i] = 0.f;
+  const uint4 zero = {0u, 0u, 0u, 0u};
+  for (int s = 0; s < steps; s += 2) {
+    uint4 wv[2][R], xv[2][C];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const bool in = 2 * E * (s + u) + E * h < a.din;
+#pragma unroll
+      for (int r = 0; r < R; ++r) wv[u][r] = in ? *reinterpret_cast<const uint4*>(wrow[r] + 2 * E * (s + u)) : zero;
+#pragma unroll
+      for (int t = 0; t < C; ++t) xv[u][t] = in ? *reinterpret_cast<const uint4*>(xrow[t] + 2 * E * (s + u)) : zero;
+    }
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+      for (int r = 0; r < R; ++r)
+#pragma unroll
+        for (int t = 0; t < C; ++t) acc[r][t] = mfma_unit<T>(wv[u][r], xv[u][t], acc[r][t]);
   }
-  for (; e < e1; ++e) {
-    const float wv = to_float(wh[static_cast<size_t>(e) * dout]);
 #pragma unroll
-    for (int r = 0; r < kRows; ++r) acc[r] = fmaf(xs[r * din + e], wv, acc[r]);
-  }
-  if (part > 0)
+  for (int t = 0; t < C; ++t)
 #pragma unroll
-    for (int r = 0; r < kRows; ++r) sums[((part - 1) * kRows + r) * kCols + c] = acc[r];
-  __syncthreads();
-  if (part > 0 || col >= dout) return;
-#pragma unroll
-  for (int r = 0; r < kRows; ++r) {
-    const float total = ((acc[r] + sums[r * kCols + c]) + sums[(kRows + r) * kCols + c]) + sums[(2 * kRows + r) * kCols + c];
-    if (r < rows) out[static_cast<size_t>(n0 + r) * out_ld + h * dout + col] = from_float<TO>(total);
-  }
+    for (int r = 0; r < R; ++r) head_store<T>(a, tok0 + 32 * t + c, head, h, col0 + 32 * r, acc[r][t]);
+}
+
+// Any sizes: a thread an output.
+template <typename T>
+__global__ __launch_bounds__(kThreads) void head_matmul_any_kernel(const HeadProduct a) {
+  const int n = blockIdx.x, head = blockIdx.y, d = blockIdx.z * kThreads + threadIdx.x;
+  if (d >= a.dout) return;
+  const T* x = static_cast<const T*>(a.x) + n * a.x_token + head * a.x_head;
+  const T* w = static_cast<const T*>(a.w) + (static_cast<size_t>(head) * a.dout + d) * a.din;
+  float v = 0.f;
+  for (int e = 0; e < a.din; ++e) v = fmaf(to_float(w[e]), to_float(x[e]), v);
+  if (a.gate) v *= a.gate[(static_cast<size_t>(n) * a.heads + head) * a.dout + d];
+  static_cast<T*>(a.out)[n * a.out_token + head * a.out_head + d] = from_float<T>(v);
 }
 
 }  // namespace
@@ -263,42 +461,62 @@ extern "C" int pyre_rope_tied_write(const void* proj, int proj_dt, int n_partial
   return check_launch("rope_tied_write");
 }
 
-extern "C" int pyre_latent_write(const void* proj, int proj_dt, int n_partials, long partial_stride, int ld, int col0,
-                                 void* q_out, int q_dt, void* c_cache, int cache_dt, const void* gain, int gain_dt,
-                                 float eps, const int* slots, int n, int q_width, int rank, int page_size, int write,
-                                 hipStream_t stream) {
-  PYRE_REQUIRE(known_dtype(proj_dt) && known_dtype(q_dt) && known_dtype(cache_dt) && n_partials >= 1, "latent_write: bad dtypes");
-  PYRE_REQUIRE(q_width > 0 && rank > 0 && page_size > 0, "latent_write: bad geometry");
-  PYRE_REQUIRE(!write || (c_cache && gain && slots && known_dtype(gain_dt) && eps > 0.f), "latent_write: a cache write needs cache, gain, slots and eps");
+extern "C" int pyre_latent_rows(const void* proj, int proj_dt, int n_partials, long partial_stride, int ld, int dt,
+                                const float* cos_t, const float* sin_t, int neighbours, const int* positions, int rank, int rot,
+                                int heads, int dim, int q_rank, int q0, void* q_out, void* wide, const float* q_gain,
+                                int r0, void* cache, const float* gain, const int* slots, int gate_width, int g0,
+                                float* gate, float eps, int n, hipStream_t stream) {
+  PYRE_REQUIRE(known_dtype(proj_dt) && known_dtype(dt) && n_partials >= 1 && proj && ld > 0, "latent_rows: bad product");
+  PYRE_REQUIRE(rank > 0 && rot >= 0 && rot % 2 == 0 && (rot == 0 || (cos_t && sin_t && positions)), "latent_rows: %d turned elements", rot);
+  PYRE_REQUIRE(heads >= 0 && q_rank >= 0 && (heads == 0 || q_rank == 0) && (heads == 0 || (dim > 0 && q_out && (rot == 0 || wide))) &&
+                   (q_rank == 0 || (q_gain && q_out)), "latent_rows: bad queries");
+  PYRE_REQUIRE(!cache || (gain && slots), "latent_rows: a row needs a gain and slots");
+  PYRE_REQUIRE(gate_width >= 0 && (gate_width == 0 || gate) && (eps > 0.f || (!cache && q_rank == 0)), "latent_rows: bad gate or eps");
+  PYRE_REQUIRE((heads == 0 || (q0 >= 0 && q0 + heads * (dim + rot) <= ld)) && (q_rank == 0 || (q0 >= 0 && q0 + q_rank <= ld)) &&
+                   (!cache || (r0 >= 0 && r0 + rank + rot <= ld)) && (gate_width == 0 || (g0 >= 0 && g0 + gate_width <= ld)),
+               "latent_rows: columns outside the product's %d", ld);
   if (n <= 0) return 0;
+  LatentRows a{};
+  a.proj = proj, a.stride = static_cast<size_t>(partial_stride), a.count = n_partials, a.ld = ld;
+  a.cos_t = cos_t, a.sin_t = sin_t, a.positions = positions, a.neighbours = neighbours;
+  a.heads = heads, a.dim = dim, a.q0 = q0, a.q_out = q_out, a.wide = wide, a.q_rank = q_rank, a.q_gain = q_gain;
+  a.rank = rank, a.rot = rot, a.r0 = r0, a.cache = cache, a.gain = gain, a.slots = slots;
+  a.gate_width = gate_width, a.g0 = g0, a.gate = gate, a.eps = eps;
+  a.row_blocks = cache ? 1 : 0, a.norm_blocks = q_rank > 0 ? 1 : 0;
   const auto a16 = [](const void* q) { return reinterpret_cast<uintptr_t>(q) % 16 == 0; };
-  if (q_width % 4 == 0 && rank % 4 == 0 && rank <= 4 * kThreads && ld % 4 == 0 && col0 % 4 == 0 && partial_stride % 4 == 0 &&
-      q_dt == cache_dt && (!write || gain_dt == cache_dt) && a16(proj) && a16(q_out) && a16(c_cache) && a16(gain)) {
-    const dim3 grid(n, 1 + (q_width + 4 * kThreads - 1) / (4 * kThreads));
-    PYRE_DISPATCH(proj_dt, TP, PYRE_DISPATCH(cache_dt, TC,
-        hipLaunchKernelGGL((latent_write_vec_kernel<TP, TC>), grid, dim3(kThreads), 0, stream, static_cast<const TP*>(proj),
-                           n_partials, static_cast<size_t>(partial_stride), ld, col0, static_cast<TC*>(q_out),
-                           static_cast<TC*>(c_cache), static_cast<const TC*>(gain), eps, slots, q_width, rank, write)));
-    return check_launch("latent_write");
-  }
-  const Proj p{proj, proj_dt, n_partials, static_cast<size_t>(partial_stride), ld, col0, nullptr, 0};
-  PYRE_DISPATCH(cache_dt, TC,
-      hipLaunchKernelGGL(latent_write_kernel<TC>, dim3(n), dim3(kThreads), 0, stream, p, q_out, q_dt,
-                         static_cast<TC*>(c_cache), gain, gain_dt, eps, slots, q_width, rank, page_size, write));
-  return check_launch("latent_write");
+  const bool vec = ld % 4 == 0 && partial_stride % 4 == 0 && q0 % 4 == 0 && r0 % 4 == 0 && g0 % 4 == 0 && rank % 4 == 0 &&
+                   rot % (neighbours ? 4 : 8) == 0 && dim % 4 == 0 && q_rank % 4 == 0 && gate_width % 4 == 0 && a16(proj) &&
+                   a16(q_out) && a16(wide) && a16(cache) && a16(gate);
+  const int per_block = kThreads * (vec ? 4 : 1);
+  a.query_blocks = heads > 0 ? (heads * (dim + rot) + per_block - 1) / per_block : 0;
+  const int blocks = a.row_blocks + a.norm_blocks + a.query_blocks + (gate_width + per_block - 1) / per_block;
+  PYRE_REQUIRE(blocks <= 65535, "latent_rows: too many columns");
+  if (blocks == 0) return 0;
+  PYRE_DISPATCH(proj_dt, TP, PYRE_DISPATCH(dt, T, {
+    if (vec) hipLaunchKernelGGL((latent_rows_kernel<TP, T, 4>), dim3(n, blocks), dim3(kThreads), 0, stream, a);
+    else hipLaunchKernelGGL((latent_rows_kernel<TP, T, 1>), dim3(n, blocks), dim3(kThreads), 0, stream, a);
+  }));
+  return check_launch("latent_rows");
 }
 
-extern "C" int pyre_head_matmul(const void* x, int x_ld, const void* w, void* out, int out_ld, int dt, int n, int heads,
-                                int din, int dout, hipStream_t stream) {
-  PYRE_REQUIRE(known_dtype(dt), "head_matmul: unknown dtype");
-  PYRE_REQUIRE(heads > 0 && heads <= 65535 && din > 0 && dout > 0 && x_ld >= heads * din && out_ld >= heads * dout,
+extern "C" int pyre_head_matmul(const void* x, long x_token, long x_head, const void* w, void* out, long out_token,
+                                long out_head, const float* gate, int dt, int n, int heads, int din, int dout,
+                                hipStream_t stream) {
+  PYRE_REQUIRE(known_dtype(dt) && x && w && out, "head_matmul: bad arguments");
+  PYRE_REQUIRE(heads > 0 && heads <= 65535 && din > 0 && dout > 0 && x_token >= 0 && x_head >= din && out_head >= dout,
                "head_matmul: bad geometry");
-  const size_t lds = sizeof(float) * (static_cast<size_t>(kRows) * din + 3 * kRows * kCols);
-  PYRE_REQUIRE(lds <= 64 * 1024 && (dout + kCols - 1) / kCols <= 65535, "head_matmul: heads of %d elements are too wide", din);
+  PYRE_REQUIRE((dout + 31) / 32 <= 65535, "head_matmul: heads of %d outputs are too wide", dout);
   if (n <= 0) return 0;
-  const dim3 grid((n + kRows - 1) / kRows, heads, (dout + kCols - 1) / kCols);
-  PYRE_DISPATCH(dt, T,
-      hipLaunchKernelGGL((head_matmul_kernel<T, T, T>), grid, dim3(kThreads), lds, stream, static_cast<const T*>(x), x_ld,
-                         static_cast<const T*>(w), static_cast<T*>(out), out_ld, n, din, dout));
+  const HeadProduct a{x, w, out, gate, x_token, x_head, out_token, out_head, n, heads, din, dout};
+  const int E = dt == kBF16 ? 8 : 4;
+  if (din % E == 0 && x_token % E == 0 && x_head % E == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0) {
+    // (the float32 form has one order of sums whatever the number of tokens)
+    if (n <= 64 || dt == kF32)
+      PYRE_DISPATCH(dt, T, hipLaunchKernelGGL(head_matmul_few_kernel<T>, dim3((n + 31) / 32, heads, (dout + 31) / 32), dim3(kThreads), 0, stream, a));
+    else
+      hipLaunchKernelGGL(head_matmul_many_kernel<bf16>, dim3((n + 127) / 128, heads, (dout + 127) / 128), dim3(kThreads), 0, stream, a);
+    return check_launch("head_matmul");
+  }
+  PYRE_DISPATCH(dt, T, hipLaunchKernelGGL(head_matmul_any_kernel<T>, dim3(n, heads, (dout + kThreads - 1) / kThreads), dim3(kThreads), 0, stream, a));
   return check_launch("head_matmul");
 }

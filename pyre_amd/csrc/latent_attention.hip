@@ -1,0 +1,477 @@
+// Softmax attention over one compressed row per token that all query heads share: the row [c | r] of a token is `rank`
+// elements c, which serve as key and as value, and `dk - rank` further elements r of the key alone (a part that was
+// turned by position). A query of head h is [Wuk_h^T q_h | turned part] of dk elements, so that its product with a row
+// is the score of the head's own key; what comes out is the weighted sum of the c. Rows lie in pages
+// [pages, 1, page, dk].
+//
+//   s(i, j) = (q_i . row_j) * scale;  i sees j iff j <= i and (window == 0 or i - j < window)
+//   out_i   = sum_j softmax_j(s(i, .)) c_j, with exp(sink[head]) in the denominator if there is a sink
+//
+// One kernel in two forms. A row tile of the matrix cores is 32 queries: for prompt portions the tokens of a tile
+// (up to 32 consecutive tokens of a request) for one head, for single tokens 32 heads of the token. G such row tiles
+// share a block and the chunk of 32 keys that it keeps in LDS; SL waves share a row tile: each takes every SL-th step
+// of the score's inner product (the parts are added through LDS, in order) and NVT * 32 columns of the output. The
+// problem is transposed, S^T[key, query] and O^T[d, query], so that a lane's sixteen scores are operands of the second
+// product as they are. Scores, maxima, weights and sums are float32, the exponentials base two on scores scaled by
+// log2(e). bfloat16 rows and queries go through the 16-bit instruction (a product of two is exact in float32), each
+// float32 weight as three bfloat16 pieces that sum to it exactly; float32 rows and queries through the float32
+// instruction.
+//
+// Chunks start at multiples of 32 positions, spans (a single token's keys dealt to several blocks) at multiples of
+// `span`: the order of a query's sums follows from its own position alone.
+#include "pyre_api.h"
+#include "pyre_common.h"
+#include "pyre_vec4.h"
+
+using namespace pyre;
+
+namespace {
+
+typedef __attribute__((ext_vector_type(16))) float f32x16;
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+typedef __attribute__((ext_vector_type(4))) __bf16 bf16x4;
+typedef __attribute__((ext_vector_type(4))) short s16x4;
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+constexpr int kKeys = 32;
+constexpr int kRing = 4;
+constexpr float kLog2e = 1.44269504088896340736f;
+
+struct LatentArgs {
+  const void* q;            // [n][heads][dk]
+  const void* rows;         // [pages][1][page][dk]
+  void* out;                // [n][heads][rank]
+  float* part;              // single tokens, several spans: [listed][heads][spans][rank + 2], else null
+  const int* list;          // tiles (first token, count), or single tokens (null: token = block)
+  const int* positions;
+  const int* seq_of_token;
+  const int* table;
+  const float* sink;        // [heads] or null
+  int table_stride, heads, rank, dk, page_size, window, span, spans, vec, tab_lds, two_buffers;
+  float scale2;             // scale * log2(e)
+};
+
+// A barrier that waits for LDS traffic alone: the next chunk's rows stay on their way.
+__device__ inline void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+__device__ inline float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
+
+// 1 / denominator for sums made against the maximum m (base two), a sink included.
+__device__ inline float latent_factor(float m, float l, const float* sink, int head) {
+  if (!sink) return l > 0.f ? 1.f / l : 0.f;
+  const float sk = sink[head] * kLog2e, M = fmaxf(m, sk);
+  const float a = m == -INFINITY ? 0.f : exp2_hw(m - M);
+  return a / (l * a + exp2_hw(sk - M));
+}
+
+// Four keys of sixteen neighbouring columns, transposed on the way out of LDS: of each group of sixteen lanes, lane j
+// gives the address of four columns 4 (j % 4) .. of key j / 4 and receives column j of the four keys.
+__device__ inline uint2 read_transposed(const bf16* p) {
+  const auto v = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+      (__attribute__((address_space(3))) s16x4*)(const_cast<bf16*>(p)));
+  return __builtin_bit_cast(uint2, v);
+}
+
+template <typename T, int G, int SL, int NVT, int KQ, bool SINGLE>
+__global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentArgs a) {
+  constexpr int NT = 64 * G * SL, TPR = NT / kKeys;     // threads that bring one key's row
+  constexpr int E = 16 / sizeof(T);                      // elements of a 16-byte unit
+  constexpr int KI = (2 * KQ * SL + TPR - 1) / TPR;      // units a thread brings of a row
+  extern __shared__ __attribute__((aligned(16))) unsigned char lds_raw[];
+  const int steps = (a.dk + 2 * E - 1) / (2 * E), ldk = 2 * E * steps + E;
+  T* Ks = reinterpret_cast<T*>(lds_raw);                                   // [1 or 2][32][ldk], then slack
+  const int buffer = kKeys * ldk, slack = max(0, 32 * NVT * SL - ldk);
+  const int k_elems = ((a.two_buffers ? 2 : 1) * buffer + slack + 7) / 8 * 8;
+  float* sred = reinterpret_cast<float*>(Ks + k_elems);                    // [G * SL][16][64] if SL > 1
+  int* tab_s = reinterpret_cast<int*>(sred + (SL > 1 ? G * SL * 1024 : 0));
+  __shared__ int slot_s[kRing][kKeys];
+
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = lane >> 5, c = lane & 31;
+  const int g = wave / SL, sl = wave % SL;
+  int t0, ntok = 1;
+  if (SINGLE) {
+    t0 = a.list ? a.list[blockIdx.x] : blockIdx.x;
+  } else {
+    t0 = a.list[2 * blockIdx.x], ntok = a.list[2 * blockIdx.x + 1];
+    if (ntok <= 0) return;
+  }
+  const int pos0 = a.positions[t0];
+  const int* table = a.table + static_cast<size_t>(a.seq_of_token[t0]) * a.table_stride;
+  // this lane's query
+  const int head = SINGLE ? (blockIdx.y * G + g) * 32 + c : blockIdx.y * G + g;
+  const int token = SINGLE ? t0 : t0 + c;
+  const bool active = SINGLE ? (blockIdx.y * G + g) * 32 < a.heads : head < a.heads;  // the whole row tile
+  const bool live = active && (SINGLE ? head < a.heads : c < ntok);
+  const auto first_seen = [&](int pos) { return a.window > 0 ? max(0, pos - a.window + 1) : 0; };
+  const int hi = SINGLE || c >= ntok ? pos0 : pos0 + c, lo = first_seen(hi);
+  const int lo_tile = first_seen(pos0), hi_tile = pos0 + ntok - 1;
+  int lo_all = lo_tile, hi_all = hi_tile;
+  if (SINGLE && a.span > 0) {
+    const int s0 = (lo_tile / a.span + static_cast<int>(blockIdx.z)) * a.span;
+    lo_all = max(lo_all, s0), hi_all = min(hi_all, s0 + a.span - 1);
+    if (lo_all > hi_all) return;
+  }
+  const int chunk0 = lo_all / kKeys, n_chunks = hi_all / kKeys - chunk0 + 1;
+  const int lo_last = first_seen(hi_tile);  // a chunk from here to pos0 is seen whole by every query
+
+  const int entry0 = lo_all / a.page_size;
+  if (a.tab_lds)
+    for (int i = tid; i < min(a.tab_lds, hi_all / a.page_size - entry0 + 1); i += NT)
+      tab_s[i] = entry0 + i < a.table_stride ? table[entry0 + i] : -1;
+
+  uint4 qf[KQ];
+  {
+    const T* qrow = static_cast<const T*>(a.q) + (static_cast<size_t>(token) * a.heads + head) * a.dk;
+#pragma unroll
+    for (int st = 0; st < KQ; ++st) {
+      const int e0 = 2 * E * (st * SL + sl) + E * h;
+      qf[st] = uint4{0u, 0u, 0u, 0u};
+      if (!live || e0 >= a.dk) continue;
+      if (a.vec) {
+        qf[st] = *reinterpret_cast<const uint4*>(qrow + e0);
+      } else {
+        uint32_t w[4] = {0u, 0u, 0u, 0u};
+#pragma unroll
+        for (int u = 0; u < E; ++u)
+          if (e0 + u < a.dk) {
+            if constexpr (sizeof(T) == 4) w[u] = __builtin_bit_cast(uint32_t, qrow[e0 + u]);
+            else w[u >> 1] |= static_cast<uint32_t>(__builtin_bit_cast(uint16_t, qrow[e0 + u])) << (16 * (u & 1));
+          }
+        qf[st] = uint4{w[0], w[1], w[2], w[3]};
+      }
+    }
+  }
+  __syncthreads();  // the table is in LDS
+
+  auto slot_of = [&](int key) {
+    if (key < lo_all || key > hi_all) return -1;
+    const int entry = key / a.page_size;
+    if (entry >= a.table_stride) return -1;
+    const int page = a.tab_lds ? tab_s[entry - entry0] : table[entry];
+    return page < 0 ? -1 : page * a.page_size + key % a.page_size;
+  };
+  const int my_row = tid / TPR, my_unit = tid % TPR;
+  uint4 reg[KI];
+  int reg_slot = -1;
+  auto ask = [&](int it) {
+    reg_slot = slot_s[it % kRing][my_row];
+    if (!a.vec) return;
+    const uint4* src = reinterpret_cast<const uint4*>(static_cast<const T*>(a.rows) + static_cast<size_t>(max(reg_slot, 0)) * a.dk);
+#pragma unroll
+    for (int k = 0; k < KI; ++k) {
+      const int unit = my_unit + k * TPR;
+      reg[k] = uint4{0u, 0u, 0u, 0u};
+      if (reg_slot >= 0 && unit * E < a.dk) reg[k] = src[unit];
+    }
+  };
+  auto stash = [&](int it) {
+    T* dst = Ks + (a.two_buffers ? (it & 1) * buffer : 0) + my_row * ldk;
+    if (a.vec) {
+#pragma unroll
+      for (int k = 0; k < KI; ++k) {
+        const int unit = my_unit + k * TPR;
+        if (unit < 2 * steps) *reinterpret_cast<uint4*>(dst + unit * E) = reg[k];
+      }
+    } else {
+      const T* src = static_cast<const T*>(a.rows) + static_cast<size_t>(max(reg_slot, 0)) * a.dk;
+      for (int e = my_unit; e < 2 * E * steps; e += TPR) dst[e] = reg_slot >= 0 && e < a.dk ? src[e] : from_float<T>(0.f);
+    }
+  };
+
+  f32x16 o[NVT];
+#pragma unroll
+  for (int dt = 0; dt < NVT; ++dt)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) o[dt][i] = 0.f;
+  float m = -INFINITY, l = 0.f;
+
+  if (tid < kKeys) {
+    slot_s[0][tid] = slot_of(chunk0 * kKeys + tid);
+    slot_s[1][tid] = slot_of((chunk0 + 1) * kKeys + tid);
+  }
+  __syncthreads();
+  ask(0);
+  stash(0);
+  __syncthreads();
+  for (int it = 0; it < n_chunks; ++it) {
+    const int key0 = (chunk0 + it) * kKeys;
+    const T* K = Ks + (a.two_buffers ? (it & 1) * buffer : 0);
+    if (it + 1 < n_chunks) ask(it + 1);
+    if (tid < kKeys && it + 2 < n_chunks) slot_s[(it + 2) % kRing][tid] = slot_of(key0 + 2 * kKeys + tid);
+
+    f32x16 s;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) s[i] = 0.f;
+    if (active) {
+      const T* krow = K + c * ldk + E * h;
+#pragma unroll
+      for (int st = 0; st < KQ; ++st) {
+        const int step = st * SL + sl;
+        if (step >= steps) continue;
+        const uint4 k4 = *reinterpret_cast<const uint4*>(krow + 2 * E * step);
+        if constexpr (sizeof(T) == 2) {
+          s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, k4), __builtin_bit_cast(bf16x8, qf[st]), s, 0, 0, 0);
+        } else {
+          const f32x4 kf = __builtin_bit_cast(f32x4, k4), qq = __builtin_bit_cast(f32x4, qf[st]);
+#pragma unroll
+          for (int u = 0; u < 4; ++u) s = __builtin_amdgcn_mfma_f32_32x32x2f32(kf[u], qq[u], s, 0, 0, 0);
+        }
+      }
+      if (SL > 1) {
+        float* mine = sred + wave * 1024 + 4 * lane;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) *reinterpret_cast<f32x4*>(mine + 256 * j) = f32x4{s[4 * j], s[4 * j + 1], s[4 * j + 2], s[4 * j + 3]};
+      }
+    }
+    if (SL > 1) lds_barrier();
+    if (active) {
+      if (SL > 1) {
+        const float* base = sred + g * SL * 1024 + 4 * lane;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          f32x4 t = *reinterpret_cast<const f32x4*>(base + 256 * j);
+#pragma unroll
+          for (int w = 1; w < SL; ++w) t += *reinterpret_cast<const f32x4*>(base + 1024 * w + 256 * j);
+#pragma unroll
+          for (int u = 0; u < 4; ++u) s[4 * j + u] = t[u];
+        }
+      }
+      // element i of s: key key0 + 8 (i / 4) + 4 h + i % 4, query c
+      float mx = -INFINITY;
+      if (key0 >= lo_last && key0 + kKeys - 1 <= pos0) {
+#pragma unroll
+        for (int i = 0; i < 16; ++i) s[i] *= a.scale2, mx = fmaxf(mx, s[i]);
+      } else {
+        const unsigned seen = static_cast<unsigned>(hi - lo), first = static_cast<unsigned>(key0 + 4 * h - lo);
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+          s[i] = first + 8 * (i >> 2) + (i & 3) <= seen ? s[i] * a.scale2 : -INFINITY;
+          mx = fmaxf(mx, s[i]);
+        }
+      }
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      const float m_new = fmaxf(m, mx), m_use = m_new == -INFINITY ? 0.f : m_new;
+      const float alpha = exp2_hw(m - m_use);
+      m = m_new;
+      float sum = 0.f;
+#pragma unroll
+      for (int i = 0; i < 16; ++i) s[i] = exp2_hw(s[i] - m_use), sum += s[i];
+      l = l * alpha + sum;
+      if (__ballot(alpha != 1.f))
+#pragma unroll
+        for (int dt = 0; dt < NVT; ++dt)
+#pragma unroll
+          for (int i = 0; i < 16; ++i) o[dt][i] *= alpha;
+      if constexpr (sizeof(T) == 2) {
+        const int j16 = lane & 15, col16 = 16 * ((lane >> 4) & 1);
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {  // keys 16 b .. 16 b + 15; the lane's eight are 16 b + 4 h + u and 16 b + 8 + 4 h + u
+          uint32_t w1[4], w2[4], w3[4];
+#pragma unroll
+          for (int u = 0; u < 4; ++u) {
+            const float p0 = s[8 * b + 2 * u], p1 = s[8 * b + 2 * u + 1];
+            w1[u] = pack_bf16x2(p0, p1);
+            const float r0 = p0 - __uint_as_float(w1[u] << 16), r1 = p1 - __uint_as_float(w1[u] & 0xffff0000u);
+            w2[u] = pack_bf16x2(r0, r1);
+            w3[u] = pack_bf16x2(r0 - __uint_as_float(w2[u] << 16), r1 - __uint_as_float(w2[u] & 0xffff0000u));
+          }
+          const bf16x8 p1 = __builtin_bit_cast(bf16x8, uint4{w1[0], w1[1], w1[2], w1[3]});
+          const bf16x8 p2 = __builtin_bit_cast(bf16x8, uint4{w2[0], w2[1], w2[2], w2[3]});
+          const bf16x8 p3 = __builtin_bit_cast(bf16x8, uint4{w3[0], w3[1], w3[2], w3[3]});
+          const bf16* vrow = reinterpret_cast<const bf16*>(K) + (16 * b + 4 * h + (j16 >> 2)) * ldk + col16 + 4 * (j16 & 3);
+#pragma unroll
+          for (int dt = 0; dt < NVT; ++dt) {
+            const int d0 = 32 * (sl * NVT + dt);
+            if (d0 >= a.rank) continue;
+            const uint2 v0 = read_transposed(vrow + d0), v1 = read_transposed(vrow + 8 * ldk + d0);
+            const bf16x8 v8 = __builtin_bit_cast(bf16x8, uint4{v0.x, v0.y, v1.x, v1.y});
+            o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8, p3, o[dt], 0, 0, 0);  // the smallest pieces first
+            o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8, p2, o[dt], 0, 0, 0);
+            o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8, p1, o[dt], 0, 0, 0);
+          }
+        }
+      } else {
+#pragma unroll
+        for (int dt = 0; dt < NVT; ++dt) {
+          const int d0 = 32 * (sl * NVT + dt);
+          if (d0 >= a.rank) continue;
+          const float* v = reinterpret_cast<const float*>(K) + 4 * h * ldk + d0 + c;
+#pragma unroll
+          for (int i = 0; i < 16; ++i)
+            o[dt] = __builtin_amdgcn_mfma_f32_32x32x2f32(v[(8 * (i >> 2) + (i & 3)) * ldk], s[i], o[dt], 0, 0, 0);
+        }
+      }
+    }
+    if (!a.two_buffers) lds_barrier();  // every wave is done with the one buffer
+    if (it + 1 < n_chunks) stash(it + 1);
+    lds_barrier();
+  }
+
+  l += __shfl_xor(l, 32, 64);
+  if (!live) return;
+  if (SINGLE && a.part) {
+    float* dst = a.part + ((static_cast<size_t>(blockIdx.x) * a.heads + head) * a.spans + blockIdx.z) * (a.rank + 2);
+#pragma unroll
+    for (int dt = 0; dt < NVT; ++dt)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int d = 32 * (sl * NVT + dt) + 8 * (i >> 2) + 4 * h + (i & 3);
+        if (d < a.rank) dst[d] = o[dt][i];
+      }
+    if (sl == 0 && h == 0) dst[a.rank] = m, dst[a.rank + 1] = l;
+    return;
+  }
+  const float f = latent_factor(m, l, a.sink, head);
+  T* dst = static_cast<T*>(a.out) + (static_cast<size_t>(token) * a.heads + head) * a.rank;
+#pragma unroll
+  for (int dt = 0; dt < NVT; ++dt)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int d = 32 * (sl * NVT + dt) + 8 * j + 4 * h;
+      if (a.vec && d + 3 < a.rank) {
+        Vec4<T>::store(dst + d, float4{o[dt][4 * j] * f, o[dt][4 * j + 1] * f, o[dt][4 * j + 2] * f, o[dt][4 * j + 3] * f});
+      } else {
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          if (d + u < a.rank) dst[d + u] = from_float<T>(o[dt][4 * j + u] * f);
+      }
+    }
+}
+
+// The spans of a single token joined, in their order, with the sink.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_join_kernel(const LatentArgs a) {
+  const int n = a.list ? a.list[blockIdx.x] : blockIdx.x, head = blockIdx.y;
+  const int pos = a.positions[n], lo = a.window > 0 ? max(0, pos - a.window + 1) : 0;
+  const int count = min(a.spans, pos / a.span - lo / a.span + 1), width = a.rank + 2;
+  const float* src = a.part + (static_cast<size_t>(blockIdx.x) * a.heads + head) * a.spans * width;
+  float M = a.sink ? a.sink[head] * kLog2e : -INFINITY;
+  for (int s = 0; s < count; ++s) M = fmaxf(M, src[s * width + a.rank]);
+  const float m_use = M == -INFINITY ? 0.f : M;
+  T* dst = static_cast<T*>(a.out) + (static_cast<size_t>(n) * a.heads + head) * a.rank;
+  for (int d = threadIdx.x; d < a.rank; d += 256) {
+    float total = 0.f, l = 0.f;
+    for (int s = 0; s < count; ++s) {
+      const float w = exp2_hw(src[s * width + a.rank] - m_use);
+      total = fmaf(src[s * width + d], w, total);
+      l = fmaf(src[s * width + a.rank + 1], w, l);
+    }
+    if (a.sink) l += exp2_hw(a.sink[head] * kLog2e - m_use);
+    dst[d] = from_float<T>(l > 0.f ? total / l : 0.f);
+  }
+}
+
+constexpr int kMaxRank = 512, kMaxRow = 640;
+
+int check_args(const char* what, const LatentArgs& a, int dt, int n) {
+  PYRE_REQUIRE(known_dtype(dt) && a.q && a.rows && a.out && a.positions && a.seq_of_token && a.table, "%s: bad arguments", what);
+  PYRE_REQUIRE(a.rank > 0 && a.rank <= kMaxRank && a.dk >= a.rank && a.dk <= kMaxRow, "%s: rows of %d elements, %d of them values, are outside %d / %d",
+               what, a.dk, a.rank, kMaxRow, kMaxRank);
+  PYRE_REQUIRE(a.heads > 0 && a.heads <= 65535 && a.page_size > 0 && a.table_stride > 0 && a.window >= 0 && n >= 0, "%s: bad geometry", what);
+  return 0;
+}
+
+// Launches one form; LDS is what the block asks for, raised once per form where it exceeds what a launch has by default.
+template <typename T, int G, int SL, int NVT, int KQ, bool SINGLE>
+int launch(const char* what, LatentArgs a, int blocks, int spans, hipStream_t stream) {
+  constexpr int E = 16 / sizeof(T);
+  const int steps = (a.dk + 2 * E - 1) / (2 * E), ldk = 2 * E * steps + E;
+  PYRE_REQUIRE(steps <= KQ * SL && a.rank <= 32 * NVT * SL, "%s: rows of %d / %d elements do not fit the form", what, a.dk, a.rank);
+  const size_t slack = 32 * NVT * SL > ldk ? 32 * NVT * SL - ldk : 0, exchange = SL > 1 ? sizeof(float) * G * SL * 1024 : 0;
+  auto k_bytes = [&](int buffers) { return sizeof(T) * ((buffers * kKeys * static_cast<size_t>(ldk) + slack + 7) / 8 * 8); };
+  const size_t budget = 156 * 1024;
+  a.two_buffers = k_bytes(2) + exchange <= budget - 16 * 1024 ? 1 : 0;
+  size_t lds = k_bytes(a.two_buffers ? 2 : 1) + exchange;
+  // the block's part of the request's block table, if it is not too long
+  const int seen = a.window > 0 ? a.window + kKeys : a.table_stride * a.page_size;
+  const int entries = min(seen / a.page_size + 2, a.table_stride + 1);
+  a.tab_lds = lds + sizeof(int) * entries <= budget && entries <= 4096 ? entries : 0;
+  lds += sizeof(int) * a.tab_lds;
+  PYRE_REQUIRE(lds <= budget, "%s: %zu bytes of LDS are more than a block has", what, lds);
+  const int groups = SINGLE ? (a.heads + 32 * G - 1) / (32 * G) : (a.heads + G - 1) / G;
+  const auto kernel = &latent_attn_kernel<T, G, SL, NVT, KQ, SINGLE>;
+  static size_t raised = 64 * 1024;
+  if (lds > raised) {
+    if (hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)) != hipSuccess)
+      return fail("%s: the device refuses %zu bytes of LDS", what, lds);
+    raised = lds;
+  }
+  hipLaunchKernelGGL((latent_attn_kernel<T, G, SL, NVT, KQ, SINGLE>), dim3(blocks, groups, spans), dim3(64 * G * SL), lds, stream, a);
+  return check_launch(what);
+}
+
+bool aligned_rows(const LatentArgs& a, int dt) {
+  const int E = dt == kBF16 ? 8 : 4;
+  return a.dk % E == 0 && a.rank % 4 == 0 && reinterpret_cast<uintptr_t>(a.q) % 16 == 0 && reinterpret_cast<uintptr_t>(a.rows) % 16 == 0 &&
+         reinterpret_cast<uintptr_t>(a.out) % 16 == 0;
+}
+
+}  // namespace
+
+extern "C" int pyre_latent_attn_tile(const void* q, const void* rows, void* out, int dt, const int* tiles, int n_tiles,
+                                     const int* positions, const int* seq_of_token, const int* block_table, int table_stride,
+                                     int heads, int rank, int dk, int page_size, float scale, int window, const float* sink,
+                                     hipStream_t stream) {
+  LatentArgs a{};
+  a.q = q, a.rows = rows, a.out = out, a.list = tiles, a.positions = positions, a.seq_of_token = seq_of_token, a.table = block_table;
+  a.sink = sink, a.table_stride = table_stride, a.heads = heads, a.rank = rank, a.dk = dk, a.page_size = page_size, a.window = window;
+  a.scale2 = scale * kLog2e;
+  if (check_args("latent_attn_tile", a, dt, n_tiles)) return 1;
+  if (n_tiles == 0) return 0;
+  PYRE_REQUIRE(tiles, "latent_attn_tile: no tiles");
+  a.vec = aligned_rows(a, dt);
+  // waves that share a row tile: as few as hold the row and the output in their registers
+  if (rank <= 128 && dk <= 256)
+    return dt == kBF16 ? launch<bf16, 4, 1, 4, 16, false>("latent_attn_tile", a, n_tiles, 1, stream)
+                       : launch<float, 4, 1, 4, 32, false>("latent_attn_tile", a, n_tiles, 1, stream);
+  if (rank <= 256 && dk <= 384)
+    return dt == kBF16 ? launch<bf16, 4, 2, 4, 12, false>("latent_attn_tile", a, n_tiles, 1, stream)
+                       : launch<float, 4, 2, 4, 24, false>("latent_attn_tile", a, n_tiles, 1, stream);
+  return dt == kBF16 ? launch<bf16, 2, 4, 4, 10, false>("latent_attn_tile", a, n_tiles, 1, stream)
+                     : launch<float, 2, 4, 4, 20, false>("latent_attn_tile", a, n_tiles, 1, stream);
+}
+
+// Spans that a single token's keys are dealt to: one where the window is short, else of 64 keys (256 without a window
+// or behind a very long one). The number follows from the window and the widest context of the launch, the span's size
+// from the window alone.
+static int span_of(int window) { return window > 0 && window <= 256 ? 0 : window > 0 && window <= 4096 ? 64 : 256; }
+
+extern "C" int pyre_latent_attn_spans(int max_keys, int window) {
+  const int span = span_of(window);
+  if (span == 0) return 1;
+  const int seen = window > 0 && window < max_keys ? window : max_keys;
+  return (seen > 0 ? seen - 1 : 0) / span + 2;  // a window that starts inside a span touches one more
+}
+
+extern "C" int pyre_latent_attn_single(const void* q, const void* rows, void* out, int dt, const int* tokens, int n,
+                                       const int* positions, const int* seq_of_token, const int* block_table, int table_stride,
+                                       int heads, int rank, int dk, int page_size, float scale, int window, const float* sink,
+                                       float* part, hipStream_t stream) {
+  LatentArgs a{};
+  a.q = q, a.rows = rows, a.out = out, a.list = tokens, a.positions = positions, a.seq_of_token = seq_of_token, a.table = block_table;
+  a.sink = sink, a.table_stride = table_stride, a.heads = heads, a.rank = rank, a.dk = dk, a.page_size = page_size, a.window = window;
+  a.scale2 = scale * kLog2e;
+  if (check_args("latent_attn_single", a, dt, n)) return 1;
+  if (n == 0) return 0;
+  a.vec = aligned_rows(a, dt);
+  a.span = span_of(window);
+  a.spans = pyre_latent_attn_spans(table_stride * page_size, window);
+  PYRE_REQUIRE(a.spans == 1 || part, "latent_attn_single: %d spans need scratch", a.spans);
+  PYRE_REQUIRE(a.spans <= 65535, "latent_attn_single: %d spans are not a launch", a.spans);
+  a.part = a.span ? part : nullptr;
+  if (a.span == 0) a.spans = 1;
+  int bad;
+  if (rank <= 128)
+    bad = dt == kBF16 ? launch<bf16, 1, 4, 1, 10, true>("latent_attn_single", a, n, a.spans, stream)
+                      : launch<float, 1, 4, 1, 20, true>("latent_attn_single", a, n, a.spans, stream);
+  else if (rank <= 256)
+    bad = dt == kBF16 ? launch<bf16, 1, 4, 2, 10, true>("latent_attn_single", a, n, a.spans, stream)
+                      : launch<float, 1, 4, 2, 20, true>("latent_attn_single", a, n, a.spans, stream);
+  else
+    bad = dt == kBF16 ? launch<bf16, 1, 4, 4, 10, true>("latent_attn_single", a, n, a.spans, stream)
+                      : launch<float, 1, 4, 4, 20, true>("latent_attn_single", a, n, a.spans, stream);
+  if (bad) return bad;
+  if (a.part)
+    PYRE_DISPATCH(dt, T, hipLaunchKernelGGL(latent_join_kernel<T>, dim3(n, heads), dim3(256), 0, stream, a));
+  return check_launch("latent_attn_single");
+}

@@ -5,7 +5,7 @@
 //   d      = sum of the pending partial sums (+ bias)
 //   y      = post ? LN(d; post_eps) * post_gain * post_scale : d       (the sublayer's own norm and layer scale)
 //   resid += y
-//   out    = LN(resid; eps) * gain
+//   out    = LN(resid; eps) * gain (+ shift)
 //   LN(x; e) = (x - mean(x)) / sqrt(mean((x - mean(x))^2) + e)
 //
 // One block per row; a thread keeps its elements in registers (every 256th), so the row is read
@@ -26,7 +26,8 @@ __global__ __launch_bounds__(kThreads) void add_layernorm_kernel(
     float* __restrict__ resid, const void* __restrict__ delta, int delta_dt, int n_partials, size_t partial_stride,
     const void* __restrict__ bias, int bias_dt, const void* __restrict__ post_gain, int post_gain_dt,
     const void* __restrict__ post_scale, int post_scale_dt, float post_eps, const void* __restrict__ gain,
-    int gain_dt, void* __restrict__ out, int out_dt, const int* __restrict__ rows, int hidden, float eps) {
+    const void* __restrict__ shift, int gain_dt, void* __restrict__ out, int out_dt, const int* __restrict__ rows,
+    int hidden, float eps) {
   __shared__ float scratch[16];
   const int r_out = blockIdx.x, r_in = rows ? rows[r_out] : r_out, tid = threadIdx.x;
   const size_t row = static_cast<size_t>(r_in) * hidden;
@@ -92,7 +93,10 @@ __global__ __launch_bounds__(kThreads) void add_layernorm_kernel(
 #pragma unroll
   for (int k = 0; k < ITEMS; ++k) {
     const int i = tid + k * kThreads;
-    if (i < hidden) store_from_float(out, out_dt, orow + i, (v[k] - mean) * inv * load_as_float(gain, gain_dt, i));
+    if (i >= hidden) continue;
+    float y = (v[k] - mean) * inv * load_as_float(gain, gain_dt, i);
+    if (shift) y += load_as_float(shift, gain_dt, i);
+    store_from_float(out, out_dt, orow + i, y);
   }
 }
 
@@ -103,7 +107,7 @@ template <typename TD, typename TG, typename TO, int THREADS, int ITEMS>
 __global__ __launch_bounds__(THREADS) void add_layernorm_vec_kernel(
     float* __restrict__ resid, const TD* __restrict__ delta, int n_partials, size_t partial_stride,
     const TG* __restrict__ post_gain, const TG* __restrict__ post_scale, float post_eps, const TG* __restrict__ gain,
-    TO* __restrict__ out, const int* __restrict__ rows, int hidden, float eps) {
+    const TG* __restrict__ shift, TO* __restrict__ out, const int* __restrict__ rows, int hidden, float eps) {
   __shared__ float scratch[16];
   const int r_out = blockIdx.x, r_in = rows ? rows[r_out] : r_out, tid = threadIdx.x, quads = hidden / 4;
   const size_t row = static_cast<size_t>(r_in) * hidden;
@@ -171,8 +175,10 @@ __global__ __launch_bounds__(THREADS) void add_layernorm_vec_kernel(
     const int i = 4 * (tid + k * THREADS);
     if (i < hidden) {
       const float4 gn = Vec4<TG>::load(gain + i);
-      Vec4<TO>::store(out + orow + i, float4{(v[k].x - mean) * inv * gn.x, (v[k].y - mean) * inv * gn.y,
-                                             (v[k].z - mean) * inv * gn.z, (v[k].w - mean) * inv * gn.w});
+      float4 y = {(v[k].x - mean) * inv * gn.x, (v[k].y - mean) * inv * gn.y, (v[k].z - mean) * inv * gn.z,
+                  (v[k].w - mean) * inv * gn.w};
+      if (shift) y = add4(y, Vec4<TG>::load(shift + i));
+      Vec4<TO>::store(out + orow + i, y);
     }
   }
 }
@@ -260,8 +266,8 @@ __global__ void scale_kernel(float* __restrict__ x, size_t total, float s) {
 extern "C" int pyre_add_layernorm(float* resid, const void* delta, int delta_dt, int n_partials, long partial_stride,
                                   const void* bias, int bias_dt, const void* post_gain, int post_gain_dt,
                                   const void* post_scale, int post_scale_dt, float post_eps, const void* gain,
-                                  int gain_dt, void* out, int out_dt, const int* rows, int n, int hidden, float eps,
-                                  hipStream_t stream) {
+                                  const void* shift, int gain_dt, void* out, int out_dt, const int* rows, int n,
+                                  int hidden, float eps, hipStream_t stream) {
   PYRE_REQUIRE(known_dtype(gain_dt) && known_dtype(out_dt), "add_layernorm: unknown dtype");
   PYRE_REQUIRE(!delta || (known_dtype(delta_dt) && n_partials >= 1), "add_layernorm: bad delta (dtype %d, partials %d)",
                delta_dt, n_partials);
@@ -276,6 +282,7 @@ extern "C" int pyre_add_layernorm(float* resid, const void* delta, int delta_dt,
   if (!bias && same_gains && hidden % 4 == 0 && hidden <= 4 * 256 * 16 && (!delta || partial_stride % 4 == 0) &&
       reinterpret_cast<uintptr_t>(delta) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0 &&
       reinterpret_cast<uintptr_t>(gain) % 16 == 0 && reinterpret_cast<uintptr_t>(post_gain) % 16 == 0 &&
+      reinterpret_cast<uintptr_t>(shift) % 16 == 0 &&
       reinterpret_cast<uintptr_t>(post_scale) % 16 == 0) {
     // which shape runs depends on the number of rows; what it computes does not: a row's sums are block
     // sums of per-thread sums either way, and the two shapes differ in how the elements are dealt to threads
@@ -285,7 +292,7 @@ extern "C" int pyre_add_layernorm(float* resid, const void* delta, int delta_dt,
   hipLaunchKernelGGL((add_layernorm_vec_kernel<TD, TG, TO, THREADS, ITEMS>), dim3(n), dim3(THREADS), 0, stream, resid, \
                      static_cast<const TD*>(delta), n_partials, static_cast<size_t>(partial_stride),                   \
                      static_cast<const TG*>(post_gain), static_cast<const TG*>(post_scale), post_eps,                  \
-                     static_cast<const TG*>(gain), static_cast<TO*>(out), rows, hidden, eps)
+                     static_cast<const TG*>(gain), static_cast<const TG*>(shift), static_cast<TO*>(out), rows, hidden, eps)
     PYRE_DISPATCH(delta ? delta_dt : kF32, TD, PYRE_DISPATCH(gain_dt, TG, PYRE_DISPATCH(out_dt, TO, {
       if (few && quads <= 1024) PYRE_LNV(1024, 1);
       else if (few) PYRE_LNV(1024, 4);
@@ -299,7 +306,7 @@ extern "C" int pyre_add_layernorm(float* resid, const void* delta, int delta_dt,
 #define PYRE_LN(ITEMS)                                                                                              \
   hipLaunchKernelGGL(add_layernorm_kernel<ITEMS>, dim3(n), dim3(kThreads), 0, stream, resid, delta, delta_dt,       \
                      n_partials, static_cast<size_t>(partial_stride), bias, bias_dt, post_gain, post_gain_dt,       \
-                     post_scale, post_scale_dt, post_eps, gain, gain_dt, out, out_dt, rows, hidden, eps)
+                     post_scale, post_scale_dt, post_eps, gain, shift, gain_dt, out, out_dt, rows, hidden, eps)
   if (hidden <= 2 * kThreads) PYRE_LN(2);
   else if (hidden <= 8 * kThreads) PYRE_LN(8);
   else if (hidden <= 32 * kThreads) PYRE_LN(32);

@@ -217,17 +217,32 @@ int pyre_gemm_mid_glu_bf16(const void* X, long ldx, const void* W, long ldw, voi
                            float limit, float slope, float shift, float cubic, hipStream_t stream);
 
 // ---- layer norm around the residual stream, clipped gated activation, scaling (layernorm.hip) ----
-// resid += y, out = LN(resid) * gain, where y is the pending term (partial sums, bias) or, with
-// post_gain, LN(term; post_eps) * post_gain (* post_scale). rows: only these rows, resid untouched.
+// resid += y, out = LN(resid) * gain (+ shift), where y is the pending term (partial sums, bias) or, with
+// post_gain, LN(term; post_eps) * post_gain (* post_scale). rows: only these rows, resid untouched. shift: gain's type,
+// or null.
 int pyre_add_layernorm(float* resid, const void* delta, int delta_dt, int n_partials, long partial_stride,
                        const void* bias, int bias_dt, const void* post_gain, int post_gain_dt,
                        const void* post_scale, int post_scale_dt, float post_eps, const void* gain,
-                       int gain_dt, void* out, int out_dt, const int* rows, int n, int hidden, float eps,
-                       hipStream_t stream);
+                       const void* shift, int gain_dt, void* out, int out_dt, const int* rows, int n, int hidden,
+                       float eps, hipStream_t stream);
 // out[n, i] = g sigmoid(slope (g + cubic g^3)) (u + shift), g = min(gate, limit), u = clamp(up, -limit, limit); gu = [gate | up].
 int pyre_clipped_glu(const void* gu, int gu_dt, int n_partials, long partial_stride, void* out, int out_dt,
                      int n, int inter, float limit, float slope, float shift, float cubic, hipStream_t stream);
 int pyre_scale(float* x, long total, float s, hipStream_t stream);
+
+// ---- a residual of several streams (streams.hip) ----
+// x [n][streams][hidden]: src, which holds one row a token (src_streams = 1: all streams equal) or all of them; with y,
+// a sublayer's result as partial sums, x_t <- sum_s mix[s][t] x_s + out_w[t] y first, stored to dst if it is given (it may
+// be src). out = norm(sum_s in_w[s] x_s) * gain (+ shift), in_w null: the plain sum; center: a layer norm, else an RMS
+// norm. picked: only these rows.
+int pyre_stream_norm(const float* src, int src_streams, float* dst, int streams, const void* y, int y_dt, int n_partials,
+                     long partial_stride, const float* mix, const float* out_w, const float* in_w, const float* gain,
+                     const float* shift, int center, float eps, void* out, int out_dt, const int* picked, int n,
+                     int hidden, hipStream_t stream);
+// out = a N(z) + b N(z^2) + c N(z^3) + e, z the partial sums of a product [n, width], N dividing a row by its root mean
+// square, abce four floats (poly_norm.hip).
+int pyre_poly_norm(const void* z, int z_dt, int n_partials, long partial_stride, const float* abce, float eps, void* out,
+                   int out_dt, int n, int width, hipStream_t stream);
 
 // ---- attention with capped scores, a bias by distance and kept first tokens (attention_biased.hip) ----
 // proj columns from col0 on: nq query heads and nkv key heads of dk, nkv value heads of dv, then (gate_out
@@ -297,15 +312,36 @@ int pyre_rope_tied_write(const void* proj, int proj_dt, int n_partials, long par
                          int cache_dt, const float* cos_t, const float* sin_t, int rot, const int* positions,
                          const int* slots, int n, int nq, int nkv, int d, int page_size, int write_kv,
                          hipStream_t stream);
-// proj columns from col0 on: q_width of queries, then (write) rank of the compressed row, which is stored divided
-// by its root mean square and times gain in c_cache [pages, 1, page, rank].
-int pyre_latent_write(const void* proj, int proj_dt, int n_partials, long partial_stride, int ld, int col0,
-                      void* q_out, int q_dt, void* c_cache, int cache_dt, const void* gain, int gain_dt, float eps,
-                      const int* slots, int n, int q_width, int rank, int page_size, int write, hipStream_t stream);
-// out[n, h, :] = x[n, h, :] w[h], w [heads, din, dout]; rows of x and out are x_ld and out_ld elements apart; one
-// element type for all three.
-int pyre_head_matmul(const void* x, int x_ld, const void* w, void* out, int out_ld, int dt, int n, int heads, int din,
-                     int dout, hipStream_t stream);
+// What an input product holds for attention over one compressed row per token; parts that are absent have size 0 or a
+// null pointer. Queries at column q0: `heads` of [dim | rot] elements, unturned parts to q_out [n][heads dim], turned parts
+// (neighbours: element 2j with 2j + 1, else j with j + rot/2) to wide [n][heads][rank + rot] behind rank; or q_rank columns,
+// divided by their root mean square, times q_gain, to q_out [n][q_rank]. The row at column r0: rank elements divided by
+// their root mean square, times gain, and rot turned ones, to cache [pages, 1, page, rank + rot] at slots. The sigmoids of
+// gate_width columns at g0, float32. dt: the type of q_out, wide and cache.
+int pyre_latent_rows(const void* proj, int proj_dt, int n_partials, long partial_stride, int ld, int dt, const float* cos_t,
+                     const float* sin_t, int neighbours, const int* positions, int rank, int rot, int heads, int dim,
+                     int q_rank, int q0, void* q_out, void* wide, const float* q_gain, int r0, void* cache,
+                     const float* gain, const int* slots, int gate_width, int g0, float* gate, float eps, int n,
+                     hipStream_t stream);
+// out[n, h, :] = w[h] x[n, h, :] (* gate[n, h, :]), w [heads, dout, din]; token n's head h lies at n x_token + h x_head
+// elements of x, at n out_token + h out_head of out; one element type for the three.
+int pyre_head_matmul(const void* x, long x_token, long x_head, const void* w, void* out, long out_token, long out_head,
+                     const float* gate, int dt, int n, int heads, int din, int dout, hipStream_t stream);
+
+// ---- softmax attention over one compressed row per token, shared by all heads (latent_attention.hip) ----
+// q [n][heads][dk] against rows [pages, 1, page, dk], whose first `rank` elements are the values as well; out
+// [n][heads][rank]; sink [heads] or null. tiles: (first token, count <= 32) pairs of prompt portions. Single tokens:
+// part float32 [n][heads][spans][rank + 2] with spans = pyre_latent_attn_spans(table_stride * page_size, window), which
+// may be null for one span.
+int pyre_latent_attn_tile(const void* q, const void* rows, void* out, int dt, const int* tiles, int n_tiles,
+                          const int* positions, const int* seq_of_token, const int* block_table, int table_stride,
+                          int heads, int rank, int dk, int page_size, float scale, int window, const float* sink,
+                          hipStream_t stream);
+int pyre_latent_attn_spans(int max_keys, int window);
+int pyre_latent_attn_single(const void* q, const void* rows, void* out, int dt, const int* tokens, int n,
+                            const int* positions, const int* seq_of_token, const int* block_table, int table_stride,
+                            int heads, int rank, int dk, int page_size, float scale, int window, const float* sink,
+                            float* part, hipStream_t stream);
 
 // ---- a mixture of experts with a sigmoid router (moe.hip) ----
 // gates[n, experts + extra] float32: for the `top` experts of largest logit z, s / (sum of the chosen s + 1e-20) with
@@ -325,10 +361,11 @@ int pyre_add_rms_terms(float* resid, const void* a, int a_dt, int a_partials, lo
                        int outer_dt, float outer_eps, const void* out_gain, int out_gain_dt, float out_eps, void* out,
                        int out_dt, const int* rows, int n, int hidden, hipStream_t stream);
 
-// out[n] = table[ids[n]] + pairs[row of (previous token, token)]; state [slots][1] float32 holds a request's last token.
+// out[n] = table[ids[n]] + pairs[row of (previous token, token)] (+ places[position], a table of n_places rows, or null);
+// state [slots][1] float32 holds a request's last token.
 int pyre_bigram_embed(const void* table, const void* pairs, int dt, const int* ids, const int* positions,
-                      const int* seq_of_token, const int* q_start, float* state, const int* state_slots, float* out, int n,
-                      int hidden, int buckets, int mul_prev, int mul_cur, hipStream_t stream);
+                      const int* seq_of_token, const int* q_start, float* state, const int* state_slots, const void* places,
+                      int n_places, float* out, int n, int hidden, int buckets, int mul_prev, int mul_cur, hipStream_t stream);
 
 // The input product of an attention whose projections go through a short causal convolution (conv_attention.hip).
 int pyre_conv_qkv_write(const void* proj, int proj_dt, int n_partials, long partial_stride, int ld, int col0,

@@ -51,6 +51,9 @@ class Engine:
         # max_position_embeddings and never consults it (`pyre/config.py:60`).
         # A model without a limit of its own (max_positions 0) takes the pool's size, or a default.
         self.max_model_len = ec.max_model_len or spec.max_positions or ec.max_cached_tokens or DEFAULT_MAX_MODEL_LEN
+        rows = getattr(model.embedding, "max_positions", 0)
+        if rows:  # learned positions are a bound: there is nothing to add behind the table's last row
+            self.max_model_len = min(self.max_model_len, rows)
         with torch.cuda.device(self.device):
             self.runtime = Runtime(self.device, self.dtype, self.max_model_len)
         specs = model.cache_specs()

@@ -11,7 +11,7 @@ from ctypes import c_float, c_int, c_long, c_void_p
 
 from pyre_amd.hip import build as _build
 
-ABI_VERSION = 28
+ABI_VERSION = 29
 
 
 class KernelError(RuntimeError):
@@ -55,9 +55,11 @@ _SIGNATURES = {
     "pyre_feed_tokens": [P, P, P, I, P],
     "pyre_gemm_skinny_glu_bf16": [P, L, P, L, P, I, I, I, F, F, F, F, P],
     "pyre_gemm_mid_glu_bf16": [P, L, P, L, P, I, I, I, F, F, F, F, P],
-    "pyre_add_layernorm": [P, P, I, I, L, P, I, P, I, P, I, F, P, I, P, I, P, I, I, F, P],
+    "pyre_add_layernorm": [P, P, I, I, L, P, I, P, I, P, I, F, P, P, I, P, I, P, I, I, F, P],
     "pyre_clipped_glu": [P, I, I, L, P, I, I, I, F, F, F, F, P],
     "pyre_scale": [P, L, F, P],
+    "pyre_stream_norm": [P, I, P, I, P, I, I, L, P, P, P, P, P, I, F, P, I, P, I, I, P],
+    "pyre_poly_norm": [P, I, I, L, P, F, P, I, I, I, P],
     "pyre_unit_qkv_write": [P, I, I, L, I, I, P, I, P, P, I, P, P, I, I, I, I, I, I, I, F, I, P],
     "pyre_attn_biased_tile": [P, P, I, I, P, P, P, F, P, I, P, P, P, I, I, I, I, I, I, F, F, P, I, I, I, I, P, I, P],
     "pyre_attn_biased_single": [P, P, I, I, P, P, P, F, P, I, P, P, P, I, I, I, I, I, I, F, F, P, I, I, I, I, P, I, P, I, P],
@@ -70,12 +72,15 @@ _SIGNATURES = {
     "pyre_add_tanhnorm": [P, P, I, I, L, P, I, F, P, I, I, L, P, I, F, P, P, P, I, P, I, P, I, I, P],
     "pyre_softcap": [P, L, F, P],
     "pyre_rope_tied_write": [P, I, I, L, I, I, P, I, P, I, P, P, I, P, P, I, P, P, I, I, I, I, I, I, P],
-    "pyre_latent_write": [P, I, I, L, I, I, P, I, P, I, P, I, F, P, I, I, I, I, I, P],
-    "pyre_head_matmul": [P, I, P, P, I, I, I, I, I, I, P],
+    "pyre_latent_rows": [P, I, I, L, I, I, P, P, I, P, I, I, I, I, I, I, P, P, P, I, P, P, P, I, I, P, F, I, P],
+    "pyre_head_matmul": [P, L, L, P, P, L, L, P, I, I, I, I, I, P],
+    "pyre_latent_attn_tile": [P, P, P, I, P, I, P, P, P, I, I, I, I, I, F, I, P, P],
+    "pyre_latent_attn_spans": [I, I],
+    "pyre_latent_attn_single": [P, P, P, I, P, I, P, P, P, I, I, I, I, I, F, I, P, P, P],
     "pyre_route_topk": [P, I, I, L, P, I, P, I, I, I, I, I, P],
     "pyre_expert_act": [P, I, I, L, P, P, I, I, I, I, I, P],
     "pyre_add_rms_terms": [P, P, I, I, L, P, I, F, P, I, I, L, P, I, F, F, P, I, F, P, I, F, P, I, P, I, I, P],
-    "pyre_bigram_embed": [P, P, I, P, P, P, P, P, P, P, I, I, I, I, I, P],
+    "pyre_bigram_embed": [P, P, I, P, P, P, P, P, P, P, I, P, I, I, I, I, I, P],
     "pyre_conv_qkv_write": [P, I, I, L, I, I, P, I, P, P, P, P, I, P, P, F, P, P, I, I, P, P, I, P, P, I, P, P, I, I, I, I,
                             I, I, I, P],
     "pyre_retention_prepare": [P, I, I, L, I, I, P, P, P, I, I, P, F, P, I, I, I, I, P],

@@ -163,8 +163,8 @@ def add_rmsnorm(resid: torch.Tensor, delta: Partials | None, gain: torch.Tensor,
 
 
 def add_layernorm(resid: torch.Tensor, delta: Partials | None, gain: torch.Tensor, eps: float,
-                  out: torch.Tensor, rows: torch.Tensor | None = None) -> None:
-    """resid += y; out = LN(resid) * gain, with LN(x) = (x - mean) / sqrt(var + eps) and y the
+                  out: torch.Tensor, rows: torch.Tensor | None = None, shift: torch.Tensor | None = None) -> None:
+    """resid += y; out = LN(resid) * gain (+ ``shift``), with LN(x) = (x - mean) / sqrt(var + eps) and y the
     pending term (all partials, then bias), which goes through its own norm first if it carries one
     (``delta.post``: y = LN(term; post.eps) * post.gain * post.scale).
 
@@ -178,6 +178,10 @@ def add_layernorm(resid: torch.Tensor, delta: Partials | None, gain: torch.Tenso
     if out.shape[-1] != hidden or out.shape[0] < n or gain.numel() != hidden:
         raise KernelError("add_layernorm: shapes of out / gain do not fit the residual")
     _contig("resid", resid), _contig("out", out), _contig("gain", gain)
+    if shift is not None:
+        if shift.numel() != hidden or shift.dtype != gain.dtype:
+            raise KernelError("add_layernorm: the shift is one number per element, of the gain's type")
+        _dev(shift), _contig("shift", shift)
     if rows is not None:
         _i32("rows", rows)
     post = (None, 0, None, 0, 0.0)
@@ -200,7 +204,7 @@ def add_layernorm(resid: torch.Tensor, delta: Partials | None, gain: torch.Tenso
                     dtype_code(pn.scale) if pn.scale is not None else 0, float(pn.eps))
     else:
         d = (None, 0, 0, 0, None, 0)
-    call("pyre_add_layernorm", resid.data_ptr(), *d, *post, gain.data_ptr(), dtype_code(gain), out.data_ptr(),
+    call("pyre_add_layernorm", resid.data_ptr(), *d, *post, gain.data_ptr(), _ptr(shift), dtype_code(gain), out.data_ptr(),
          dtype_code(out), _ptr(rows), n, hidden, float(eps), _stream())
 
 
@@ -1067,50 +1071,199 @@ def rope_tied_write(proj: Partials, col0: int, q_out: torch.Tensor, k_cache: tor
          positions.data_ptr(), _ptr(slots), n, nq, nkv, d, page_size, 1 if write else 0, _stream())
 
 
-def latent_write(proj: Partials, col0: int, q_out: torch.Tensor, c_cache: torch.Tensor | None,
-                 gain: torch.Tensor | None, eps: float, slots: torch.Tensor | None, n: int, q_width: int, rank: int,
-                 page_size: int) -> None:
-    """Finish a step's input product from column ``col0`` on: ``q_width`` columns of queries to ``q_out [N, q_width]``
-    and, if ``c_cache [pages, 1, page, rank]`` is given, the ``rank`` columns behind them divided by their root mean
-    square (``eps`` inside the root), times ``gain``, to the cache at ``slots``."""
-    _dev(proj.data, q_out, c_cache, gain, slots)
-    write = c_cache is not None
-    args = _proj_args(proj, col0, q_width + (rank if write else 0))
-    if proj.rows < n or q_out.numel() < n * q_width:
-        raise KernelError("latent_write: buffers are smaller than the batch")
-    _contig("q_out", q_out)
-    cache_dt = dtype_code(q_out)
-    if write:
-        if gain is None or slots is None or gain.numel() != rank:
-            raise KernelError("latent_write: a cache write needs a gain over the rank and slots")
-        _i32("slots", slots, n), _contig("c_cache", c_cache), _contig("gain", gain)
-        if tuple(c_cache.shape[1:]) != (1, page_size, rank):
-            raise KernelError(f"latent_write: cache {tuple(c_cache.shape)} does not fit page={page_size} rank={rank}")
-        cache_dt = dtype_code(c_cache)
-    call("pyre_latent_write", *args, q_out.data_ptr(), dtype_code(q_out), _ptr(c_cache), cache_dt, _ptr(gain),
-         dtype_code(gain) if gain is not None else 0, float(eps), _ptr(slots), n, q_width, rank, page_size,
-         1 if write else 0, _stream())
+def latent_rows(proj: Partials, n: int, rank: int, rot: int, dtype: torch.dtype, cos: torch.Tensor | None = None,
+                sin: torch.Tensor | None = None, neighbours: bool = False, positions: torch.Tensor | None = None,
+                queries: tuple | None = None, normed_queries: tuple | None = None, row: tuple | None = None,
+                gate: tuple | None = None, eps: float = 0.0) -> None:
+    """What an input product holds for attention over one compressed row per token, any of:
+
+    ``queries`` = (column, heads, dim, q_out [N, heads * dim], wide [N, heads * (rank + rot)]): heads of [dim | rot]
+    columns, the first part to ``q_out``, the second turned by position into ``wide`` behind ``rank``;
+    ``normed_queries`` = (column, width, gain, out [N, width]): divided by their root mean square, times the gain;
+    ``row`` = (column, gain, cache [pages, 1, page, rank + rot], slots): ``rank`` columns divided by their root mean
+    square, times the gain, then ``rot`` columns turned; ``gate`` = (column, width, out float32 [N, width]): sigmoids.
+
+    Turned pairs: element 2j with 2j + 1 (``neighbours``) or j with j + rot/2; ``cos`` / ``sin`` float32 [positions,
+    rot/2]. Gains are float32."""
+    _dev(proj.data, proj.bias, cos, sin, positions)
+    if proj.bias is not None or proj.rows < n:
+        raise KernelError("latent_rows: a product without a bias and with the step's rows is expected")
+    if rot:
+        if cos is None or sin is None or positions is None or cos.dtype != torch.float32 or sin.dtype != torch.float32 or \
+                cos.shape[1] != rot // 2 or tuple(sin.shape) != tuple(cos.shape):
+            raise KernelError("latent_rows: cos and sin are float32 [positions, rot / 2]")
+        _contig("cos", cos), _contig("sin", sin), _i32("positions", positions, n)
+    if queries is not None and normed_queries is not None:
+        raise KernelError("latent_rows: queries either as they are or compressed")
+
+    def rows_of(name, t, width, dt):
+        _dev(t), _contig(name, t)
+        if t.dtype != dt or t.numel() < n * width:
+            raise KernelError(f"latent_rows: {name} is {dt} with {width} columns for each of {n} rows")
+        return t.data_ptr()
+
+    def gain_of(t, width):
+        _dev(t), _contig("gain", t)
+        if t.dtype != torch.float32 or t.numel() != width:
+            raise KernelError(f"latent_rows: a gain is float32 [{width}]")
+        return t.data_ptr()
+
+    heads = dim = q_rank = q0 = r0 = g0 = gate_width = 0
+    q_out = wide = q_gain = cache = gain = slots = gate_out = None
+    if queries is not None:
+        q0, heads, dim, q_t, wide_t = queries
+        q_out = rows_of("q_out", q_t, heads * dim, dtype)
+        wide = rows_of("wide", wide_t, heads * (rank + rot), dtype) if rot else None
+    if normed_queries is not None:
+        q0, q_rank, g, q_t = normed_queries
+        q_gain, q_out = gain_of(g, q_rank), rows_of("q_out", q_t, q_rank, dtype)
+    if row is not None:
+        r0, g, c, s = row
+        _dev(c, s), _contig("cache", c), _i32("slots", s, n)
+        if c.dim() != 4 or c.shape[1] != 1 or c.shape[3] != rank + rot or c.dtype != dtype:
+            raise KernelError(f"latent_rows: the cache is {dtype} [pages, 1, page, {rank + rot}], not {tuple(c.shape)}")
+        cache, gain, slots = c.data_ptr(), gain_of(g, rank), s.data_ptr()
+    if gate is not None:
+        g0, gate_width, out_t = gate
+        gate_out = rows_of("gate", out_t, gate_width, torch.float32)
+    call("pyre_latent_rows", proj.data.data_ptr(), dtype_code(proj.data), proj.count, proj.stride, proj.width, dtype_code(dtype),
+         _ptr(cos) if rot else None, _ptr(sin) if rot else None, int(neighbours), _ptr(positions), rank, rot, heads, dim,
+         q_rank, q0, q_out, wide, q_gain, r0, cache, gain, slots, gate_width, g0, gate_out, float(eps), n, _stream())
 
 
-HEAD_MATMUL_MAX_IN = 768  #: the widest head that the per-head product takes (latent.hip)
-
-
-def head_matmul(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, n: int) -> None:
-    """out[n, h, :] = x[n, h, :] @ w[h] for every head: ``w [heads, din, dout]``, ``x [>= n, heads * din]`` and
-    ``out [>= n, heads * dout]`` with contiguous rows, one element type."""
-    _dev(x, w, out)
+def head_matmul(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, n: int, gate: torch.Tensor | None = None) -> None:
+    """out[n, h] = w[h] @ x[n, h] (times ``gate[n, h]``) for every head: ``w [heads, dout, din]``, ``x [>= n, heads, >= din]``
+    (its first din elements), ``out [>= n, heads, >= dout]``, the last axis contiguous, one element type; ``gate`` float32
+    [>= n, heads * dout]."""
+    _dev(x, w, out, gate)
     if w.dim() != 3 or not w.is_contiguous():
-        raise KernelError("head_matmul: w is contiguous [heads, din, dout]")
-    heads, din, dout = w.shape
+        raise KernelError("head_matmul: w is contiguous [heads, dout, din]")
+    heads, dout, din = w.shape
     if not (x.dtype == w.dtype == out.dtype):
         raise KernelError("head_matmul: one element type for x, w and out")
-    if x.dim() != 2 or out.dim() != 2 or x.stride(1) != 1 or out.stride(1) != 1 or x.shape[1] < heads * din or \
-            out.shape[1] < heads * dout or x.shape[0] < n or out.shape[0] < n:
-        raise KernelError("head_matmul: x [>= n, heads*din] and out [>= n, heads*dout] with contiguous rows expected")
-    if din > HEAD_MATMUL_MAX_IN:
-        raise KernelError(f"head_matmul: heads of {din} elements are more than {HEAD_MATMUL_MAX_IN}")
-    call("pyre_head_matmul", x.data_ptr(), x.stride(0), w.data_ptr(), out.data_ptr(), out.stride(0), dtype_code(x), n,
-         heads, din, dout, _stream())
+    for name, t, width in (("x", x, din), ("out", out, dout)):
+        if t.dim() != 3 or t.stride(2) != 1 or t.shape[0] < n or t.shape[1] != heads or t.shape[2] < width:
+            raise KernelError(f"head_matmul: {name} is [>= {n}, {heads}, >= {width}] with contiguous heads, not {tuple(t.shape)}")
+    if gate is not None:
+        _contig("gate", gate)
+        if gate.dtype != torch.float32 or gate.numel() < n * heads * dout:
+            raise KernelError("head_matmul: the gate is float32 [>= n, heads * dout]")
+    call("pyre_head_matmul", x.data_ptr(), x.stride(0), x.stride(1), w.data_ptr(), out.data_ptr(), out.stride(0),
+         out.stride(1), _ptr(gate), dtype_code(x), n, heads, din, dout, _stream())
+
+
+LATENT_MAX_RANK, LATENT_MAX_ROW = 512, 640  #: the longest rows that the kernels take (latent_attention.hip)
+
+
+def _latent_attn_args(q, rows, out, positions, seq_of_token, block_table, heads, rank, dk, page_size, sink):
+    _dev(q, rows, out, positions, seq_of_token, block_table, sink)
+    if not (q.dtype == rows.dtype == out.dtype):
+        raise KernelError("latent attention: one element type for queries, rows and output")
+    if tuple(rows.shape[1:]) != (1, page_size, dk):
+        raise KernelError(f"latent attention: rows {tuple(rows.shape)} do not fit page={page_size} and {dk} elements")
+    if rank > LATENT_MAX_RANK or dk > LATENT_MAX_ROW or not (0 < rank <= dk):
+        raise KernelError(f"latent attention: rows of {dk} elements, {rank} of them values, are more than the kernels take")
+    for t, name in ((q, "q"), (rows, "rows"), (out, "out")):
+        _contig(name, t)
+    _i32("positions", positions), _i32("seq_of_token", seq_of_token), _i32("block_table", block_table)
+    if sink is not None:
+        if sink.dtype != torch.float32 or sink.numel() != heads:
+            raise KernelError("latent attention: the sink is float32 [heads]")
+        _contig("sink", sink)
+
+
+def latent_attn_tile(q, rows, out, tiles, n_tiles, positions, seq_of_token, block_table, heads, rank, dk, page_size, scale,
+                     window=0, sink=None) -> None:
+    """Prompt portions: ``q [N, heads * dk]`` over the tokens' compressed rows ``[pages, 1, page, dk]`` -> ``out [N, heads *
+    rank]``, the softmax-weighted sum of the rows' first ``rank`` elements; scores, weights and sums float32."""
+    _latent_attn_args(q, rows, out, positions, seq_of_token, block_table, heads, rank, dk, page_size, sink)
+    _i32("tiles", tiles, 2 * n_tiles)
+    call("pyre_latent_attn_tile", q.data_ptr(), rows.data_ptr(), out.data_ptr(), dtype_code(q), tiles.data_ptr(), n_tiles,
+         positions.data_ptr(), seq_of_token.data_ptr(), block_table.data_ptr(), block_table.shape[1], heads, rank, dk,
+         page_size, float(scale), int(window), _ptr(sink), _stream())
+
+
+def latent_attn_spans(table_width: int, page_size: int, window: int) -> int:
+    """Spans of keys that a single token of such a launch is dealt in; more than one need scratch."""
+    from pyre_amd.hip.lib import lib
+
+    return lib().pyre_latent_attn_spans(int(table_width * page_size), int(window))
+
+
+def latent_attn_single(q, rows, out, tokens, n, positions, seq_of_token, block_table, heads, rank, dk, page_size, scale,
+                       window=0, sink=None, scratch=None) -> None:
+    """The same for ``n`` single tokens (``tokens``: their rows of the step; None: all rows): 32 heads of a token are a
+    row tile. ``scratch``: float32, n * heads * spans * (rank + 2) elements, where :func:`latent_attn_spans` says more
+    than one span."""
+    _latent_attn_args(q, rows, out, positions, seq_of_token, block_table, heads, rank, dk, page_size, sink)
+    if tokens is not None:
+        _i32("tokens", tokens, n)
+    spans = latent_attn_spans(block_table.shape[1], page_size, window)
+    if spans > 1:
+        if scratch is None or scratch.dtype != torch.float32 or scratch.numel() < n * heads * spans * (rank + 2):
+            raise KernelError(f"latent attention: {spans} spans need {n * heads * spans * (rank + 2)} float32 of scratch")
+        _dev(scratch)
+    call("pyre_latent_attn_single", q.data_ptr(), rows.data_ptr(), out.data_ptr(), dtype_code(q), _ptr(tokens), n,
+         positions.data_ptr(), seq_of_token.data_ptr(), block_table.data_ptr(), block_table.shape[1], heads, rank, dk,
+         page_size, float(scale), int(window), _ptr(sink), _ptr(scratch) if spans > 1 else None, _stream())
+
+
+MAX_STREAMS = 8  #: streams of a residual that the kernel takes (streams.hip)
+
+
+def stream_norm(src: torch.Tensor, dst: torch.Tensor | None, streams: int, delta: Partials | None, mix: torch.Tensor | None,
+                out_w: torch.Tensor | None, in_w: torch.Tensor | None, gain: torch.Tensor, shift: torch.Tensor | None,
+                eps: float, out: torch.Tensor, center: bool = True, rows: torch.Tensor | None = None) -> None:
+    """A residual of ``streams`` streams x [N, streams, H]: ``src`` is float32 [N, streams * H], or [N, H] while all streams
+    are equal. With ``delta``, a sublayer's result y: x_t <- sum_s mix[s, t] x_s + out_w[t] y first, stored to ``dst``
+    if it is given (which may be ``src``). out = norm(sum_s in_w[s] x_s) * gain (+ shift), a layer norm (``center``) or
+    an RMS norm; ``in_w`` None: the plain sum. ``rows``: only these rows, into ``out[0 .. len(rows))``. Weights float32."""
+    _dev(src, dst, mix, out_w, in_w, gain, shift, out, rows)
+    hidden = gain.numel()
+    if not 1 <= streams <= MAX_STREAMS:
+        raise KernelError(f"stream_norm: {streams} streams are outside 1..{MAX_STREAMS}")
+    if src.dtype != torch.float32 or src.dim() != 2 or src.shape[1] not in (hidden, streams * hidden):
+        raise KernelError("stream_norm: the residual is float32 [N, H] or [N, streams * H]")
+    n = src.shape[0] if rows is None else rows.numel()
+    _contig("src", src), _contig("out", out)
+    if out.shape[-1] != hidden or out.shape[0] < n:
+        raise KernelError("stream_norm: out does not fit")
+    for name, t, k in (("gain", gain, hidden), ("shift", shift, hidden), ("mix", mix, streams ** 2), ("out_w", out_w, streams),
+                       ("in_w", in_w, streams)):
+        if t is not None:
+            _contig(name, t)
+            if t.dtype != torch.float32 or t.numel() != k:
+                raise KernelError(f"stream_norm: {name} is float32 with {k} elements")
+    d = (None, 0, 0, 0)
+    if delta is not None:
+        if mix is None or out_w is None:
+            raise KernelError("stream_norm: a result goes back through mix and out_w")
+        if delta.rows < src.shape[0] or delta.width != hidden or delta.bias is not None or delta.post is not None or \
+                delta.scale != 1.0 or delta.more is not None or delta.outer is not None:
+            raise KernelError("stream_norm: a plain result of the residual's size is expected")
+        d = (delta.data.data_ptr(), dtype_code(delta.data), delta.count, delta.stride)
+    if dst is not None:
+        _contig("dst", dst)
+        if dst.dtype != torch.float32 or dst.numel() < src.shape[0] * streams * hidden or rows is not None:
+            raise KernelError("stream_norm: dst is float32 [N, streams * H], and rows are not stored")
+    if rows is not None:
+        _i32("rows", rows)
+    call("pyre_stream_norm", src.data_ptr(), src.shape[1] // hidden, _ptr(dst), streams, *d, _ptr(mix), _ptr(out_w),
+         _ptr(in_w), gain.data_ptr(), _ptr(shift), int(center), float(eps), out.data_ptr(), dtype_code(out), _ptr(rows), n,
+         hidden, _stream())
+
+
+def poly_norm(z: Partials, abce: torch.Tensor, eps: float, out: torch.Tensor, n: int) -> None:
+    """out[n] = a N(z) + b N(z^2) + c N(z^3) + e over the rows of a product (its partial sums added first), powers element
+    by element, N dividing a row by its root mean square; ``abce`` float32 [4]."""
+    _dev(z.data, abce, out)
+    if z.bias is not None or z.rows < n or out.shape[-1] != z.width or out.shape[0] < n:
+        raise KernelError("poly_norm: a product without a bias and an output of its size are expected")
+    if abce.dtype != torch.float32 or abce.numel() != 4:
+        raise KernelError("poly_norm: the coefficients are float32 [4]")
+    _contig("abce", abce), _contig("out", out)
+    call("pyre_poly_norm", z.data.data_ptr(), dtype_code(z.data), z.count, z.stride, abce.data_ptr(), float(eps),
+         out.data_ptr(), dtype_code(out), n, z.width, _stream())
 
 
 ROUTE_MAX_EXPERTS = 512  #: the most experts that the routing kernel chooses among (moe.hip)
@@ -1217,12 +1370,16 @@ def add_rms_terms(resid: torch.Tensor, delta: Partials | None, gain: torch.Tenso
 
 def bigram_embed(table: torch.Tensor, pairs: torch.Tensor, ids: torch.Tensor, positions: torch.Tensor,
                  seq_of_token: torch.Tensor, q_start: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor,
-                 out: torch.Tensor, buckets: int, mul_prev: int, mul_cur: int) -> None:
+                 out: torch.Tensor, buckets: int, mul_prev: int, mul_cur: int, places: torch.Tensor | None = None) -> None:
     """out[n] = float32(table[ids[n]]) + float32(pairs[row]), row = (previous token * mul_prev + ids[n] * mul_cur) mod
-    buckets, or ``buckets`` at position 0. The previous token of a request's first token of the step is
+    buckets, or ``buckets`` at position 0; with ``places`` [rows, H] also + float32(places[positions[n]]). The previous token of a request's first token of the step is
     ``state[slot, 0]`` (float32, an integer value), which then takes the request's last token of the step."""
-    _dev(table, pairs, ids, positions, seq_of_token, q_start, state, state_slots, out)
+    _dev(table, pairs, ids, positions, seq_of_token, q_start, state, state_slots, out, places)
     n, hidden = out.shape
+    if places is not None:
+        if places.dim() != 2 or places.shape[1] != hidden or places.dtype != table.dtype or places.shape[0] < 1:
+            raise KernelError("bigram_embed: the table of positions is [rows, H] of the other tables' type")
+        _contig("places", places)
     if table.dim() != 2 or table.shape[1] != hidden or out.dtype != torch.float32 or table.dtype != pairs.dtype:
         raise KernelError("bigram_embed: tables [V, H] / [buckets + 1, H] of one type and float32 out [N, H] expected")
     if tuple(pairs.shape) != (buckets + 1, hidden) or buckets <= 0 or mul_prev < 0 or mul_cur < 0:
@@ -1233,8 +1390,8 @@ def bigram_embed(table: torch.Tensor, pairs: torch.Tensor, ids: torch.Tensor, po
     _i32("ids", ids, n), _i32("positions", positions, n), _i32("seq_of_token", seq_of_token, n)
     _i32("q_start", q_start), _i32("state_slots", state_slots)
     call("pyre_bigram_embed", table.data_ptr(), pairs.data_ptr(), dtype_code(table), ids.data_ptr(), positions.data_ptr(),
-         seq_of_token.data_ptr(), q_start.data_ptr(), state.data_ptr(), state_slots.data_ptr(), out.data_ptr(), n, hidden,
-         int(buckets), int(mul_prev), int(mul_cur), _stream())
+         seq_of_token.data_ptr(), q_start.data_ptr(), state.data_ptr(), state_slots.data_ptr(), _ptr(places),
+         places.shape[0] if places is not None else 0, out.data_ptr(), n, hidden, int(buckets), int(mul_prev), int(mul_cur), _stream())
 
 
 CONV_MAX_TAPS = 16  #: the most taps of the short convolution (conv_attention.hip)

@@ -340,11 +340,13 @@ class AttentionSpec:
 
 @dataclass(frozen=True)
 class LayerNormSpec:
-    """(x - mean) / sqrt(var + eps) * gain, no bias; ``name`` is the gain's tensor."""
+    """(x - mean) / sqrt(var + eps) * gain; ``name`` is the gain's tensor. ``bias``: the tensor ``name + ".b"`` is
+    added."""
 
     hidden_size: int
     eps: float
     name: str
+    bias: bool = False
     kind: ClassVar[str] = "layernorm"
 
 
@@ -428,8 +430,13 @@ class LatentAttentionSpec:
     """Causal softmax attention whose keys and values of all heads are made of one compressed row per token:
     c = rms_norm(Wdkv h) * gain [rank]; per head k = Wuk c (``key_dim``), v = Wuv c (``value_dim``). Only c is
     kept. ``own_latent`` False: the layer has no Wdkv and reads the rows that another layer keeps (the order of
-    layers names it as the entry whose cache this one reads). Tensors: ``prefix + .q / .dkv / .dkv.norm / .uk /
-    .uv / .o``."""
+    layers names it as the entry whose cache this one reads). Options: ``rot_dim`` > 0: every query head has that many
+    further elements, and Wdkv that many further rows, which make one key part for all heads (not normed, kept beside
+    c); both are turned by position (``position``: either pairing) and their product joins the score. ``q_rank`` > 0:
+    queries are made of a compressed row of their own, Wuq rms_norm(Wdq h). ``window``: only that many last tokens are
+    seen (0: all). ``sink``: exp of a learned number per head joins the softmax's denominator. ``gated``: the heads'
+    outputs are multiplied element by element with sigmoid(G h). Tensors: ``prefix + .q`` (or ``.dq / .dq.norm / .uq``)
+    ``/ .dkv / .dkv.norm / .uk / .uv / .sink / .g / .o``."""
 
     hidden_size: int
     num_heads: int
@@ -440,6 +447,12 @@ class LatentAttentionSpec:
     norm_eps: float
     prefix: str
     own_latent: bool = True
+    rot_dim: int = 0
+    position: Any = None
+    q_rank: int = 0
+    window: int = 0
+    sink: bool = False
+    gated: bool = False
     kind: ClassVar[str] = "latent_attention"
 
 
@@ -522,6 +535,19 @@ class ReluSquaredMLPSpec:
     intermediate_size: int
     prefix: str
     kind: ClassVar[str] = "relu2_mlp"
+
+
+@dataclass(frozen=True)
+class PolyNormMLPSpec:
+    """down(act(up(x))), act(z) = a N(z) + b N(z^2) + c N(z^3) + e with four learned numbers, powers element by element
+    and N dividing a token's row of hidden units by its root mean square. No biases. Tensors: ``prefix + .up / .act /
+    .down``."""
+
+    hidden_size: int
+    intermediate_size: int
+    prefix: str
+    norm_eps: float
+    kind: ClassVar[str] = "poly_norm_mlp"
 
 
 @dataclass(frozen=True)
@@ -727,6 +753,31 @@ class BlockSpec:
 
 
 @dataclass(frozen=True)
+class HyperConnectionSpec:
+    """A sublayer between the streams of a residual: it reads u = sum_s in[s] x_s and its result y goes back to all
+    streams, x_t <- sum_s mix[s, t] x_s + out[t] y. Tensors: ``prefix + .in / .out / .mix``."""
+
+    streams: int
+    prefix: str
+
+
+@dataclass(frozen=True)
+class HyperConnectionBlockSpec:
+    """mixer(norm(u)) and then feed_forward(norm(u)) (None: the first alone), each between the streams through a
+    :class:`HyperConnectionSpec` of its own. The model's ``streams`` says how many there are."""
+
+    mixer: Any
+    mixer_norm: Any
+    mixer_connection: HyperConnectionSpec
+    feed_forward: Any = None
+    feed_forward_norm: Any = None
+    feed_forward_connection: HyperConnectionSpec | None = None
+    #: tensors (name, shape) that a file may hold for this layer though nothing reads them
+    unused: tuple = ()
+    kind: ClassVar[str] = "hyper_connections"
+
+
+@dataclass(frozen=True)
 class EmbeddingSpec:
     vocab_size: int
     hidden_size: int
@@ -738,7 +789,9 @@ class EmbeddingSpec:
 @dataclass(frozen=True)
 class BigramEmbeddingSpec:
     """table[token] + pairs[(previous token * mul_prev + token * mul_cur) mod buckets]; a request's first token
-    takes row ``buckets`` of ``pairs`` (its last). The previous token is state that a request keeps."""
+    takes row ``buckets`` of ``pairs`` (its last). The previous token is state that a request keeps. ``places_name``:
+    a table of ``places`` rows, of which a token's position takes one that is added as well (None: no such table); no
+    request can then be longer than the table."""
 
     vocab_size: int
     hidden_size: int
@@ -747,6 +800,8 @@ class BigramEmbeddingSpec:
     mul_cur: int
     name: str = "embed"
     pairs_name: str = "bigram"
+    places: int = 0
+    places_name: str | None = None
     kind: ClassVar[str] = "bigram_embedding"
 
 
@@ -784,4 +839,7 @@ class ModelSpec:
     schedule: tuple[LayerCall, ...]
     final_norm: Any
     head: Any
+    #: streams of the residual (blocks of hyper-connections); 0: the residual is one row a token. All streams are the
+    #: embedding's output at the start, and the final norm reads their sum
+    streams: int = 0
     extra: dict = field(default_factory=dict, compare=False)

@@ -14,10 +14,14 @@ from pyre_amd.parts.base import (Block, BlockSpec, ParallelBlockSpec, PostNormBl
 @dataclass
 class Hidden:
     """The residual stream (float32 [N, H]) and the term not yet added to it: the
-    next norm adds it in the same kernel that norms the sum."""
+    next norm adds it in the same kernel that norms the sum. A residual of several
+    ``streams`` is [N, streams * H] (or [N, H] while they are all equal), and the pending
+    term goes back to them through ``weights``, the connection of its sublayer."""
 
     resid: torch.Tensor
     pending: Partials | None = None
+    streams: int = 0
+    weights: object = None
 
 
 class PreNormBlock(Block):

@@ -38,25 +38,35 @@ class BigramEmbedding(Part):
             raise ValueError("bigram embedding: more buckets than a 32-bit row number holds")
         if spec.vocab_size >= 1 << 24:
             raise ValueError("bigram embedding: the previous token is kept as a float32, which holds numbers below 2^24")
+        if (spec.places_name is not None) != (spec.places > 0):
+            raise ValueError("bigram embedding: a table of positions needs a name and rows")
         self.spec = spec
-        self.table = self.pairs = None
+        self.table = self.pairs = self.places = None
+
+    @property
+    def max_positions(self) -> int:
+        """Positions that the tables have rows for (0: no such bound); the engine takes no longer request."""
+        return self.spec.places
 
     def cache_specs(self) -> list:
         return [StateCacheSpec((1,), "float32")]
 
     def tensor_specs(self) -> list[TensorSpec]:
         s = self.spec
-        return [TensorSpec(s.name, (s.vocab_size, s.hidden_size)), TensorSpec(s.pairs_name, (s.buckets + 1, s.hidden_size))]
+        specs = [TensorSpec(s.name, (s.vocab_size, s.hidden_size)), TensorSpec(s.pairs_name, (s.buckets + 1, s.hidden_size))]
+        return specs + ([TensorSpec(s.places_name, (s.places, s.hidden_size))] if s.places_name else [])
 
     def bind(self, tensors, runtime) -> None:
         self.table = tensors[self.spec.name].contiguous()
         self.pairs = tensors[self.spec.pairs_name].to(self.table.dtype).contiguous()
+        if self.spec.places_name:
+            self.places = tensors[self.spec.places_name].to(self.table.dtype).contiguous()
 
     def forward(self, ctx, resid: torch.Tensor, caches: list) -> None:
         s = self.spec
         # (p a + t b) mod m = (p (a mod m) + t (b mod m)) mod m: the kernel's 64-bit products hold whatever the multipliers are
         ops.bigram_embed(self.table, self.pairs, ctx.tokens, ctx.positions, ctx.seq_of_token, ctx.q_start,
-                         caches[0].tensor, caches[0].slots, resid, s.buckets, s.mul_prev % s.buckets, s.mul_cur % s.buckets)
+                         caches[0].tensor, caches[0].slots, resid, s.buckets, s.mul_prev % s.buckets, s.mul_cur % s.buckets, self.places)
 
 
 class LMHead(Part):

@@ -93,7 +93,8 @@ LIBRARY_F32_ROLES = frozenset({"attn.qkv", "attn.out", "mix.in", "mix.out", "cat
                                "glu.down", "tattn.qk", "tattn.out", "lattn.in", "lattn.out", "geglu.down", "moe.router",
                                "moe.down", "mix.out0", "mix.out1", "sattn.in", "sattn.out", "ret.in", "ret.out",
                                "relu2.down", "gmoe.router", "gmoe.down", "wattn.in", "wattn.out", "gdr.in", "gdr.out",
-                               "stmoe.router", "stmoe.down", "side.gate", "side.proj"})
+                               "stmoe.router", "stmoe.down", "side.gate", "side.proj", "lattn.q_up", "poly.up",
+                               "poly.down"})
 
 
 def _is_bf16(ctx, lin, x) -> bool:

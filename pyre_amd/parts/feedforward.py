@@ -6,7 +6,8 @@ import torch
 
 from pyre_amd.hip import ops
 from pyre_amd.parts import fast
-from pyre_amd.parts.base import ClippedGLUSpec, FeedForward, GeluGLUSpec, ReluSquaredMLPSpec, SwiGLUSpec, TensorSpec, take
+from pyre_amd.parts.base import (ClippedGLUSpec, FeedForward, GeluGLUSpec, PolyNormMLPSpec, ReluSquaredMLPSpec, SwiGLUSpec,
+                                 TensorSpec, take)
 from pyre_amd.parts.linear import Linear, linear_specs
 
 
@@ -145,4 +146,37 @@ class ReluSquaredMLP(FeedForward):
         n = ctx.n_tokens
         act = ctx.workspace.get("ffn.act", (n, self.spec.intermediate_size), ctx.dtype)
         ops.relu2(self.up.forward(ctx, h, n), act, n)
+        return self.down.forward(ctx, act, n)
+
+
+class PolyNormMLP(FeedForward):
+    """down(a N(z) + b N(z^2) + c N(z^3) + e), z = up(x): a polynomial of the hidden units whose powers are normed over
+    the token's row."""
+
+    def __init__(self, spec: PolyNormMLPSpec):
+        if not spec.norm_eps > 0:
+            raise ValueError("polynomial activation: eps must be positive")
+        self.spec = spec
+        self.up = Linear(spec.hidden_size, spec.intermediate_size, "poly.up")
+        self.down = Linear(spec.intermediate_size, spec.hidden_size, "poly.down")
+        self.coefficients = None
+
+    def tensor_specs(self) -> list[TensorSpec]:
+        s, p = self.spec, self.spec.prefix
+        return [TensorSpec(f"{p}.up", (s.intermediate_size, s.hidden_size)), TensorSpec(f"{p}.act", (4,), init="gain"),
+                TensorSpec(f"{p}.down", (s.hidden_size, s.intermediate_size))]
+
+    def bind(self, tensors, runtime) -> None:
+        p = self.spec.prefix
+        self.up.set(take(tensors, f"{p}.up"))
+        self.down.set(take(tensors, f"{p}.down"))
+        self.coefficients = take(tensors, f"{p}.act").float().contiguous()
+
+    def linears(self) -> list:
+        return [self.up, self.down]
+
+    def forward(self, ctx, h):
+        n = ctx.n_tokens
+        act = ctx.workspace.get("ffn.act", (n, self.spec.intermediate_size), ctx.dtype)
+        ops.poly_norm(self.up.forward(ctx, h, n), self.coefficients, self.spec.norm_eps, act, n)
         return self.down.forward(ctx, act, n)

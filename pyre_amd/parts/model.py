@@ -6,6 +6,7 @@ import torch
 
 from pyre_amd.parts.base import ModelSpec, Part, TensorBag, TensorSpec, make_part
 from pyre_amd.parts.block import Hidden
+from pyre_amd.parts.streams import StreamReader, summed_streams
 
 
 class LayeredModel(Part):
@@ -20,6 +21,11 @@ class LayeredModel(Part):
         self.embedding = make_part("embedding", spec.embedding)
         self.layers = [make_part("block", b) for b in spec.layers]
         self.final_norm = make_part("norm", spec.final_norm)
+        self.final_reader = None  #: with a residual of several streams: reads their sum through the final norm
+        for b in self.layers:
+            if bool(getattr(b, "connections", None)) != bool(spec.streams) or \
+                    any(c.streams != spec.streams for c in getattr(b, "connections", ())):
+                raise ValueError(f"a layer's connections do not fit the model's {spec.streams} streams")
         self.head = make_part("head", spec.head)
         self.schedule = list(spec.schedule)
         for pos, call in enumerate(self.schedule):
@@ -85,6 +91,8 @@ class LayeredModel(Part):
         tensors.clear()
         for p in self.parts():
             p.bind(bag, runtime)
+        if self.spec.streams:
+            self.final_reader = StreamReader(self.final_norm)
 
     def forward(self, ctx, caches: list, tap=None) -> torch.Tensor | None:
         """Run the step's tokens; returns float32 logits [n_logits, vocab] (None if none are wanted).
@@ -97,7 +105,7 @@ class LayeredModel(Part):
             self.embedding.forward(ctx, resid, caches[len(self.schedule)])
         else:
             self.embedding.forward(ctx, resid)
-        state = Hidden(resid)
+        state = Hidden(resid, streams=self.spec.streams)
         for pos, call in enumerate(self.schedule):
             self.layers[call.layer].forward(ctx, state, caches[pos])
             if tap is not None:
@@ -106,12 +114,17 @@ class LayeredModel(Part):
         if m == 0:
             return None
         h = ctx.workspace.get("head.h", (m, self.spec.hidden_size), ctx.dtype)
-        self.final_norm.forward(ctx, state.resid, state.pending, h, rows=ctx.logit_rows)
+        if self.final_reader is not None:
+            self.final_reader.read(ctx, state, h, rows=ctx.logit_rows)
+        else:
+            self.final_norm.forward(ctx, state.resid, state.pending, h, rows=ctx.logit_rows)
         return self.head.forward(ctx, h, m)
 
     def _hidden_rows(self, ctx, state: Hidden) -> torch.Tensor:
         """The residual stream as it stands after a layer, the term that the next norm would add
         included (its partial sums in their order, then the bias)."""
+        if state.streams:
+            return summed_streams(state, ctx.n_tokens)
         rows = state.resid[:ctx.n_tokens].clone()
 
         def normed(term, post):

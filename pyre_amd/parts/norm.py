@@ -30,22 +30,25 @@ class RMSNorm(Norm):
 
 
 class LayerNorm(Norm):
-    """(x - mean) / sqrt(var + eps) * gain without a bias, fused with the residual sum before it. The
+    """(x - mean) / sqrt(var + eps) * gain (+ a bias), fused with the residual sum before it. The
     pending term may carry a norm of its own (``Partials.post``: a sublayer's result that is normed
     and scaled before it is added); the same kernel applies it."""
 
     def __init__(self, spec: LayerNormSpec):
         self.spec = spec
-        self.gain = None
+        self.gain = self.shift = None
 
     def tensor_specs(self) -> list[TensorSpec]:
-        return [TensorSpec(self.spec.name, (self.spec.hidden_size,), init="gain")]
+        n, h = self.spec.name, self.spec.hidden_size
+        return [TensorSpec(n, (h,), init="gain")] + ([TensorSpec(f"{n}.b", (h,))] if self.spec.bias else [])
 
     def bind(self, tensors, runtime) -> None:
         self.gain = tensors[self.spec.name].contiguous()
+        if self.spec.bias:
+            self.shift = tensors[f"{self.spec.name}.b"].to(self.gain.dtype).contiguous()
 
     def forward(self, ctx, resid, delta, out, rows=None) -> None:
-        ops.add_layernorm(resid, delta, self.gain, self.spec.eps, out, rows)
+        ops.add_layernorm(resid, delta, self.gain, self.spec.eps, out, rows, self.shift)
 
 
 class TanhNorm(Norm):

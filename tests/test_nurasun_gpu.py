@@ -428,18 +428,27 @@ def test_routing_tells_experts_apart_whose_scores_round_to_one():
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("n,heads,din,dout", [(1, 3, 7, 19), (37, 5, 40, 24), (70, 2, 136, 300)])
-def test_the_product_per_head(dtype, n, heads, din, dout):
+@pytest.mark.parametrize("gated", [False, True])
+@pytest.mark.parametrize("n,heads,din,dout,wide", [(1, 3, 7, 19, 0), (37, 5, 40, 24, 8), (70, 2, 136, 300, 0), (9, 4, 24, 70, 2),
+                                                   (129, 3, 64, 33, 5), (200, 1, 512, 128, 64), (64, 2, 8, 32, 0), (65, 2, 20, 6, 1)])
+def test_the_product_per_head(dtype, n, heads, din, dout, wide, gated):
+    """Sizes for each form (few and many tokens, units of 16 bytes or not, tiles that are not full), heads of the output
+    further apart than they are wide, with and without a gate per element."""
     from pyre_amd.hip import ops
 
     g = torch.Generator().manual_seed(n)
-    x = torch.randn(n + 2, heads * din + 3, generator=g).to(dtype)
-    w = (torch.randn(heads, din, dout, generator=g) * 0.3).to(dtype)
-    out = torch.zeros(n, heads * dout, device=DEV, dtype=dtype)
-    ops.head_matmul(x.to(DEV), w.to(DEV), out, n)
-    want = torch.einsum("nhi,hio->nho", x[:n, :heads * din].double().view(n, heads, din), w.double()).reshape(n, -1)
+    x = torch.randn(n + 2, heads, din, generator=g).to(dtype)
+    w = (torch.randn(heads, dout, din, generator=g) * 0.3).to(dtype)
+    gate = torch.rand(n, heads * dout, generator=g)
+    out = torch.full((n, heads, dout + wide), 7.0, device=DEV, dtype=dtype)
+    ops.head_matmul(x.to(DEV), w.to(DEV), out, n, gate.to(DEV) if gated else None)
+    want = torch.einsum("nhi,hoi->nho", x[:n].double(), w.double())
+    if gated:
+        want = want * gate.double().view(n, heads, dout)
     tol = 1e-5 if dtype == torch.float32 else 1e-2
-    assert float((out.cpu().double() - want).abs().max()) < tol * float(want.abs().max())
+    got = out.cpu().double()
+    assert float((got[:, :, :dout] - want).abs().max()) < tol * float(want.abs().max())
+    assert bool((got[:, :, dout:] == 7).all())    # what lies between the heads is left alone
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
@@ -476,10 +485,11 @@ def test_what_stands_between_the_input_product_and_attention(dtype):
     gain = (1 + 0.3 * torch.randn(rank, generator=g))
     q2 = torch.zeros(n, qw, device=DEV, dtype=dtype)
     cc = torch.zeros(pages, 1, page, rank, device=DEV, dtype=dtype)
-    ops.latent_write(ops.Partials(parts.to(DEV)), 1, q2, cc, gain.to(dtype).to(DEV), 1e-3, slots.to(DEV), n, qw, rank, page)
+    ops.latent_rows(ops.Partials(parts.to(DEV)), n, rank, 0, dtype, queries=(1, 2, qw // 2, q2, None),
+                    row=(1 + qw, gain.to(DEV), cc, slots.to(DEV)), eps=1e-3)
     total = parts.double().sum(0)[:, 1:]
     assert float((q2.cpu().double() - total[:, :qw]).abs().max()) < tol * scale
-    rows = P.unit_rms(total[:, qw:qw + rank], 1e-3) * gain.to(dtype).double()
+    rows = P.unit_rms(total[:, qw:qw + rank], 1e-3) * gain.double()
     for t, slot in enumerate(slots.tolist()):
         if slot >= 0:
             assert float((cc[slot // page, 0, slot % page].cpu().double() - rows[t]).abs().max()) < tol * float(rows.abs().max())
