@@ -2,7 +2,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--context 4096] [--model qwen2.5-7b]
     python bench.py --workload serve [--model qwen2.5-1.5b] [--requests 256] [--max-batch 256]
-    python bench.py --workload designs [--shapes 1.5b,7b] [--layers 4] [--designs qwen2,mafurax,nurasun,durelix,zorulix]
+    python bench.py --workload designs [--shapes 1.5b,7b] [--layers 4] [--designs qwen2,mafurax,nurasun,durelix,zorulix,rukosun]
 
 A step is one decode step of the scheduler: every running request gets one new
 token (plan, one engine step over the paged cache, greedy sampling, token fed
@@ -41,7 +41,9 @@ the Mafurax design's split of the heads (a window of 1,024 tokens behind a convo
 between down(relu(up)^2) of the same width and a mixture of 8 gated experts of a quarter of it and 4 identity experts),
 and the Zorulix design, whose layers alternate between attention over a window of 1,024 tokens (every second such layer
 reading the keys and values of the one before) and windowed attention beside the gated delta rule at the same split of
-the heads, every layer with the mixture of 8 gated experts and a shared one and with 64 columns of a second token table.
+the heads, every layer with the mixture of 8 gated experts and a shared one and with 64 columns of a second token table,
+and the Rukosun design, whose layers alternate between its two kinds of latent attention (the same heads over rows of
+512 + 64 elements and a window of 1,024 tokens) with a dense feed-forward of the same width and two residual streams.
 For each:
 the prefill of a 2,048-token prompt, decode steps at 8 and 64 requests with contexts of 4,096, and
 the device time of every kernel of a prefill step and of a decode step at 8 requests.
@@ -292,7 +294,17 @@ def designs(args) -> dict:
                 owner = i if owner is None else None
         zorulix = {"architecture": "Zorulix", "vocab": sh["vocab"], "width": sh["width"], "norm": {"eps": 1e-6},
                    "embedding": {"scale": 1.0}, "token_side": {"dim": 64}, "layers": zlayers}
-        made = {"qwen2": qwen, "mafurax": mafurax, "nurasun": nurasun, "durelix": durelix, "zorulix": zorulix}
+        # Rukosun: layers alternate between the two kinds of attention over a compressed row (all heads, of a head's
+        # elements unturned and half as many turned, rows of 512 + 64 elements at heads of 128, a window of 1,024 tokens;
+        # every second layer with queries from a row of three eighths of the width, a sink and an output gate); a dense
+        # feed-forward of the shape's width with the polynomial activation, two streams
+        rrow = {"heads": sh["heads"], "dim": sh["head"], "rot_dim": sh["head"] // 2, "vdim": sh["head"], "kv_rank": 4 * sh["head"],
+                "scale": (1.5 * sh["head"]) ** -0.5, "mask": {"size": 1024}, "rot": {"base": 1e4, "dims": sh["head"] // 2}}
+        rukosun = {"architecture": "Rukosun", "vocab": sh["vocab"], "width": sh["width"], "norm": {"eps": 1e-6}, "streams": 2,
+                   "max_positions": 32768, "embedding": {"bigram": {"buckets": 65521, "mul_prev": 1000003, "mul_cur": 31}},
+                   "layers": [{"type": "latent_attention" if i % 2 else "latent_attention_2", "mlp": {"kind": "dense", "ff": sh["ff"]},
+                               "mixer": dict(rrow, q_rank=3 * sh["width"] // 8) if i % 2 else rrow} for i in range(layers)]}
+        made = {"qwen2": qwen, "mafurax": mafurax, "nurasun": nurasun, "durelix": durelix, "zorulix": zorulix, "rukosun": rukosun}
         return {name: config_from_dict(made[name]) for name in args.designs.split(",") if name}
 
     def kernels_of(run, per: int) -> dict:
@@ -441,8 +453,8 @@ def main() -> int:
     ap.add_argument("--model", default=None, help="preset shape (qwen2.5-7b; for --workload serve qwen2.5-1.5b)")
     ap.add_argument("--workload", default="decode", choices=["decode", "serve", "designs"])
     ap.add_argument("--shapes", default="1.5b,7b", help="designs: the layer sizes to compare at (1.5b, 7b)")
-    ap.add_argument("--designs", default="qwen2,mafurax,nurasun,durelix,zorulix",
-                    help="designs: which of qwen2, mafurax, nurasun, durelix, zorulix to measure")
+    ap.add_argument("--designs", default="qwen2,mafurax,nurasun,durelix,zorulix,rukosun",
+                    help="designs: which of qwen2, mafurax, nurasun, durelix, zorulix, rukosun to measure")
     ap.add_argument("--requests", type=int, default=256, help="serve: number of requests")
     ap.add_argument("--max-batch", type=int, default=256, help="serve: requests that run at a time")
     ap.add_argument("--seed", type=int, default=0, help="serve: seed of the lengths and token ids")
