@@ -295,7 +295,7 @@ struct HeadProduct {
 };
 
 template <typename T>
-__device__ inline f32x16 mfma_unit(uint4 a, uint4 b, f32x16 acc) {
+__device__ __forceinline__ f32x16 mfma_unit(uint4 a, uint4 b, f32x16 acc) {
   if constexpr (sizeof(T) == 2) {
     acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), acc, 0, 0, 0);
   } else {
@@ -307,7 +307,7 @@ __device__ inline f32x16 mfma_unit(uint4 a, uint4 b, f32x16 acc) {
 }
 
 template <typename T>
-__device__ inline void head_store(const HeadProduct& a, int token, int head, int h, int col0, const f32x16& acc) {
+__device__ __forceinline__ void head_store(const HeadProduct& a, int token, int head, int h, int col0, const f32x16& acc) {
   if (token >= a.n) return;
   T* dst = static_cast<T*>(a.out) + token * a.out_token + head * a.out_head;
   const float* gate = a.gate ? a.gate + (static_cast<size_t>(token) * a.heads + head) * a.dout : nullptr;
@@ -329,8 +329,8 @@ __device__ inline void head_store(const HeadProduct& a, int token, int head, int
 
 // On the matrix cores: rows of the tile are columns of the output (W's rows), its columns are tokens, so that a lane
 // holds neighbouring outputs of one token. A lane's operands are 16-byte units of W's rows and of x, straight from
-// memory (both are small and shared by many blocks). FEW: a block is one tile of 32 outputs and 32 tokens whose
-// inner product its four waves share (parts added through LDS, in order); else a wave has R x C such tiles.
+// memory (both are small and shared by many blocks). Few tokens: a block is one tile of 32 outputs and 32 tokens whose
+// inner product its four waves share (parts added through LDS, in order).
 template <typename T>
 __global__ __launch_bounds__(kThreads) void head_matmul_few_kernel(const HeadProduct a) {
   constexpr int E = 16 / sizeof(T);
@@ -371,49 +371,98 @@ __global__ __launch_bounds__(kThreads) void head_matmul_few_kernel(const HeadPro
   head_store<T>(a, token, head, h, col0, acc);
 }
 
-template <typename T>
-__global__ __launch_bounds__(kThreads) void head_matmul_many_kernel(const HeadProduct a) {
-  constexpr int E = 16 / sizeof(T), R = 2, C = 2;  // tiles of outputs, tiles of tokens of a wave
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, h = lane >> 5, c = lane & 31;
-  const int head = blockIdx.y, col0 = blockIdx.z * 64 * R + (wave & 1) * 32 * R, tok0 = blockIdx.x * 64 * C + (wave >> 1) * 32 * C;
-  const int steps = (a.din + 2 * E - 1) / (2 * E);
-  if (col0 >= a.dout || tok0 >= a.n) return;
-  const T* wrow[R];
-  const T* xrow[C];
+// Many tokens (bfloat16): a block has 128 outputs of a head against 128 tokens, a wave 64 x 64 of them; 64 elements of the
+// inner product at a time through two buffers in LDS, the next ones on their way meanwhile. The results go out through
+// LDS as well, so that a token's outputs are stored in whole lines (and its gate is read in such).
+constexpr int kTile = 128, kSlice = 64, kSlicePad = kSlice + 8, kOutPad = kTile + 8;
+__global__ __launch_bounds__(kThreads) void head_matmul_many_kernel(const HeadProduct a, int wide_stores) {
+  __shared__ __attribute__((aligned(16))) bf16 lds[2 * 2 * kTile * kSlicePad];  // [buffer][W rows, tokens][kTile][kSlicePad]
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = lane >> 5, c = lane & 31;
+  const int head = blockIdx.y, col0 = blockIdx.z * kTile, tok0 = blockIdx.x * kTile;
+  const int slices = (a.din + kSlice - 1) / kSlice;
+  // a thread brings 16 bytes of four W rows and of four tokens a slice: rows r, r + 32, ..., the same eight elements of each
+  const int r = tid >> 3, e8 = 8 * (tid & 7);
+  const bf16* w_src = static_cast<const bf16*>(a.w) + static_cast<size_t>(head) * a.dout * a.din + e8;
+  const bf16* x_src = static_cast<const bf16*>(a.x) + head * a.x_head + e8;
+  uint4 w_reg[4], x_reg[4];
+  auto ask = [&](int s) {
+    const bool in = s * kSlice + e8 < a.din;
 #pragma unroll
-  for (int r = 0; r < R; ++r)
-    wrow[r] = static_cast<const T*>(a.w) + (static_cast<size_t>(head) * a.dout + min(col0 + 32 * r + c, a.dout - 1)) * a.din + E * h;
-#pragma unroll
-  for (int t = 0; t < C; ++t) xrow[t] = static_cast<const T*>(a.x) + min(tok0 + 32 * t + c, a.n - 1) * a.x_token + head * a.x_head + E * h;
-  f32x16 acc[R][C];
-#pragma unroll
-  for (int r = 0; r < R; ++r)
-#pragma unroll
-    for (int t = 0; t < C; ++t)
-#pragma unroll
-      for (int i = 0; i < 16; ++i) acc[r][t][i] = 0.f;
-  const uint4 zero = {0u, 0u, 0u, 0u};
-  for (int s = 0; s < steps; s += 2) {
-    uint4 wv[2][R], xv[2][C];
-#pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      const bool in = 2 * E * (s + u) + E * h < a.din;
-#pragma unroll
-      for (int r = 0; r < R; ++r) wv[u][r] = in ? *reinterpret_cast<const uint4*>(wrow[r] + 2 * E * (s + u)) : zero;
-#pragma unroll
-      for (int t = 0; t < C; ++t) xv[u][t] = in ? *reinterpret_cast<const uint4*>(xrow[t] + 2 * E * (s + u)) : zero;
+    for (int k = 0; k < 4; ++k) {
+      w_reg[k] = x_reg[k] = uint4{0u, 0u, 0u, 0u};
+      if (!in) continue;
+      w_reg[k] = *reinterpret_cast<const uint4*>(w_src + static_cast<size_t>(min(col0 + r + 32 * k, a.dout - 1)) * a.din + s * kSlice);
+      x_reg[k] = *reinterpret_cast<const uint4*>(x_src + min(tok0 + r + 32 * k, a.n - 1) * a.x_token + s * kSlice);
     }
+  };
+  auto stash = [&](int s) {
+    bf16* dst = lds + (s & 1) * 2 * kTile * kSlicePad + r * kSlicePad + e8;
 #pragma unroll
-    for (int u = 0; u < 2; ++u)
+    for (int k = 0; k < 4; ++k) {
+      *reinterpret_cast<uint4*>(dst + 32 * k * kSlicePad) = w_reg[k];
+      *reinterpret_cast<uint4*>(dst + (kTile + 32 * k) * kSlicePad) = x_reg[k];
+    }
+  };
+  f32x16 acc[2][2];
 #pragma unroll
-      for (int r = 0; r < R; ++r)
+  for (int i = 0; i < 2; ++i)
 #pragma unroll
-        for (int t = 0; t < C; ++t) acc[r][t] = mfma_unit<T>(wv[u][r], xv[u][t], acc[r][t]);
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+      for (int u = 0; u < 16; ++u) acc[i][t][u] = 0.f;
+  const int wr = 64 * (wave & 1), wt = 64 * (wave >> 1);
+  ask(0);
+  stash(0);
+  __syncthreads();
+  for (int s = 0; s < slices; ++s) {
+    if (s + 1 < slices) ask(s + 1);
+    const bf16* ws = lds + (s & 1) * 2 * kTile * kSlicePad + (wr + c) * kSlicePad + 8 * h;
+    const bf16* xs = lds + (s & 1) * 2 * kTile * kSlicePad + (kTile + wt + c) * kSlicePad + 8 * h;
+#pragma unroll
+    for (int e = 0; e < kSlice; e += 16) {
+      uint4 wv[2], xv[2];
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        wv[i] = *reinterpret_cast<const uint4*>(ws + 32 * i * kSlicePad + e);
+        xv[i] = *reinterpret_cast<const uint4*>(xs + 32 * i * kSlicePad + e);
+      }
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int t = 0; t < 2; ++t) acc[i][t] = mfma_unit<bf16>(wv[i], xv[t], acc[i][t]);
+    }
+    if (s + 1 < slices) stash(s + 1);  // into the buffer whose readers passed the barrier before
+    __syncthreads();
   }
+  if (!wide_stores) {
 #pragma unroll
-  for (int t = 0; t < C; ++t)
+    for (int t = 0; t < 2; ++t)
 #pragma unroll
-    for (int r = 0; r < R; ++r) head_store<T>(a, tok0 + 32 * t + c, head, h, col0 + 32 * r, acc[r][t]);
+      for (int i = 0; i < 2; ++i) head_store<bf16>(a, tok0 + wt + 32 * t + c, head, h, col0 + wr + 32 * i, acc[i][t]);
+    return;
+  }
+  bf16* rows = lds;  // [kTile tokens][kOutPad]
+#pragma unroll
+  for (int t = 0; t < 2; ++t)
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int t_in = wt + 32 * t + c, d_in = wr + 32 * i + 8 * j + 4 * h;
+        float4 v = {acc[i][t][4 * j], acc[i][t][4 * j + 1], acc[i][t][4 * j + 2], acc[i][t][4 * j + 3]};
+        if (a.gate && tok0 + t_in < a.n && col0 + d_in < a.dout) {
+          const float4 gv = Vec4<float>::load(a.gate + (static_cast<size_t>(tok0 + t_in) * a.heads + head) * a.dout + col0 + d_in);
+          v = float4{v.x * gv.x, v.y * gv.y, v.z * gv.z, v.w * gv.w};
+        }
+        Vec4<bf16>::store(rows + t_in * kOutPad + d_in, v);
+      }
+  __syncthreads();
+  for (int k = tid; k < kTile * (kTile / 8); k += kThreads) {
+    const int t = k / (kTile / 8), d = 8 * (k % (kTile / 8));
+    if (tok0 + t < a.n && col0 + d < a.dout)
+      *reinterpret_cast<uint4*>(static_cast<bf16*>(a.out) + (tok0 + t) * a.out_token + head * a.out_head + col0 + d) =
+          *reinterpret_cast<const uint4*>(rows + t * kOutPad + d);
+  }
 }
 
 // Any sizes: a thread an output.
@@ -514,7 +563,9 @@ extern "C" int pyre_head_matmul(const void* x, long x_token, long x_head, const 
     if (n <= 64 || dt == kF32)
       PYRE_DISPATCH(dt, T, hipLaunchKernelGGL(head_matmul_few_kernel<T>, dim3((n + 31) / 32, heads, (dout + 31) / 32), dim3(kThreads), 0, stream, a));
     else
-      hipLaunchKernelGGL(head_matmul_many_kernel<bf16>, dim3((n + 127) / 128, heads, (dout + 127) / 128), dim3(kThreads), 0, stream, a);
+      hipLaunchKernelGGL(head_matmul_many_kernel, dim3((n + kTile - 1) / kTile, heads, (dout + kTile - 1) / kTile), dim3(kThreads), 0,
+                         stream, a, dout % 8 == 0 && out_token % 8 == 0 && out_head % 8 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0 &&
+                             reinterpret_cast<uintptr_t>(gate) % 16 == 0);
     return check_launch("head_matmul");
   }
   PYRE_DISPATCH(dt, T, hipLaunchKernelGGL(head_matmul_any_kernel<T>, dim3(n, heads, (dout + kThreads - 1) / kThreads), dim3(kThreads), 0, stream, a));

@@ -41,7 +41,8 @@ struct LatentArgs {
   const void* q;            // [n][heads][dk]
   const void* rows;         // [pages][1][page][dk]
   void* out;                // [n][heads][rank]
-  float* part;              // single tokens, several spans: [listed][heads][spans][rank + 2], else null
+  float* part;              // single tokens, several spans: sums [listed][heads][spans][rank], else null
+  float* part_ml;           // and behind them maximum and weight [listed][heads][spans][2]
   const int* list;          // tiles (first token, count), or single tokens (null: token = block)
   const int* positions;
   const int* seq_of_token;
@@ -310,15 +311,22 @@ __global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentAr
   l += __shfl_xor(l, 32, 64);
   if (!live) return;
   if (SINGLE && a.part) {
-    float* dst = a.part + ((static_cast<size_t>(blockIdx.x) * a.heads + head) * a.spans + blockIdx.z) * (a.rank + 2);
+    const size_t at = (static_cast<size_t>(blockIdx.x) * a.heads + head) * a.spans + blockIdx.z;
+    float* dst = a.part + at * a.rank;
 #pragma unroll
     for (int dt = 0; dt < NVT; ++dt)
 #pragma unroll
-      for (int i = 0; i < 16; ++i) {
-        const int d = 32 * (sl * NVT + dt) + 8 * (i >> 2) + 4 * h + (i & 3);
-        if (d < a.rank) dst[d] = o[dt][i];
+      for (int j = 0; j < 4; ++j) {
+        const int d = 32 * (sl * NVT + dt) + 8 * j + 4 * h;
+        if (a.rank % 4 == 0) {
+          if (d < a.rank) *reinterpret_cast<f32x4*>(dst + d) = f32x4{o[dt][4 * j], o[dt][4 * j + 1], o[dt][4 * j + 2], o[dt][4 * j + 3]};
+        } else {
+#pragma unroll
+          for (int u = 0; u < 4; ++u)
+            if (d + u < a.rank) dst[d + u] = o[dt][4 * j + u];
+        }
       }
-    if (sl == 0 && h == 0) dst[a.rank] = m, dst[a.rank + 1] = l;
+    if (sl == 0 && h == 0) a.part_ml[2 * at] = m, a.part_ml[2 * at + 1] = l;
     return;
   }
   const float f = latent_factor(m, l, a.sink, head);
@@ -338,27 +346,60 @@ __global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentAr
     }
 }
 
-// The spans of a single token joined, in their order, with the sink.
-template <typename T>
-__global__ __launch_bounds__(256) void latent_join_kernel(const LatentArgs a) {
-  const int n = a.list ? a.list[blockIdx.x] : blockIdx.x, head = blockIdx.y;
+// The spans of a single token joined, in their order, with the sink: a block per token and head. The spans' factors are
+// formed once, into LDS, up to kJoin of them at a time; W elements a thread, eight spans' sums asked for together.
+constexpr int kJoin = 256;
+template <typename T, int W>
+__global__ __launch_bounds__(kJoin) void latent_join_kernel(const LatentArgs a) {
+  __shared__ float scratch[16], factor_s[kJoin];
+  const int n = a.list ? a.list[blockIdx.x] : blockIdx.x, head = blockIdx.y, tid = threadIdx.x;
   const int pos = a.positions[n], lo = a.window > 0 ? max(0, pos - a.window + 1) : 0;
-  const int count = min(a.spans, pos / a.span - lo / a.span + 1), width = a.rank + 2;
-  const float* src = a.part + (static_cast<size_t>(blockIdx.x) * a.heads + head) * a.spans * width;
-  float M = a.sink ? a.sink[head] * kLog2e : -INFINITY;
-  for (int s = 0; s < count; ++s) M = fmaxf(M, src[s * width + a.rank]);
+  const int count = min(a.spans, pos / a.span - lo / a.span + 1);
+  const size_t at = (static_cast<size_t>(blockIdx.x) * a.heads + head) * a.spans;
+  const float* ml = a.part_ml + 2 * at;
+  const float sink = a.sink ? a.sink[head] * kLog2e : -INFINITY;
+  float M = sink;
+  for (int s = tid; s < count; s += kJoin) M = fmaxf(M, ml[2 * s]);
+  M = block_max(M, scratch);
   const float m_use = M == -INFINITY ? 0.f : M;
-  T* dst = static_cast<T*>(a.out) + (static_cast<size_t>(n) * a.heads + head) * a.rank;
-  for (int d = threadIdx.x; d < a.rank; d += 256) {
-    float total = 0.f, l = 0.f;
-    for (int s = 0; s < count; ++s) {
-      const float w = exp2_hw(src[s * width + a.rank] - m_use);
-      total = fmaf(src[s * width + d], w, total);
-      l = fmaf(src[s * width + a.rank + 1], w, l);
+  float total[W], l = 0.f;
+  const int d = W * tid;
+  static_assert(W * kJoin >= 512, "a thread has all its elements at once");
+#pragma unroll
+  for (int e = 0; e < W; ++e) total[e] = 0.f;
+  for (int s0 = 0; s0 < count; s0 += kJoin) {
+    const int here = min(kJoin, count - s0);
+    __syncthreads();
+    float w = 0.f;
+    if (tid < here) {
+      w = exp2_hw(ml[2 * (s0 + tid)] - m_use);
+      l = fmaf(ml[2 * (s0 + tid) + 1], w, l);
     }
-    if (a.sink) l += exp2_hw(a.sink[head] * kLog2e - m_use);
-    dst[d] = from_float<T>(l > 0.f ? total / l : 0.f);
+    factor_s[tid] = w;
+    __syncthreads();
+    if (d < a.rank) {
+      const float* src = a.part + (at + s0) * a.rank + d;
+      for (int s = 0; s < here; s += 8) {
+        float v[8][W];
+#pragma unroll
+        for (int u = 0; u < 8; ++u)
+#pragma unroll
+          for (int e = 0; e < W; ++e) v[u][e] = s + u < here && d + e < a.rank ? src[static_cast<size_t>(s + u) * a.rank + e] : 0.f;
+#pragma unroll
+        for (int u = 0; u < 8; ++u)
+#pragma unroll
+          for (int e = 0; e < W; ++e) total[e] = fmaf(v[u][e], factor_s[min(s + u, kJoin - 1)], total[e]);
+      }
+    }
   }
+  l = block_sum(l, scratch);
+  if (a.sink) l += exp2_hw(sink - m_use);
+  if (d >= a.rank) return;
+  T* dst = static_cast<T*>(a.out) + (static_cast<size_t>(n) * a.heads + head) * a.rank + d;
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+#pragma unroll
+  for (int e = 0; e < W; ++e)
+    if (d + e < a.rank) dst[e] = from_float<T>(total[e] * inv);
 }
 
 constexpr int kMaxRank = 512, kMaxRow = 640;
@@ -456,9 +497,10 @@ extern "C" int pyre_latent_attn_single(const void* q, const void* rows, void* ou
   a.vec = aligned_rows(a, dt);
   a.span = span_of(window);
   a.spans = pyre_latent_attn_spans(table_stride * page_size, window);
-  PYRE_REQUIRE(a.spans == 1 || part, "latent_attn_single: %d spans need scratch", a.spans);
+  PYRE_REQUIRE(a.spans == 1 || (part && reinterpret_cast<uintptr_t>(part) % 16 == 0), "latent_attn_single: %d spans need scratch", a.spans);
   PYRE_REQUIRE(a.spans <= 65535, "latent_attn_single: %d spans are not a launch", a.spans);
   a.part = a.span ? part : nullptr;
+  a.part_ml = a.part ? part + static_cast<size_t>(n) * heads * a.spans * rank : nullptr;
   if (a.span == 0) a.spans = 1;
   int bad;
   if (rank <= 128)
@@ -472,6 +514,6 @@ extern "C" int pyre_latent_attn_single(const void* q, const void* rows, void* ou
                       : launch<float, 1, 4, 4, 20, true>("latent_attn_single", a, n, a.spans, stream);
   if (bad) return bad;
   if (a.part)
-    PYRE_DISPATCH(dt, T, hipLaunchKernelGGL(latent_join_kernel<T>, dim3(n, heads), dim3(256), 0, stream, a));
+    PYRE_DISPATCH(dt, T, hipLaunchKernelGGL((latent_join_kernel<T, 2>), dim3(n, heads), dim3(kJoin), 0, stream, a));
   return check_launch("latent_attn_single");
 }

@@ -430,7 +430,7 @@ def test_routing_tells_experts_apart_whose_scores_round_to_one():
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("gated", [False, True])
 @pytest.mark.parametrize("n,heads,din,dout,wide", [(1, 3, 7, 19, 0), (37, 5, 40, 24, 8), (70, 2, 136, 300, 0), (9, 4, 24, 70, 2),
-                                                   (129, 3, 64, 33, 5), (200, 1, 512, 128, 64), (64, 2, 8, 32, 0), (65, 2, 20, 6, 1)])
+                                                   (129, 3, 64, 33, 5), (200, 1, 512, 128, 64), (300, 2, 136, 264, 8), (66, 3, 24, 40, 16), (64, 2, 8, 32, 0), (65, 2, 20, 6, 1)])
 def test_the_product_per_head(dtype, n, heads, din, dout, wide, gated):
     """Sizes for each form (few and many tokens, units of 16 bytes or not, tiles that are not full), heads of the output
     further apart than they are wide, with and without a gate per element."""
