@@ -113,6 +113,7 @@ __global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentAr
     if (lo_all > hi_all) return;
   }
   const int chunk0 = lo_all / kKeys, n_chunks = hi_all / kKeys - chunk0 + 1;
+  const int last_tile = (a.rank - 1) / 32;
   const int lo_last = first_seen(hi_tile);  // a chunk from here to pos0 is seen whole by every query
 
   const int entry0 = lo_all / a.page_size;
@@ -204,20 +205,33 @@ __global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentAr
 #pragma unroll
     for (int i = 0; i < 16; ++i) s[i] = 0.f;
     if (active) {
+      // four steps' keys at a time, in two chains of sums; steps behind the row's last one meet a query of zeros
       const T* krow = K + c * ldk + E * h;
+      f32x16 s2;
 #pragma unroll
-      for (int st = 0; st < KQ; ++st) {
-        const int step = st * SL + sl;
-        if (step >= steps) continue;
-        const uint4 k4 = *reinterpret_cast<const uint4*>(krow + 2 * E * step);
-        if constexpr (sizeof(T) == 2) {
-          s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, k4), __builtin_bit_cast(bf16x8, qf[st]), s, 0, 0, 0);
-        } else {
-          const f32x4 kf = __builtin_bit_cast(f32x4, k4), qq = __builtin_bit_cast(f32x4, qf[st]);
+      for (int i = 0; i < 16; ++i) s2[i] = 0.f;
 #pragma unroll
-          for (int u = 0; u < 4; ++u) s = __builtin_amdgcn_mfma_f32_32x32x2f32(kf[u], qq[u], s, 0, 0, 0);
-        }
+      for (int st0 = 0; st0 < KQ; st0 += 4) {
+        if (st0 * SL + sl >= steps) continue;
+        uint4 k4[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          if (st0 + u < KQ) k4[u] = *reinterpret_cast<const uint4*>(krow + 2 * E * min((st0 + u) * SL + sl, steps - 1));
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          if (st0 + u < KQ) {
+            f32x16& sum = u & 1 ? s2 : s;
+            if constexpr (sizeof(T) == 2) {
+              sum = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, k4[u]), __builtin_bit_cast(bf16x8, qf[st0 + u]), sum, 0, 0, 0);
+            } else {
+              const f32x4 kf = __builtin_bit_cast(f32x4, k4[u]), qq = __builtin_bit_cast(f32x4, qf[st0 + u]);
+#pragma unroll
+              for (int v = 0; v < 4; ++v) sum = __builtin_amdgcn_mfma_f32_32x32x2f32(kf[v], qq[v], sum, 0, 0, 0);
+            }
+          }
       }
+#pragma unroll
+      for (int i = 0; i < 16; ++i) s[i] += s2[i];
       if (SL > 1) {
         float* mine = sred + wave * 1024 + 4 * lane;
 #pragma unroll
@@ -280,26 +294,35 @@ __global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentAr
           const bf16x8 p2 = __builtin_bit_cast(bf16x8, uint4{w2[0], w2[1], w2[2], w2[3]});
           const bf16x8 p3 = __builtin_bit_cast(bf16x8, uint4{w3[0], w3[1], w3[2], w3[3]});
           const bf16* vrow = reinterpret_cast<const bf16*>(K) + (16 * b + 4 * h + (j16 >> 2)) * ldk + col16 + 4 * (j16 & 3);
+          // all columns' values first, then the pieces in turn, the smallest first: neighbouring products add to
+          // different sums (columns behind the last tile repeat it, and nobody reads their sums)
+          bf16x8 v8[NVT];
 #pragma unroll
           for (int dt = 0; dt < NVT; ++dt) {
-            const int d0 = 32 * (sl * NVT + dt);
-            if (d0 >= a.rank) continue;
+            const int d0 = 32 * min(sl * NVT + dt, last_tile);
             const uint2 v0 = read_transposed(vrow + d0), v1 = read_transposed(vrow + 8 * ldk + d0);
-            const bf16x8 v8 = __builtin_bit_cast(bf16x8, uint4{v0.x, v0.y, v1.x, v1.y});
-            o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8, p3, o[dt], 0, 0, 0);  // the smallest pieces first
-            o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8, p2, o[dt], 0, 0, 0);
-            o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8, p1, o[dt], 0, 0, 0);
+            v8[dt] = __builtin_bit_cast(bf16x8, uint4{v0.x, v0.y, v1.x, v1.y});
           }
+#pragma unroll
+          for (int dt = 0; dt < NVT; ++dt) o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8[dt], p3, o[dt], 0, 0, 0);
+#pragma unroll
+          for (int dt = 0; dt < NVT; ++dt) o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8[dt], p2, o[dt], 0, 0, 0);
+#pragma unroll
+          for (int dt = 0; dt < NVT; ++dt) o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8[dt], p1, o[dt], 0, 0, 0);
         }
       } else {
+        const float* v = reinterpret_cast<const float*>(K) + 4 * h * ldk + c;
 #pragma unroll
-        for (int dt = 0; dt < NVT; ++dt) {
-          const int d0 = 32 * (sl * NVT + dt);
-          if (d0 >= a.rank) continue;
-          const float* v = reinterpret_cast<const float*>(K) + 4 * h * ldk + d0 + c;
+        for (int i0 = 0; i0 < 16; i0 += 4) {
+          float vv[4][NVT];
 #pragma unroll
-          for (int i = 0; i < 16; ++i)
-            o[dt] = __builtin_amdgcn_mfma_f32_32x32x2f32(v[(8 * (i >> 2) + (i & 3)) * ldk], s[i], o[dt], 0, 0, 0);
+          for (int u = 0; u < 4; ++u)
+#pragma unroll
+            for (int dt = 0; dt < NVT; ++dt) vv[u][dt] = v[(2 * i0 + u) * ldk + 32 * min(sl * NVT + dt, last_tile)];
+#pragma unroll
+          for (int u = 0; u < 4; ++u)
+#pragma unroll
+            for (int dt = 0; dt < NVT; ++dt) o[dt] = __builtin_amdgcn_mfma_f32_32x32x2f32(vv[u][dt], s[i0 + u], o[dt], 0, 0, 0);
         }
       }
     }
