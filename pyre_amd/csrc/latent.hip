@@ -333,7 +333,7 @@ __device__ __forceinline__ void head_store(const HeadProduct& a, int token, int 
 // inner product its four waves share (parts added through LDS, in order).
 template <typename T>
 __global__ __launch_bounds__(kThreads) void head_matmul_few_kernel(const HeadProduct a) {
-  constexpr int E = 16 / sizeof(T);
+  constexpr int E = 16 / sizeof(T), kAhead = 8;
   __shared__ __attribute__((aligned(16))) float parts[3][4][64][4];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, h = lane >> 5, c = lane & 31;
   const int head = blockIdx.y, col0 = blockIdx.z * 32, token = blockIdx.x * 32 + c;
@@ -343,17 +343,18 @@ __global__ __launch_bounds__(kThreads) void head_matmul_few_kernel(const HeadPro
   f32x16 acc;
 #pragma unroll
   for (int i = 0; i < 16; ++i) acc[i] = 0.f;
-  const uint4 zero = {0u, 0u, 0u, 0u};
-  for (int s = s0; s < s1; s += 4) {
-    uint4 wv[4], xv[4];
+  for (int s = s0; s < s1; s += kAhead) {  // so many steps' operands on their way together
+    uint4 wv[kAhead], xv[kAhead];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
+    for (int u = 0; u < kAhead; ++u) {
       const bool in = s + u < s1 && 2 * E * (s + u) + E * h < a.din;
-      wv[u] = in ? *reinterpret_cast<const uint4*>(wrow + 2 * E * (s + u)) : zero;
-      xv[u] = in ? *reinterpret_cast<const uint4*>(xrow + 2 * E * (s + u)) : zero;
+      wv[u] = xv[u] = uint4{0u, 0u, 0u, 0u};
+      if (!in) continue;
+      wv[u] = *reinterpret_cast<const uint4*>(wrow + 2 * E * (s + u));
+      xv[u] = *reinterpret_cast<const uint4*>(xrow + 2 * E * (s + u));
     }
 #pragma unroll
-    for (int u = 0; u < 4; ++u) acc = mfma_unit<T>(wv[u], xv[u], acc);
+    for (int u = 0; u < kAhead; ++u) acc = mfma_unit<T>(wv[u], xv[u], acc);
   }
   if (wave > 0)
 #pragma unroll

@@ -65,6 +65,18 @@ __device__ inline float latent_factor(float m, float l, const float* sink, int h
   return a / (l * a + exp2_hw(sk - M));
 }
 
+// A chunk's weights of one row tile on their way to the waves that share it: three bfloat16 pieces of 32 x 32 weights, in
+// the order of the second product's operands, or the weights themselves.
+template <typename T> constexpr int weight_bytes() { return sizeof(T) == 2 ? 3 * 2048 : 4096; }
+
+// Two weights as three bfloat16 pieces each, which sum to them exactly.
+__device__ inline void split_pair(float p0, float p1, uint32_t& w1, uint32_t& w2, uint32_t& w3) {
+  w1 = pack_bf16x2(p0, p1);
+  const float r0 = p0 - __uint_as_float(w1 << 16), r1 = p1 - __uint_as_float(w1 & 0xffff0000u);
+  w2 = pack_bf16x2(r0, r1);
+  w3 = pack_bf16x2(r0 - __uint_as_float(w2 << 16), r1 - __uint_as_float(w2 & 0xffff0000u));
+}
+
 // Four keys of sixteen neighbouring columns, transposed on the way out of LDS: of each group of sixteen lanes, lane j
 // gives the address of four columns 4 (j % 4) .. of key j / 4 and receives column j of the four keys.
 __device__ inline uint2 read_transposed(const bf16* p) {
@@ -74,7 +86,7 @@ __device__ inline uint2 read_transposed(const bf16* p) {
 }
 
 template <typename T, int G, int SL, int NVT, int KQ, bool SINGLE>
-__global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentArgs a) {
+__global__ __launch_bounds__(64 * G * SL, sizeof(T) == 2 && !SINGLE ? 2 : 1) void latent_attn_kernel(const LatentArgs a) {
   constexpr int NT = 64 * G * SL, TPR = NT / kKeys;     // threads that bring one key's row
   constexpr int E = 16 / sizeof(T);                      // elements of a 16-byte unit
   constexpr int KI = (2 * KQ * SL + TPR - 1) / TPR;      // units a thread brings of a row
@@ -84,8 +96,10 @@ __global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentAr
   const int buffer = kKeys * ldk, slack = max(0, 32 * NVT * SL - ldk);
   const int k_elems = ((a.two_buffers ? 2 : 1) * buffer + slack + 7) / 8 * 8;
   float* sred = reinterpret_cast<float*>(Ks + k_elems);                    // [G * SL][16][64] if SL > 1
-  int* tab_s = reinterpret_cast<int*>(sred + (SL > 1 ? G * SL * 1024 : 0));
+  unsigned char* Ps = reinterpret_cast<unsigned char*>(sred + (SL > 1 ? G * SL * 1024 : 0));  // [G] x weight_bytes<T>() if SL > 1
+  int* tab_s = reinterpret_cast<int*>(Ps + (SL > 1 ? G * weight_bytes<T>() : 0));
   __shared__ int slot_s[kRing][kKeys];
+  __shared__ float row_s[SL > 1 ? G * SL : 1][32];  // the waves' maxima of their keys, per query; at the end their weights
 
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = lane >> 5, c = lane & 31;
   const int g = wave / SL, sl = wave % SL;
@@ -93,13 +107,13 @@ __global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentAr
   if (SINGLE) {
     t0 = a.list ? a.list[blockIdx.x] : blockIdx.x;
   } else {
-    t0 = a.list[2 * blockIdx.x], ntok = a.list[2 * blockIdx.x + 1];
+    t0 = a.list[2 * blockIdx.y], ntok = a.list[2 * blockIdx.y + 1];
     if (ntok <= 0) return;
   }
   const int pos0 = a.positions[t0];
   const int* table = a.table + static_cast<size_t>(a.seq_of_token[t0]) * a.table_stride;
   // this lane's query
-  const int head = SINGLE ? (blockIdx.y * G + g) * 32 + c : blockIdx.y * G + g;
+  const int head = SINGLE ? (blockIdx.y * G + g) * 32 + c : blockIdx.x * G + g;
   const int token = SINGLE ? t0 : t0 + c;
   const bool active = SINGLE ? (blockIdx.y * G + g) * 32 < a.heads : head < a.heads;  // the whole row tile
   const bool live = active && (SINGLE ? head < a.heads : c < ntok);
@@ -238,40 +252,88 @@ __global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentAr
         for (int j = 0; j < 4; ++j) *reinterpret_cast<f32x4*>(mine + 256 * j) = f32x4{s[4 * j], s[4 * j + 1], s[4 * j + 2], s[4 * j + 3]};
       }
     }
+    // Element i of s: key key0 + 8 (i / 4) + 4 h + i % 4, query c. Of SL waves each turns 16 / SL of them into weights:
+    // the parts of its own ones are added up (in order), the maxima and then the weights go round through LDS.
+    constexpr int EW = 16 / SL;
     if (SL > 1) lds_barrier();
+    float w[EW], mx = -INFINITY;
     if (active) {
       if (SL > 1) {
-        const float* base = sred + g * SL * 1024 + 4 * lane;
+        const float* base = sred + g * SL * 1024 + 4 * lane + 256 * (EW / 4) * sl;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
+        for (int j = 0; j < EW / 4; ++j) {
           f32x4 t = *reinterpret_cast<const f32x4*>(base + 256 * j);
 #pragma unroll
-          for (int w = 1; w < SL; ++w) t += *reinterpret_cast<const f32x4*>(base + 1024 * w + 256 * j);
+          for (int o2 = 1; o2 < SL; ++o2) t += *reinterpret_cast<const f32x4*>(base + 1024 * o2 + 256 * j);
 #pragma unroll
-          for (int u = 0; u < 4; ++u) s[4 * j + u] = t[u];
+          for (int u = 0; u < 4; ++u) w[4 * j + u] = t[u];
         }
+      } else {
+#pragma unroll
+        for (int i = 0; i < EW; ++i) w[i] = s[i];
       }
-      // element i of s: key key0 + 8 (i / 4) + 4 h + i % 4, query c
-      float mx = -INFINITY;
       if (key0 >= lo_last && key0 + kKeys - 1 <= pos0) {
 #pragma unroll
-        for (int i = 0; i < 16; ++i) s[i] *= a.scale2, mx = fmaxf(mx, s[i]);
+        for (int i = 0; i < EW; ++i) w[i] *= a.scale2, mx = fmaxf(mx, w[i]);
       } else {
-        const unsigned seen = static_cast<unsigned>(hi - lo), first = static_cast<unsigned>(key0 + 4 * h - lo);
+        const unsigned seen = static_cast<unsigned>(hi - lo), first = static_cast<unsigned>(key0 + 8 * (EW / 4) * sl * (SL > 1) + 4 * h - lo);
 #pragma unroll
-        for (int i = 0; i < 16; ++i) {
-          s[i] = first + 8 * (i >> 2) + (i & 3) <= seen ? s[i] * a.scale2 : -INFINITY;
-          mx = fmaxf(mx, s[i]);
+        for (int i = 0; i < EW; ++i) {
+          w[i] = first + 8 * (i >> 2) + (i & 3) <= seen ? w[i] * a.scale2 : -INFINITY;
+          mx = fmaxf(mx, w[i]);
         }
       }
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      if (SL > 1 && h == 0) row_s[wave % (SL > 1 ? G * SL : 1)][c] = mx;
+    }
+    if (SL > 1) lds_barrier();
+    float alpha = 1.f;
+    uint4 pieces[3][2];
+    if (active) {
+      if (SL > 1)
+#pragma unroll
+        for (int o2 = 0; o2 < SL; ++o2) mx = fmaxf(mx, row_s[SL > 1 ? g * SL + o2 : 0][c]);
       const float m_new = fmaxf(m, mx), m_use = m_new == -INFINITY ? 0.f : m_new;
-      const float alpha = exp2_hw(m - m_use);
+      alpha = exp2_hw(m - m_use);
       m = m_new;
       float sum = 0.f;
 #pragma unroll
-      for (int i = 0; i < 16; ++i) s[i] = exp2_hw(s[i] - m_use), sum += s[i];
+      for (int i = 0; i < EW; ++i) w[i] = exp2_hw(w[i] - m_use), sum += w[i];
       l = l * alpha + sum;
+      if constexpr (sizeof(T) == 2) {
+        // piece pc of keys 16 b .. 16 b + 15: the lane's eight are those of elements 8 b .. 8 b + 7
+        uint32_t w1[EW / 2], w2[EW / 2], w3[EW / 2];
+#pragma unroll
+        for (int u = 0; u < EW / 2; ++u) split_pair(w[2 * u], w[2 * u + 1], w1[u], w2[u], w3[u]);
+        if constexpr (SL == 1) {
+#pragma unroll
+          for (int b = 0; b < 2; ++b) {
+            pieces[0][b] = uint4{w1[4 * b], w1[4 * b + 1], w1[4 * b + 2], w1[4 * b + 3]};
+            pieces[1][b] = uint4{w2[4 * b], w2[4 * b + 1], w2[4 * b + 2], w2[4 * b + 3]};
+            pieces[2][b] = uint4{w3[4 * b], w3[4 * b + 1], w3[4 * b + 2], w3[4 * b + 3]};
+          }
+        } else {
+#pragma unroll
+          for (int j = 0; j < EW / 4; ++j) {
+            const int quad = sl * (EW / 4) + j;  // elements 4 quad .. 4 quad + 3
+            unsigned char* dst = Ps + g * weight_bytes<T>() + (quad >> 1) * 1024 + 16 * lane + 8 * (quad & 1);
+            *reinterpret_cast<uint2*>(dst) = uint2{w1[2 * j], w1[2 * j + 1]};
+            *reinterpret_cast<uint2*>(dst + 2048) = uint2{w2[2 * j], w2[2 * j + 1]};
+            *reinterpret_cast<uint2*>(dst + 4096) = uint2{w3[2 * j], w3[2 * j + 1]};
+          }
+        }
+      } else if constexpr (SL > 1) {
+#pragma unroll
+        for (int j = 0; j < EW / 4; ++j)
+          *reinterpret_cast<f32x4*>(Ps + g * weight_bytes<T>() + (sl * (EW / 4) + j) * 1024 + 16 * lane) = f32x4{w[4 * j], w[4 * j + 1], w[4 * j + 2], w[4 * j + 3]};
+      }
+    }
+    if (SL > 1) {
+      // the other buffer's last readers, of the chunk before, have passed this chunk's first barrier
+      if (a.two_buffers && it + 1 < n_chunks) stash(it + 1);
+      lds_barrier();
+    }
+    if (active) {
       if (__ballot(alpha != 1.f))
 #pragma unroll
         for (int dt = 0; dt < NVT; ++dt)
@@ -281,18 +343,9 @@ __global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentAr
         const int j16 = lane & 15, col16 = 16 * ((lane >> 4) & 1);
 #pragma unroll
         for (int b = 0; b < 2; ++b) {  // keys 16 b .. 16 b + 15; the lane's eight are 16 b + 4 h + u and 16 b + 8 + 4 h + u
-          uint32_t w1[4], w2[4], w3[4];
+          if constexpr (SL > 1)
 #pragma unroll
-          for (int u = 0; u < 4; ++u) {
-            const float p0 = s[8 * b + 2 * u], p1 = s[8 * b + 2 * u + 1];
-            w1[u] = pack_bf16x2(p0, p1);
-            const float r0 = p0 - __uint_as_float(w1[u] << 16), r1 = p1 - __uint_as_float(w1[u] & 0xffff0000u);
-            w2[u] = pack_bf16x2(r0, r1);
-            w3[u] = pack_bf16x2(r0 - __uint_as_float(w2[u] << 16), r1 - __uint_as_float(w2[u] & 0xffff0000u));
-          }
-          const bf16x8 p1 = __builtin_bit_cast(bf16x8, uint4{w1[0], w1[1], w1[2], w1[3]});
-          const bf16x8 p2 = __builtin_bit_cast(bf16x8, uint4{w2[0], w2[1], w2[2], w2[3]});
-          const bf16x8 p3 = __builtin_bit_cast(bf16x8, uint4{w3[0], w3[1], w3[2], w3[3]});
+            for (int pc = 0; pc < 3; ++pc) pieces[pc][b] = *reinterpret_cast<const uint4*>(Ps + g * weight_bytes<T>() + pc * 2048 + b * 1024 + 16 * lane);
           const bf16* vrow = reinterpret_cast<const bf16*>(K) + (16 * b + 4 * h + (j16 >> 2)) * ldk + col16 + 4 * (j16 & 3);
           // all columns' values first, then the pieces in turn, the smallest first: neighbouring products add to
           // different sums (columns behind the last tile repeat it, and nobody reads their sums)
@@ -304,34 +357,46 @@ __global__ __launch_bounds__(64 * G * SL) void latent_attn_kernel(const LatentAr
             v8[dt] = __builtin_bit_cast(bf16x8, uint4{v0.x, v0.y, v1.x, v1.y});
           }
 #pragma unroll
-          for (int dt = 0; dt < NVT; ++dt) o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8[dt], p3, o[dt], 0, 0, 0);
+          for (int pc = 2; pc >= 0; --pc)
 #pragma unroll
-          for (int dt = 0; dt < NVT; ++dt) o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8[dt], p2, o[dt], 0, 0, 0);
-#pragma unroll
-          for (int dt = 0; dt < NVT; ++dt) o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8[dt], p1, o[dt], 0, 0, 0);
+            for (int dt = 0; dt < NVT; ++dt)
+              o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8[dt], __builtin_bit_cast(bf16x8, pieces[pc][b]), o[dt], 0, 0, 0);
         }
       } else {
         const float* v = reinterpret_cast<const float*>(K) + 4 * h * ldk + c;
 #pragma unroll
-        for (int i0 = 0; i0 < 16; i0 += 4) {
+        for (int j = 0; j < 4; ++j) {
+          f32x4 p4;
+          if constexpr (SL > 1) p4 = *reinterpret_cast<const f32x4*>(Ps + g * weight_bytes<T>() + j * 1024 + 16 * lane);
+          else p4 = f32x4{w[4 * j], w[4 * j + 1], w[4 * j + 2], w[4 * j + 3]};
           float vv[4][NVT];
 #pragma unroll
           for (int u = 0; u < 4; ++u)
 #pragma unroll
-            for (int dt = 0; dt < NVT; ++dt) vv[u][dt] = v[(2 * i0 + u) * ldk + 32 * min(sl * NVT + dt, last_tile)];
+            for (int dt = 0; dt < NVT; ++dt) vv[u][dt] = v[(8 * j + u) * ldk + 32 * min(sl * NVT + dt, last_tile)];
 #pragma unroll
           for (int u = 0; u < 4; ++u)
 #pragma unroll
-            for (int dt = 0; dt < NVT; ++dt) o[dt] = __builtin_amdgcn_mfma_f32_32x32x2f32(vv[u][dt], s[i0 + u], o[dt], 0, 0, 0);
+            for (int dt = 0; dt < NVT; ++dt) o[dt] = __builtin_amdgcn_mfma_f32_32x32x2f32(vv[u][dt], p4[u], o[dt], 0, 0, 0);
         }
       }
     }
-    if (!a.two_buffers) lds_barrier();  // every wave is done with the one buffer
-    if (it + 1 < n_chunks) stash(it + 1);
-    lds_barrier();
+    if (SL == 1 || !a.two_buffers) {
+      if (!a.two_buffers) lds_barrier();  // every wave is done with the one buffer
+      if (it + 1 < n_chunks) stash(it + 1);
+      lds_barrier();
+    }
   }
 
   l += __shfl_xor(l, 32, 64);
+  if (SL > 1) {  // the waves' shares of the weights, in order
+    lds_barrier();
+    if (h == 0) row_s[wave % (SL > 1 ? G * SL : 1)][c] = l;
+    lds_barrier();
+    l = 0.f;
+#pragma unroll
+    for (int o2 = 0; o2 < SL; ++o2) l += row_s[SL > 1 ? g * SL + o2 : 0][c];
+  }
   if (!live) return;
   if (SINGLE && a.part) {
     const size_t at = (static_cast<size_t>(blockIdx.x) * a.heads + head) * a.spans + blockIdx.z;
@@ -441,7 +506,7 @@ int launch(const char* what, LatentArgs a, int blocks, int spans, hipStream_t st
   constexpr int E = 16 / sizeof(T);
   const int steps = (a.dk + 2 * E - 1) / (2 * E), ldk = 2 * E * steps + E;
   PYRE_REQUIRE(steps <= KQ * SL && a.rank <= 32 * NVT * SL, "%s: rows of %d / %d elements do not fit the form", what, a.dk, a.rank);
-  const size_t slack = 32 * NVT * SL > ldk ? 32 * NVT * SL - ldk : 0, exchange = SL > 1 ? sizeof(float) * G * SL * 1024 : 0;
+  const size_t slack = 32 * NVT * SL > ldk ? 32 * NVT * SL - ldk : 0, exchange = SL > 1 ? sizeof(float) * G * SL * 1024 + G * weight_bytes<T>() : 0;
   auto k_bytes = [&](int buffers) { return sizeof(T) * ((buffers * kKeys * static_cast<size_t>(ldk) + slack + 7) / 8 * 8); };
   const size_t budget = 156 * 1024;
   a.two_buffers = k_bytes(2) + exchange <= budget - 16 * 1024 ? 1 : 0;
@@ -460,7 +525,11 @@ int launch(const char* what, LatentArgs a, int blocks, int spans, hipStream_t st
       return fail("%s: the device refuses %zu bytes of LDS", what, lds);
     raised = lds;
   }
-  hipLaunchKernelGGL((latent_attn_kernel<T, G, SL, NVT, KQ, SINGLE>), dim3(blocks, groups, spans), dim3(64 * G * SL), lds, stream, a);
+  // prompt tiles come with those that see the most keys first: all heads of the longest start before the shorter ones,
+  // which then fill the compute units that are done
+  PYRE_REQUIRE(SINGLE || blocks <= 65535, "%s: %d tiles are more than a launch holds", what, blocks);
+  const dim3 grid = SINGLE ? dim3(blocks, groups, spans) : dim3(groups, blocks, 1);
+  hipLaunchKernelGGL((latent_attn_kernel<T, G, SL, NVT, KQ, SINGLE>), grid, dim3(64 * G * SL), lds, stream, a);
   return check_launch(what);
 }
 
@@ -485,14 +554,15 @@ extern "C" int pyre_latent_attn_tile(const void* q, const void* rows, void* out,
   PYRE_REQUIRE(tiles, "latent_attn_tile: no tiles");
   a.vec = aligned_rows(a, dt);
   // waves that share a row tile: as few as hold the row and the output in their registers
+  if (rank <= 128 && dk <= 128 && dt == kBF16) return launch<bf16, 4, 1, 4, 8, false>("latent_attn_tile", a, n_tiles, 1, stream);
   if (rank <= 128 && dk <= 256)
     return dt == kBF16 ? launch<bf16, 4, 1, 4, 16, false>("latent_attn_tile", a, n_tiles, 1, stream)
                        : launch<float, 4, 1, 4, 32, false>("latent_attn_tile", a, n_tiles, 1, stream);
   if (rank <= 256 && dk <= 384)
     return dt == kBF16 ? launch<bf16, 4, 2, 4, 12, false>("latent_attn_tile", a, n_tiles, 1, stream)
-                       : launch<float, 4, 2, 4, 24, false>("latent_attn_tile", a, n_tiles, 1, stream);
+                       : launch<float, 2, 2, 4, 24, false>("latent_attn_tile", a, n_tiles, 1, stream);
   return dt == kBF16 ? launch<bf16, 2, 4, 4, 10, false>("latent_attn_tile", a, n_tiles, 1, stream)
-                     : launch<float, 2, 4, 4, 20, false>("latent_attn_tile", a, n_tiles, 1, stream);
+                     : launch<float, 1, 4, 4, 20, false>("latent_attn_tile", a, n_tiles, 1, stream);
 }
 
 // Spans that a single token's keys are dealt to: one where the window is short, else of 64 keys (256 without a window

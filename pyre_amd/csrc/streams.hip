@@ -151,22 +151,26 @@ extern "C" int pyre_stream_norm(const float* src, int src_streams, float* dst, i
                      static_cast<TO*>(out), picked, hidden)
   // as for the other norms: which shape runs depends on the number of rows, what it computes does not but for the order
   // in which a row's block sum adds its threads; a few rows (a decode step) are spread over more threads each
-#define PYRE_SN_SHAPE(S)                                                  \
-  do {                                                                    \
-    const int quads = hidden / 4;                                         \
-    if (!vec && hidden <= 256) PYRE_SN(S, 256, 1, false);                 \
-    else if (!vec && hidden <= 4096) PYRE_SN(S, 1024, 4, false);          \
-    else if (!vec) PYRE_SN(S, 1024, 16, false);                           \
-    else if (quads <= 256) PYRE_SN(S, 256, 1, true);                      \
-    else if (n <= 128 && quads <= 1024) PYRE_SN(S, 1024, 1, true);        \
-    else if (quads <= 1024) PYRE_SN(S, 256, 4, true);                     \
-    else PYRE_SN(S, 1024, 4, true);                                       \
+#define PYRE_SN_SHAPE(S)                                            \
+  do {                                                              \
+    const int quads = hidden / 4;                                   \
+    if (quads <= 256) PYRE_SN(S, 256, 1, true);                     \
+    else if (n <= 128 && quads <= 1024) PYRE_SN(S, 1024, 1, true);  \
+    else if (quads <= 1024) PYRE_SN(S, 256, 4, true);               \
+    else PYRE_SN(S, 1024, 4, true);                                 \
   } while (0)
   PYRE_DISPATCH(y ? y_dt : kF32, TD, PYRE_DISPATCH(out_dt, TO, {
-    if (streams == 1) PYRE_SN_SHAPE(1);
-    else if (streams == 2) PYRE_SN_SHAPE(2);
-    else if (streams <= 4) PYRE_SN_SHAPE(4);
-    else PYRE_SN_SHAPE(8);
+    if (!vec) {  // any width, any number of streams
+      if (hidden <= 256) PYRE_SN(kMaxStreams, 256, 1, false);
+      else if (hidden <= 4096) PYRE_SN(kMaxStreams, 1024, 4, false);
+      else PYRE_SN(kMaxStreams, 1024, 16, false);
+    } else if (streams <= 2) {
+      PYRE_SN_SHAPE(2);
+    } else if (streams <= 4) {
+      PYRE_SN_SHAPE(4);
+    } else {
+      PYRE_SN_SHAPE(kMaxStreams);
+    }
   }));
 #undef PYRE_SN_SHAPE
 #undef PYRE_SN
