@@ -168,8 +168,10 @@ extern "C" int pyre_stream_norm(const float* src, int src_streams, float* dst, i
       PYRE_SN_SHAPE(2);
     } else if (streams <= 4) {
       PYRE_SN_SHAPE(4);
+    } else if (hidden <= 4096) {
+      PYRE_SN(kMaxStreams, 1024, 1, true);
     } else {
-      PYRE_SN_SHAPE(kMaxStreams);
+      PYRE_SN(kMaxStreams, 1024, 4, true);
     }
   }));
 #undef PYRE_SN_SHAPE
