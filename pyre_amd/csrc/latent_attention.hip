@@ -10,7 +10,8 @@
 // One kernel in two forms. A row tile of the matrix cores is 32 queries: for prompt portions the tokens of a tile
 // (up to 32 consecutive tokens of a request) for one head, for single tokens 32 heads of the token. G such row tiles
 // share a block and the chunk of 32 keys that it keeps in LDS; SL waves share a row tile: each takes every SL-th step
-// of the score's inner product (the parts are added through LDS, in order) and NVT * 32 columns of the output. The
+// of the score's inner product (the parts are added through LDS, in order), turns its share of the chunk's scores into
+// weights, which go round through LDS as well, and has NVT * 32 columns of the output. The
 // problem is transposed, S^T[key, query] and O^T[d, query], so that a lane's sixteen scores are operands of the second
 // product as they are. Scores, maxima, weights and sums are float32, the exponentials base two on scores scaled by
 // log2(e). bfloat16 rows and queries go through the 16-bit instruction (a product of two is exact in float32), each
@@ -29,7 +30,6 @@ namespace {
 
 typedef __attribute__((ext_vector_type(16))) float f32x16;
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
-typedef __attribute__((ext_vector_type(4))) __bf16 bf16x4;
 typedef __attribute__((ext_vector_type(4))) short s16x4;
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
@@ -99,7 +99,7 @@ __global__ __launch_bounds__(64 * G * SL, sizeof(T) == 2 && !SINGLE ? 2 : 1) voi
   unsigned char* Ps = reinterpret_cast<unsigned char*>(sred + (SL > 1 ? G * SL * 1024 : 0));  // [G] x weight_bytes<T>() if SL > 1
   int* tab_s = reinterpret_cast<int*>(Ps + (SL > 1 ? G * weight_bytes<T>() : 0));
   __shared__ int slot_s[kRing][kKeys];
-  __shared__ float row_s[SL > 1 ? G * SL : 1][32];  // the waves' maxima of their keys, per query; at the end their weights
+  __shared__ float row_s[G * SL][32];  // the waves' maxima of their keys, per query; at the end their weights
 
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = lane >> 5, c = lane & 31;
   const int g = wave / SL, sl = wave % SL;
@@ -276,7 +276,7 @@ __global__ __launch_bounds__(64 * G * SL, sizeof(T) == 2 && !SINGLE ? 2 : 1) voi
 #pragma unroll
         for (int i = 0; i < EW; ++i) w[i] *= a.scale2, mx = fmaxf(mx, w[i]);
       } else {
-        const unsigned seen = static_cast<unsigned>(hi - lo), first = static_cast<unsigned>(key0 + 8 * (EW / 4) * sl * (SL > 1) + 4 * h - lo);
+        const unsigned seen = static_cast<unsigned>(hi - lo), first = static_cast<unsigned>(key0 + 8 * (EW / 4) * sl + 4 * h - lo);
 #pragma unroll
         for (int i = 0; i < EW; ++i) {
           w[i] = first + 8 * (i >> 2) + (i & 3) <= seen ? w[i] * a.scale2 : -INFINITY;
@@ -284,7 +284,7 @@ __global__ __launch_bounds__(64 * G * SL, sizeof(T) == 2 && !SINGLE ? 2 : 1) voi
         }
       }
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-      if (SL > 1 && h == 0) row_s[wave % (SL > 1 ? G * SL : 1)][c] = mx;
+      if (SL > 1 && h == 0) row_s[wave][c] = mx;
     }
     if (SL > 1) lds_barrier();
     float alpha = 1.f;
@@ -292,7 +292,7 @@ __global__ __launch_bounds__(64 * G * SL, sizeof(T) == 2 && !SINGLE ? 2 : 1) voi
     if (active) {
       if (SL > 1)
 #pragma unroll
-        for (int o2 = 0; o2 < SL; ++o2) mx = fmaxf(mx, row_s[SL > 1 ? g * SL + o2 : 0][c]);
+        for (int o2 = 0; o2 < SL; ++o2) mx = fmaxf(mx, row_s[g * SL + o2][c]);
       const float m_new = fmaxf(m, mx), m_use = m_new == -INFINITY ? 0.f : m_new;
       alpha = exp2_hw(m - m_use);
       m = m_new;
@@ -391,11 +391,11 @@ __global__ __launch_bounds__(64 * G * SL, sizeof(T) == 2 && !SINGLE ? 2 : 1) voi
   l += __shfl_xor(l, 32, 64);
   if (SL > 1) {  // the waves' shares of the weights, in order
     lds_barrier();
-    if (h == 0) row_s[wave % (SL > 1 ? G * SL : 1)][c] = l;
+    if (h == 0) row_s[wave][c] = l;
     lds_barrier();
     l = 0.f;
 #pragma unroll
-    for (int o2 = 0; o2 < SL; ++o2) l += row_s[SL > 1 ? g * SL + o2 : 0][c];
+    for (int o2 = 0; o2 < SL; ++o2) l += row_s[g * SL + o2][c];
   }
   if (!live) return;
   if (SINGLE && a.part) {
