@@ -17,6 +17,8 @@
 //                      token, whose waves take a head at a time.
 // conv_state_update    one block a request, after every token has read the old state: the last T - 1 rows u of the
 //                      request, taken from the step's rows and, for a step shorter than that, from the old state.
+//                      In a step of one token a request (`single`) the four-element form leaves the new state behind itself:
+//                      whoever reads a channel's old rows is the only one to do so.
 //
 // A sum over the taps runs in the order j = 0 .. T - 1 wherever its inputs come from, so a token's result does not
 // depend on where a step begins. All arithmetic float32.
@@ -106,7 +108,7 @@ __global__ __launch_bounds__(kWave) void conv_qkv_write_vec_kernel(
     const float* __restrict__ q_gain, const float* __restrict__ k_gain, float eps, const float* __restrict__ cos,
     const float* __restrict__ sin, int rot, int neighbours, const int* __restrict__ positions, TC* __restrict__ q_out,
     TC* __restrict__ k_cache, TC* __restrict__ v_cache, float* __restrict__ gate_out, const int* __restrict__ slots,
-    int nq, int nkv, int dk, int dv, int page_size, int write_kv) {
+    int nq, int nkv, int dk, int dv, int page_size, int write_kv, float* shift_state) {
   __shared__ __attribute__((aligned(16))) float xs[kMaxHead];
   const int n = blockIdx.x, lane = threadIdx.x;
   const int seq = seq_of_token[n], run = n - q_start[seq], st = state_slots[seq];
@@ -117,10 +119,10 @@ __global__ __launch_bounds__(kWave) void conv_qkv_write_vec_kernel(
     // 256 columns of the values, then of the gates
     const int i = (static_cast<int>(blockIdx.y) - nq - nkv) * 4 * kWave + 4 * lane, nv = nkv * dv;
     if (i < nv) {
-      if (slot >= 0) {
+      if (slot >= 0 || shift_state) {
         const int g = i / dv, e = i % dv;
-        Vec4<TC>::store(v_cache + ((static_cast<size_t>(page) * nkv + g) * page_size + off) * dv + e,
-                        conv_value4(in, proj, n, run, st, (nq + nkv) * dk + i));
+        const float4 v = conv_value4(in, proj, n, run, st, (nq + nkv) * dk + i, shift_state);
+        if (slot >= 0) Vec4<TC>::store(v_cache + ((static_cast<size_t>(page) * nkv + g) * page_size + off) * dv + e, v);
       }
     } else if (gate_out && i - nv < nq * dv) {
       const float4 z = sum_partials4(proj + static_cast<size_t>(n) * in.ld + in.col0 + in.channels + (i - nv), in.partial_stride, in.n_partials);
@@ -132,7 +134,7 @@ __global__ __launch_bounds__(kWave) void conv_qkv_write_vec_kernel(
   const int head = blockIdx.y, e = 4 * lane, half = rot / 2;
   const bool mine = e < dk;
   float4 x = {0.f, 0.f, 0.f, 0.f};
-  if (mine) x = conv_value4(in, proj, n, run, st, head * dk + e);
+  if (mine) x = conv_value4(in, proj, n, run, st, head * dk + e, shift_state);
   const float* gain = head < nq ? q_gain : k_gain;
   if (gain) {
     // the sum of squares in the order of the kernel above: a lane's elements e, e + 64, .. there, four neighbours here;
@@ -174,7 +176,7 @@ extern "C" int pyre_conv_qkv_write(const void* proj, int proj_dt, int n_partials
                                    const float* k_gain, float eps, const float* cos, const float* sin, int rot,
                                    int neighbours, const int* positions, void* q_out, int q_dt, void* k_cache,
                                    void* v_cache, int cache_dt, float* gate_out, const int* slots, int n, int nq, int nkv,
-                                   int dk, int dv, int page_size, int write_kv, hipStream_t stream) {
+                                   int dk, int dv, int page_size, int write_kv, int single, hipStream_t stream) {
   PYRE_REQUIRE(known_dtype(proj_dt) && known_dtype(q_dt) && known_dtype(cache_dt) && n_partials >= 1, "conv_qkv_write: bad dtypes");
   PYRE_REQUIRE(nq > 0 && nkv > 0 && dk > 0 && dk <= kMaxHead && dv > 0 && page_size > 0,
                "conv_qkv_write: head sizes %d / %d are outside what the kernel takes (keys up to %d)", dk, dv, kMaxHead);
@@ -197,7 +199,8 @@ extern "C" int pyre_conv_qkv_write(const void* proj, int proj_dt, int n_partials
         hipLaunchKernelGGL((conv_qkv_write_vec_kernel<TP, TC>), dim3(n, nq + nkv + tail_blocks), dim3(kWave), 0, stream, in,
                            state_slots, seq_of_token, q_start, q_gain, k_gain, eps, cos, sin, rot, neighbours, positions,
                            static_cast<TC*>(q_out), static_cast<TC*>(k_cache), static_cast<TC*>(v_cache), gate_out, slots,
-                           nq, nkv, dk, dv, page_size, write_kv)));
+                           nq, nkv, dk, dv, page_size, write_kv, single && taps > 1 ? conv_state : nullptr)));
+    if (single) return check_launch("conv_qkv_write");
   } else {
     PYRE_DISPATCH(cache_dt, TC,
         hipLaunchKernelGGL(conv_qkv_write_kernel<TC>, dim3(n), dim3(kThreads), 0, stream, in, state_slots, seq_of_token,

@@ -230,20 +230,6 @@ __global__ __launch_bounds__(kThreads) void gdr_scan_kernel(const float* __restr
 // slot. The two meet at a barrier per slot that waits for LDS alone, so the walking wave never waits for memory: its
 // chain from token to token is arithmetic and LDS reads, and it reads a token's rows while it works on the one before.
 
-// The sum over a group of four or eight neighbouring lanes, in every lane of the group, by exchanges through the data
-// path of the vector unit itself (no LDS): neighbours at distance one, then two, then the other quad of the eight
-// (a mirror within the half row: all lanes of a quad hold the quad's sum by then, so any lane of the other quad will do).
-template <int CTRL>
-__device__ inline float lane_exchange(float v) {
-  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true));
-}
-template <int LPC>
-__device__ inline float lanes_sum(float v) {
-  v += lane_exchange<0xB1>(v);               // quad_perm [1, 0, 3, 2]
-  v += lane_exchange<0x4E>(v);               // quad_perm [2, 3, 0, 1]
-  if (LPC == 8) v += lane_exchange<0x141>(v);  // row_half_mirror
-  return v;
-}
 __device__ inline void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
 template <int DR, int LPC, int kGroup>

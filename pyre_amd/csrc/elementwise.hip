@@ -8,25 +8,34 @@
 using namespace pyre;
 
 // ---------------------------------------------------------------------------
-// Embedding: out[n, :] = float(table[ids[n], :]) * scale   (pyre/model.py:196)
+// Embedding: out[n, :] = float(table[ids[n], :]) * scale   (pyre/model.py:196), and, with a table of learned positions,
+// + float(places[positions[n], :])
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict__ ids,
+                             const int* __restrict__ positions, const T* __restrict__ places, int n_places,
                              float* __restrict__ out, int hidden, float scale) {
   const int n = blockIdx.x;
   const T* row = table + static_cast<size_t>(ids[n]) * hidden;
   float* o = out + static_cast<size_t>(n) * hidden;
+  if (places) {  // the engine takes no request that is longer than the table
+    const T* place = places + static_cast<size_t>(min(positions[n], n_places - 1)) * hidden;
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x) o[i] = fmaf(to_float(row[i]), scale, to_float(place[i]));
+    return;
+  }
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) o[i] = to_float(row[i]) * scale;
 }
 
-extern "C" int pyre_embed(const void* table, int table_dt, const int* ids, float* out, int n,
-                          int hidden, float scale, hipStream_t stream) {
+extern "C" int pyre_embed(const void* table, int table_dt, const int* ids, const int* positions, const void* places,
+                          int n_places, float* out, int n, int hidden, float scale, hipStream_t stream) {
+  PYRE_REQUIRE(!places || (positions && n_places > 0), "embed: a table of positions needs rows and the tokens' positions");
   PYRE_REQUIRE(known_dtype(table_dt), "embed: unknown table dtype %d", table_dt);
   PYRE_REQUIRE(n >= 0 && hidden > 0, "embed: bad sizes n=%d hidden=%d", n, hidden);
   if (n == 0) return 0;
   PYRE_DISPATCH(table_dt, T,
                 hipLaunchKernelGGL(embed_kernel<T>, dim3(n), dim3(256), 0, stream,
-                                   static_cast<const T*>(table), ids, out, hidden, scale));
+                                   static_cast<const T*>(table), ids, positions, static_cast<const T*>(places), n_places,
+                                   out, hidden, scale));
   return check_launch("embed");
 }
 

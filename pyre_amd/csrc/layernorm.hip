@@ -183,7 +183,17 @@ __global__ __launch_bounds__(THREADS) void add_layernorm_vec_kernel(
   }
 }
 
-// act[n, i] = g * sigmoid(slope * (g + cubic g^3)) * (u + shift), g = min(gate[n, i], limit), u = clamp(up[n, i], -limit, limit);
+__device__ inline float clipped_unit(float g, float u, float limit, float slope, float shift, float cubic) {
+  if (limit > 0.f) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+  }
+  if (is_step(slope)) return fmaxf(g, 0.f) * (u + shift);
+  return g / (1.f + expf(-slope * fmaf(cubic * g, g * g, g))) * (u + shift);
+}
+
+// act[n, i] = g * sigmoid(slope * (g + cubic g^3)) * (u + shift), g = min(gate[n, i], limit), u = clamp(up[n, i], -limit, limit)
+// (an infinite slope: max(g, 0) (u + shift));
 // gate = gu[:, :I], up = gu[:, I:], the partial sums added first. limit <= 0: no clipping.
 __global__ void clipped_glu_kernel(const void* __restrict__ gu, int gu_dt, int n_partials, size_t partial_stride,
                                    void* __restrict__ out, int out_dt, size_t total, int inter, float limit,
@@ -197,19 +207,7 @@ __global__ void clipped_glu_kernel(const void* __restrict__ gu, int gu_dt, int n
     g += load_as_float(gu, gu_dt, p * partial_stride + gi);
     u += load_as_float(gu, gu_dt, p * partial_stride + ui);
   }
-  if (limit > 0.f) {
-    g = fminf(g, limit);
-    u = fminf(fmaxf(u, -limit), limit);
-  }
-  store_from_float(out, out_dt, i, g / (1.f + expf(-slope * fmaf(cubic * g, g * g, g))) * (u + shift));
-}
-
-__device__ inline float clipped_unit(float g, float u, float limit, float slope, float shift, float cubic) {
-  if (limit > 0.f) {
-    g = fminf(g, limit);
-    u = fminf(fmaxf(u, -limit), limit);
-  }
-  return g / (1.f + expf(-slope * fmaf(cubic * g, g * g, g))) * (u + shift);
+  store_from_float(out, out_dt, i, clipped_unit(g, u, limit, slope, shift, cubic));
 }
 
 // The same, four elements a thread (inter and the partial sums' stride are multiples of four).
@@ -246,6 +244,7 @@ __global__ __launch_bounds__(256) void clipped_glu_stream_kernel(const bf16* __r
       gv = fminf(gv, limit);
       uv = fminf(fmaxf(uv, -limit), limit);
     }
+    if (is_step(slope)) return fmaxf(gv, 0.f) * (uv + shift);
     return gv * __builtin_amdgcn_rcpf(1.f + __expf(-slope * fmaf(cubic * gv, gv * gv, gv))) * (uv + shift);
   };
   u32x4 y;

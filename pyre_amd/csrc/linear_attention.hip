@@ -11,6 +11,7 @@
 // gla_chunks   the same for requests that bring many tokens, sixteen tokens at a time on the matrix cores.
 // gla_finish   divides every head's output by its root mean square, times a gain over dv that the
 //              heads share, times silu(g) and a scale; writes the rows that the output product reads.
+// gla_finish_wide  the same for heads that are normed together, with sigmoid(g).
 //
 // Decays, their logarithms, the state and the unit norm are float32 whatever the model's type.
 #include "pyre_api.h"
@@ -23,6 +24,8 @@ namespace {
 
 constexpr int kThreads = 256;
 constexpr int kMaxRank = 512;
+
+__device__ inline float silu_of(float z) { return z / (1.f + expf(-z)); }
 
 __global__ __launch_bounds__(kThreads) void gla_prepare_kernel(
     const void* __restrict__ proj, int proj_dt, int n_partials, size_t partial_stride, int ld, int col0,
@@ -332,13 +335,47 @@ __global__ __launch_bounds__(kThreads) void gla_finish_kernel(
   }
 }
 
+// The finish of a recurrence whose heads are normed together: a token's row of all heads divided by its root mean
+// square over H dv, times a gain over that row, times sigmoid(g) and a scale. One block a token, VEC elements to a load.
+template <typename TG, typename TO, int VEC>
+__global__ __launch_bounds__(kThreads) void gla_finish_wide_kernel(
+    const float* __restrict__ o, const float* __restrict__ x, const TG* __restrict__ gain, float eps, float out_scale,
+    TO* __restrict__ out, size_t out_ld, int hk, int hv) {
+  __shared__ float scratch[16];
+  const int n = blockIdx.x, tid = threadIdx.x;
+  const float* row = o + static_cast<size_t>(n) * hv;
+  const float* g = x + static_cast<size_t>(n) * (3 * hk + 2 * hv) + 3 * hk + hv;
+  TO* dst = out + static_cast<size_t>(n) * out_ld;
+  float ss = 0.f;
+  for (int i = VEC * tid; i < hv; i += VEC * kThreads) {
+    if constexpr (VEC == 4) {
+      const float4 v = Vec4<float>::load(row + i);
+      ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+    } else {
+      ss += row[i] * row[i];
+    }
+  }
+  const float f = 1.f / sqrtf(block_sum(ss, scratch) / static_cast<float>(hv) + eps) * out_scale;
+  for (int i = VEC * tid; i < hv; i += VEC * kThreads) {
+    if constexpr (VEC == 4) {
+      const float4 v = Vec4<float>::load(row + i), w = Vec4<TG>::load(gain + i), z = Vec4<float>::load(g + i);
+      Vec4<TO>::store(dst + i, float4{v.x * f * w.x / (1.f + expf(-z.x)), v.y * f * w.y / (1.f + expf(-z.y)),
+                                      v.z * f * w.z / (1.f + expf(-z.z)), v.w * f * w.w / (1.f + expf(-z.w))});
+    } else {
+      dst[i] = from_float<TO>(row[i] * f * to_float(gain[i]) / (1.f + expf(-g[i])));
+    }
+  }
+}
+
 // The rows [q | k | ld | v | g] for a recurrence whose decay is one fixed number per head: the first `rot` elements of
 // every query and key head are turned by position (pairs (e, e + rot / 2), or neighbours (2e, 2e + 1)), the keys then
-// scaled; ld of every key channel of head h is log_decay[h]. One block a token, a thread a pair (or an element).
+// scaled; ld of every key channel of head h is log_decay[h]. `silu`: queries, keys and values go through silu first.
+// One block a token, a thread a pair (or an element).
 __global__ __launch_bounds__(kThreads) void retention_prepare_kernel(
     const void* __restrict__ proj, int proj_dt, int n_partials, size_t partial_stride, int ld, int col0,
     const float* __restrict__ log_decay, const float* __restrict__ cos, const float* __restrict__ sin, int rot,
-    int neighbours, const int* __restrict__ positions, float kscale, float* __restrict__ x, int heads, int dk, int dv) {
+    int neighbours, const int* __restrict__ positions, float kscale, int silu, float* __restrict__ x, int heads, int dk,
+    int dv) {
   const int n = blockIdx.x, tid = threadIdx.x;
   const size_t in_row = static_cast<size_t>(n) * ld + col0;
   const int hk = heads * dk, hv = heads * dv, width = 3 * hk + 2 * hv, half = rot / 2;
@@ -346,7 +383,7 @@ __global__ __launch_bounds__(kThreads) void retention_prepare_kernel(
   auto value = [&](int col) {
     float v = 0.f;
     for (int p = 0; p < n_partials; ++p) v += load_as_float(proj, proj_dt, p * partial_stride + in_row + col);
-    return v;
+    return silu && col < 2 * hk + hv ? silu_of(v) : v;
   };
   const size_t trig = static_cast<size_t>(positions[n]) * half;
   // queries (columns 0 .. hk) and keys (hk .. 2 hk): the turned pairs of every head, then the elements that pass
@@ -376,7 +413,8 @@ template <typename TP>
 __global__ __launch_bounds__(kWave) void retention_prepare_vec_kernel(
     const TP* __restrict__ proj, int n_partials, size_t partial_stride, int ld, int col0,
     const float* __restrict__ log_decay, const float* __restrict__ cos, const float* __restrict__ sin, int rot,
-    int neighbours, const int* __restrict__ positions, float kscale, float* __restrict__ x, int heads, int dk, int dv) {
+    int neighbours, const int* __restrict__ positions, float kscale, int silu, float* __restrict__ x, int heads, int dk,
+    int dv) {
   __shared__ __attribute__((aligned(16))) float xs[256];
   const int n = blockIdx.x, lane = threadIdx.x;
   const TP* in = proj + static_cast<size_t>(n) * ld + col0;
@@ -388,7 +426,9 @@ __global__ __launch_bounds__(kWave) void retention_prepare_vec_kernel(
       const float l = log_decay[i / dk];  // four neighbours share a head: dk is a multiple of four
       *reinterpret_cast<float4*>(xr + 2 * hk + i) = float4{l, l, l, l};
     } else if (i < hk + 2 * hv) {
-      *reinterpret_cast<float4*>(xr + 2 * hk + i) = sum_partials4(in + 2 * hk + (i - hk), partial_stride, n_partials);
+      float4 v = sum_partials4(in + 2 * hk + (i - hk), partial_stride, n_partials);
+      if (silu && i < hk + hv) v = float4{silu_of(v.x), silu_of(v.y), silu_of(v.z), silu_of(v.w)};
+      *reinterpret_cast<float4*>(xr + 2 * hk + i) = v;
     }
     return;
   }
@@ -397,6 +437,7 @@ __global__ __launch_bounds__(kWave) void retention_prepare_vec_kernel(
   float4 v = {0.f, 0.f, 0.f, 0.f};
   if (mine) {
     v = sum_partials4(in + head * dk + e, partial_stride, n_partials);
+    if (silu) v = float4{silu_of(v.x), silu_of(v.y), silu_of(v.z), silu_of(v.w)};
     *reinterpret_cast<float4*>(xs + e) = v;
   }
   __syncthreads();
@@ -506,10 +547,30 @@ extern "C" int pyre_gla_finish(const float* o, const float* x, const void* gain,
   return check_launch("gla_finish");
 }
 
+extern "C" int pyre_gla_finish_wide(const float* o, const float* x, const void* gain, int gain_dt, float eps,
+                                    float out_scale, void* out, int out_dt, long out_ld, int n, int heads, int dk, int dv,
+                                    hipStream_t stream) {
+  PYRE_REQUIRE(known_dtype(gain_dt) && known_dtype(out_dt) && gain, "gla_finish_wide: bad dtypes, or no gain");
+  PYRE_REQUIRE(heads > 0 && dk > 0 && dv > 0 && eps > 0.f, "gla_finish_wide: sizes %d x %d / %d are not taken", heads, dk, dv);
+  if (n <= 0) return 0;
+  const int hk = heads * dk, hv = heads * dv;
+  const auto a16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  const bool vec = hk % 4 == 0 && hv % 4 == 0 && out_ld % 4 == 0 && a16(o) && a16(x) && a16(gain) && a16(out);
+  PYRE_DISPATCH(gain_dt, TG, PYRE_DISPATCH(out_dt, TO, {
+    if (vec)
+      hipLaunchKernelGGL((gla_finish_wide_kernel<TG, TO, 4>), dim3(n), dim3(kThreads), 0, stream, o, x,
+                         static_cast<const TG*>(gain), eps, out_scale, static_cast<TO*>(out), static_cast<size_t>(out_ld), hk, hv);
+    else
+      hipLaunchKernelGGL((gla_finish_wide_kernel<TG, TO, 1>), dim3(n), dim3(kThreads), 0, stream, o, x,
+                         static_cast<const TG*>(gain), eps, out_scale, static_cast<TO*>(out), static_cast<size_t>(out_ld), hk, hv);
+  }));
+  return check_launch("gla_finish_wide");
+}
+
 extern "C" int pyre_retention_prepare(const void* proj, int proj_dt, int n_partials, long partial_stride, int ld, int col0,
                                       const float* log_decay, const float* cos, const float* sin, int rot, int neighbours,
-                                      const int* positions, float kscale, float* x, int n, int heads, int dk, int dv,
-                                      hipStream_t stream) {
+                                      const int* positions, float kscale, int silu, float* x, int n, int heads, int dk,
+                                      int dv, hipStream_t stream) {
   PYRE_REQUIRE(known_dtype(proj_dt) && n_partials >= 1, "retention_prepare: bad dtypes");
   PYRE_REQUIRE(heads > 0 && dk > 0 && dv > 0 && log_decay && positions, "retention_prepare: bad sizes");
   PYRE_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= dk && (rot == 0 || (cos && sin)),
@@ -521,11 +582,11 @@ extern "C" int pyre_retention_prepare(const void* proj, int proj_dt, int n_parti
     PYRE_DISPATCH(proj_dt, TP,
         hipLaunchKernelGGL(retention_prepare_vec_kernel<TP>, dim3(n, 2 * heads + tail_blocks), dim3(kWave), 0, stream,
                            static_cast<const TP*>(proj), n_partials, static_cast<size_t>(partial_stride), ld, col0,
-                           log_decay, cos, sin, rot, neighbours, positions, kscale, x, heads, dk, dv));
+                           log_decay, cos, sin, rot, neighbours, positions, kscale, silu, x, heads, dk, dv));
     return check_launch("retention_prepare");
   }
   hipLaunchKernelGGL(retention_prepare_kernel, dim3(n), dim3(kThreads), 0, stream, proj, proj_dt, n_partials,
                      static_cast<size_t>(partial_stride), ld, col0, log_decay, cos, sin, rot, neighbours, positions, kscale,
-                     x, heads, dk, dv);
+                     silu, x, heads, dk, dv);
   return check_launch("retention_prepare");
 }

@@ -21,9 +21,9 @@ const char* pyre_sources_digest();
 // a measurement of achievable read bandwidth.
 int pyre_read_probe(const void* p, size_t bytes, int blocks, unsigned* sink, hipStream_t stream);
 
-// out[n] = table[ids[n]] * scale, float32.
-int pyre_embed(const void* table, int table_dt, const int* ids, float* out, int n, int hidden, float scale,
-               hipStream_t stream);
+// out[n] = table[ids[n]] * scale (+ places[positions[n]], a table of n_places rows of the same type, or null), float32.
+int pyre_embed(const void* table, int table_dt, const int* ids, const int* positions, const void* places, int n_places,
+               float* out, int n, int hidden, float scale, hipStream_t stream);
 
 int pyre_add_rmsnorm(float* resid, const void* delta, int delta_dt, int n_partials,
                      long partial_stride, const void* bias, int bias_dt, const void* gain,
@@ -373,13 +373,41 @@ int pyre_conv_qkv_write(const void* proj, int proj_dt, int n_partials, long part
                         const int* q_start, int n_seqs, const float* q_gain, const float* k_gain, float eps,
                         const float* cos, const float* sin, int rot, int neighbours, const int* positions, void* q_out,
                         int q_dt, void* k_cache, void* v_cache, int cache_dt, float* gate_out, const int* slots, int n,
-                        int nq, int nkv, int dk, int dv, int page_size, int write_kv, hipStream_t stream);
+                        int nq, int nkv, int dk, int dv, int page_size, int write_kv, int single, hipStream_t stream);
 
 // The rows [q | k | log decay | v | g] of the recurrent kernels for a fixed decay per head, queries and keys turned.
 int pyre_retention_prepare(const void* proj, int proj_dt, int n_partials, long partial_stride, int ld, int col0,
                            const float* log_decay, const float* cos, const float* sin, int rot, int neighbours,
-                           const int* positions, float kscale, float* x, int n, int heads, int dk, int dv,
+                           const int* positions, float kscale, int silu, float* x, int n, int heads, int dk, int dv,
                            hipStream_t stream);
+// o over all heads divided by its root mean square, times gain [heads dv], times sigmoid(g) and out_scale.
+int pyre_gla_finish_wide(const float* o, const float* x, const void* gain, int gain_dt, float eps, float out_scale, void* out,
+                         int out_dt, long out_ld, int n, int heads, int dk, int dv, hipStream_t stream);
+
+// ---- a selective scan (selective_scan.hip) ----
+// x[n, inner] = silu(conv over time of the product's columns from col0 on + conv_b); state [slots][taps - 1][inner] is
+// brought up to date. `single`: the step brings one token a request.
+int pyre_ssm_conv(const void* proj, int proj_dt, int n_partials, long partial_stride, int ld, int col0, const float* taps_w,
+                  int taps, const float* conv_b, float* conv_state, const int* state_slots, const int* seq_of_token,
+                  const int* q_start, int n_seqs, int single, void* x, int x_dt, int n, int inner, hipStream_t stream);
+// out[n] = the product's first `rank` columns as operands of the next product: float32 [n, padded], or bfloat16
+// [n, 2 padded], rounded to bfloat16 and what the rounding left; zeros from `rank` to `padded`.
+int pyre_ssm_low(const void* sel, int sel_dt, int n_partials, long partial_stride, int ld, void* out, int out_dt, int rank,
+                 int padded, int n, hipStream_t stream);
+// The recurrence over each request's tokens of the step: dt = softplus(z + dt_b), S <- exp(dt A) S + dt x B,
+// out = (S C + D x) silu(gate) out_scale; B and C the columns b0 .. of `sel`, the gate the columns g0 .. of `proj`.
+// A2 [inner][state] = A log2(e); S float32 [slots][inner][state].
+int pyre_ssm_scan(const void* z, int z_dt, int z_partials, long z_stride, const float* dt_b, const void* x, int x_dt,
+                  const void* sel, int sel_dt, int sel_partials, long sel_stride, int sel_ld, int b0, const void* proj,
+                  int proj_dt, int proj_partials, long proj_stride, int proj_ld, int g0, const float* A2, const float* D,
+                  float* state, const int* q_start, const int* state_slots, int n_seqs, float out_scale, void* out, int out_dt,
+                  long out_ld, int inner, int n_state, hipStream_t stream);
+// The same for steps of one token a request, the step size's product included: z = dt_w [inner][rank, rows dt_ld apart] sel[0 .. rank).
+int pyre_ssm_step(const void* dt_w, int dt_w_dt, long dt_ld, const float* dt_b, const void* x, int x_dt, const void* sel,
+                  int sel_dt, int sel_partials, long sel_stride, int sel_ld, int rank, const void* proj, int proj_dt,
+                  int proj_partials, long proj_stride, int proj_ld, int g0, const float* A2, const float* D, float* state,
+                  const int* state_slots, int n_seqs, float out_scale, void* out, int out_dt, long out_ld, int inner,
+                  int n_state, hipStream_t stream);
 
 int pyre_route_grouped(const void* z, int z_dt, int n_partials, long partial_stride, const void* bias, int bias_dt,
                        const float* correction, float* gates, int n, int experts, int top, int groups, int keep_groups,

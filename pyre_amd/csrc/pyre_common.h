@@ -113,15 +113,19 @@ __device__ inline void store_from_float(void* p, int dt, size_t i, float v) {
 // The gated unit that a gate/up product may finish in its epilogue: g sigmoid(slope (g + cubic g^3)) (u + shift) with
 // g = min(gate, limit), u = clamp(up, -limit, limit) (limit <= 0: no clipping). The defaults are the SiLU-gate;
 // slope 2 sqrt(2 / pi) with cubic 0.044715 is the tanh form of GELU, since (1 + tanh z) / 2 = sigmoid(2 z);
+// an infinite slope makes the sigmoid a step: the unit is then max(g, 0) (u + shift), the ReLU-gate;
 // the exponential is the hardware's (the result is rounded to bfloat16).
 struct GateShape {
   float limit = 0.f, slope = 1.f, shift = 0.f, cubic = 0.f;
 };
+// What gates whatever exponential a kernel uses: the step that an infinite slope stands for.
+__device__ inline bool is_step(float slope) { return slope == INFINITY; }
 __device__ inline float gated_unit(float gate, float up, GateShape a) {
   if (a.limit > 0.f) {
     gate = fminf(gate, a.limit);
     up = fminf(fmaxf(up, -a.limit), a.limit);
   }
+  if (is_step(a.slope)) return fmaxf(gate, 0.f) * (up + a.shift);
   return gate / (1.f + __expf(-a.slope * fmaf(a.cubic * gate, gate * gate, gate))) * (up + a.shift);
 }
 
@@ -133,6 +137,21 @@ __device__ inline float wave_sum(float v) {
 __device__ inline float wave_max(float v) {
 #pragma unroll
   for (int o = kWave / 2; o > 0; o >>= 1) v = fmaxf(v, __shfl_xor(v, o, kWave));
+  return v;
+}
+
+// The sum over a group of four or eight neighbouring lanes, in every lane of the group, by exchanges through the data
+// path of the vector unit itself (no LDS): neighbours at distance one, then two, then the other quad of the eight
+// (a mirror within the half row: all lanes of a quad hold the quad's sum by then, so any lane of the other quad will do).
+template <int CTRL>
+__device__ inline float lane_exchange(float v) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true));
+}
+template <int LPC>
+__device__ inline float lanes_sum(float v) {
+  v += lane_exchange<0xB1>(v);               // quad_perm [1, 0, 3, 2]
+  v += lane_exchange<0x4E>(v);               // quad_perm [2, 3, 0, 1]
+  if (LPC == 8) v += lane_exchange<0x141>(v);  // row_half_mirror
   return v;
 }
 

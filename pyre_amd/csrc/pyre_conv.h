@@ -48,8 +48,11 @@ __device__ inline float conv_value(const ConvIn& in, int n, int run, int slot, i
 // of four, the pointers on 16 bytes): every tap's input asked for before the first is used; the same sums in the same
 // order as conv_value.
 constexpr int kConvVecTaps = 8;  // the most taps of this form
+// `shift_state` (the states, as in.state, or null): the step brings one token a request, so
+// these four channels' inputs, which lie in registers, less the oldest are the new state and go there at once.
 template <typename TP>
-__device__ inline float4 conv_value4(const ConvIn& in, const TP* proj, int n, int run, int slot, int ch) {
+__device__ inline float4 conv_value4(const ConvIn& in, const TP* proj, int n, int run, int slot, int ch,
+                                     float* shift_state = nullptr) {
   const TP* row = proj + static_cast<size_t>(n) * in.ld + in.col0 + ch;
   const float4 b = in.bias ? *reinterpret_cast<const float4*>(in.bias + in.col0 + ch) : float4{0.f, 0.f, 0.f, 0.f};
   if (!in.taps_w) return in.bias ? add4(sum_partials4(row, in.partial_stride, in.n_partials), b) : sum_partials4(row, in.partial_stride, in.n_partials);
@@ -69,6 +72,8 @@ __device__ inline float4 conv_value4(const ConvIn& in, const TP* proj, int n, in
     if (j >= in.taps) break;
     const float4 w = *reinterpret_cast<const float4*>(in.taps_w + static_cast<size_t>(j) * in.channels + ch);
     y = float4{fmaf(w.x, u[j].x, y.x), fmaf(w.y, u[j].y, y.y), fmaf(w.z, u[j].z, y.z), fmaf(w.w, u[j].w, y.w)};
+    if (shift_state && j > 0)
+      *reinterpret_cast<float4*>(shift_state + (static_cast<size_t>(slot) * (in.taps - 1) + (j - 1)) * in.channels + ch) = u[j];
   }
   return y;
 }

@@ -122,15 +122,21 @@ class Partials:
                 _ptr(self.bias), dtype_code(self.bias) if self.bias is not None else 0)
 
 
-def embed(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor, scale: float = 1.0) -> None:
-    """out[n] = float32(table[ids[n]]) * scale; ids must already be checked against the vocabulary."""
-    _dev(table, ids, out)
+def embed(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor, scale: float = 1.0,
+          positions: torch.Tensor | None = None, places: torch.Tensor | None = None) -> None:
+    """out[n] = float32(table[ids[n]]) * scale; ids must already be checked against the vocabulary. With ``places``
+    [rows, H] also + float32(places[positions[n]])."""
+    _dev(table, ids, out, positions, places)
     n, hidden = out.shape
     if table.dim() != 2 or table.shape[1] != hidden or out.dtype != torch.float32:
         raise KernelError("embed: table [V, H] and float32 out [N, H] expected")
     _contig("table", table), _contig("out", out), _i32("ids", ids, n)
-    call("pyre_embed", table.data_ptr(), dtype_code(table), ids.data_ptr(), out.data_ptr(), n, hidden,
-         float(scale), _stream())
+    if places is not None:
+        if places.dim() != 2 or places.shape[1] != hidden or places.dtype != table.dtype or places.shape[0] < 1 or positions is None:
+            raise KernelError("embed: the table of positions is [rows, H] of the token table's type, with the tokens' positions")
+        _contig("places", places), _i32("positions", positions, n)
+    call("pyre_embed", table.data_ptr(), dtype_code(table), ids.data_ptr(), _ptr(positions), _ptr(places),
+         places.shape[0] if places is not None else 0, out.data_ptr(), n, hidden, float(scale), _stream())
 
 
 def add_rmsnorm(resid: torch.Tensor, delta: Partials | None, gain: torch.Tensor, eps: float,
@@ -208,6 +214,8 @@ def add_layernorm(resid: torch.Tensor, delta: Partials | None, gain: torch.Tenso
          dtype_code(out), _ptr(rows), n, hidden, float(eps), _stream())
 
 
+#: slope at which the gated unit's sigmoid is a step: max(g, 0) (u + shift)
+RELU_SLOPE = float("inf")
 #: slope and cubic term that make g sigmoid(slope (g + cubic g^3)) the tanh form of GELU: (1 + tanh z) / 2 = sigmoid(2 z)
 GELU_TANH_SLOPE, GELU_TANH_CUBIC = 2.0 * (2.0 / 3.141592653589793) ** 0.5, 0.044715
 
@@ -215,7 +223,8 @@ GELU_TANH_SLOPE, GELU_TANH_CUBIC = 2.0 * (2.0 / 3.141592653589793) ** 0.5, 0.044
 def clipped_glu(gu: Partials, out: torch.Tensor, n: int, limit: float, slope: float, shift: float = 1.0,
                 cubic: float = 0.0) -> None:
     """out[n, i] = g * sigmoid(slope * (g + cubic g^3)) * (u + shift) with g = min(gate, limit),
-    u = clamp(up, -limit, limit), gate = gu[:, :I], up = gu[:, I:] (``limit`` <= 0: no clipping)."""
+    u = clamp(up, -limit, limit), gate = gu[:, :I], up = gu[:, I:] (``limit`` <= 0: no clipping; an infinite ``slope``:
+    max(g, 0) (u + shift))."""
     _dev(gu.data, out)
     inter = out.shape[-1]
     if gu.width != 2 * inter or gu.rows < n or out.shape[0] < n:
@@ -426,6 +435,21 @@ def gla_finish(o: torch.Tensor, x: torch.Tensor, gain: torch.Tensor | None, eps:
     if gain is not None:
         _contig("gain", gain)
     call("pyre_gla_finish", o.data_ptr(), x.data_ptr(), _ptr(gain), dtype_code(gain) if gain is not None else 0, float(eps), float(out_scale),
+         out.data_ptr(), dtype_code(out), out.stride(0), n, heads, dk, dv, _stream())
+
+
+def gla_finish_wide(o: torch.Tensor, x: torch.Tensor, gain: torch.Tensor, eps: float, out_scale: float, out: torch.Tensor,
+                    n: int, heads: int, dk: int, dv: int) -> None:
+    """out[n] = o / rms(o over all heads' heads*dv) * gain * sigmoid(g) * out_scale, the gate g from the rows ``x``; ``out``
+    has contiguous rows."""
+    _dev(o, x, gain, out)
+    if o.dtype != torch.float32 or x.dtype != torch.float32 or not o.is_contiguous() or not x.is_contiguous():
+        raise KernelError("gla_finish_wide: o and x are contiguous float32")
+    if gain.numel() != heads * dv or out.dim() != 2 or out.stride(1) != 1 or out.shape[1] < heads * dv or out.shape[0] < n or \
+            o.shape[-1] != heads * dv or o.shape[0] < n or x.shape[-1] != gla_row_width(heads, dk, dv) or x.shape[0] < n:
+        raise KernelError("gla_finish_wide: gain [heads*dv] and out [>= n, >= heads*dv] expected")
+    _contig("gain", gain)
+    call("pyre_gla_finish_wide", o.data_ptr(), x.data_ptr(), gain.data_ptr(), dtype_code(gain), float(eps), float(out_scale),
          out.data_ptr(), dtype_code(out), out.stride(0), n, heads, dk, dv, _stream())
 
 
@@ -1402,7 +1426,8 @@ def conv_qkv_write(proj: Partials, col0: int, taps_w: torch.Tensor | None, conv_
                    q_gain: torch.Tensor | None, k_gain: torch.Tensor | None, eps: float, cos: torch.Tensor | None,
                    sin: torch.Tensor | None, rot: int, neighbours: bool, positions: torch.Tensor, q_out: torch.Tensor,
                    k_cache: torch.Tensor | None, v_cache: torch.Tensor | None, gate_out: torch.Tensor | None,
-                   slots: torch.Tensor | None, n: int, nq: int, nkv: int, dk: int, dv: int, page_size: int) -> None:
+                   slots: torch.Tensor | None, n: int, nq: int, nkv: int, dk: int, dv: int, page_size: int,
+                   single: bool = False) -> None:
     """Finish a step's input product from column ``col0`` on (``nq`` query and ``nkv`` key heads of ``dk``, ``nkv`` value
     heads of ``dv``, then ``nq * dv`` gate columns if ``gate_out`` is given). Queries, keys and values first go through a
     causal convolution over the request's tokens, ``taps_w`` float32 [taps, channels] (None: none), whose inputs before
@@ -1410,7 +1435,10 @@ def conv_qkv_write(proj: Partials, col0: int, taps_w: torch.Tensor | None, conv_
     rows; it is brought up to date after every token has read it). Then queries and keys are divided by their root mean
     square per head, times ``q_gain`` / ``k_gain`` over ``dk`` (None: not normed), and their first ``rot`` elements turned
     by position (``neighbours``: element 2e with 2e + 1, else e with e + rot/2). Queries go to ``q_out [N, nq*dk]``, keys and
-    values to their pages at ``slots``, sigmoid(gate) to float32 ``gate_out [N, nq*dv]``."""
+    values to their pages at ``slots``, sigmoid(gate) to float32 ``gate_out [N, nq*dv]``. ``single``: the step brings one
+    token a request (token i is request i's), so that the state can be brought up to date as it is read."""
+    if single and n != n_seqs:
+        raise KernelError(f"conv_qkv_write: {n} tokens of {n_seqs} requests are not one token each")
     _dev(proj.data, taps_w, conv_state, state_slots, seq_of_token, q_start, q_gain, k_gain, cos, sin, positions, q_out,
          k_cache, v_cache, gate_out, slots)
     channels = (nq + nkv) * dk + nkv * dv
@@ -1456,14 +1484,14 @@ def conv_qkv_write(proj: Partials, col0: int, taps_w: torch.Tensor | None, conv_
          seq_of_token.data_ptr(), q_start.data_ptr(), n_seqs, _ptr(q_gain), _ptr(k_gain), float(eps),
          _ptr(cos) if rot else None, _ptr(sin) if rot else None, int(rot), int(bool(neighbours)), positions.data_ptr(),
          q_out.data_ptr(), dtype_code(q_out), _ptr(k_cache), _ptr(v_cache), cache_dt, _ptr(gate_out), _ptr(slots), n, nq,
-         nkv, dk, dv, page_size, 1 if write else 0, _stream())
+         nkv, dk, dv, page_size, 1 if write else 0, int(bool(single)), _stream())
 
 
 def retention_prepare(proj: Partials, col0: int, log_decay: torch.Tensor, cos: torch.Tensor | None,
                       sin: torch.Tensor | None, rot: int, neighbours: bool, positions: torch.Tensor, kscale: float,
-                      x: torch.Tensor, n: int, heads: int, dk: int, dv: int) -> None:
+                      x: torch.Tensor, n: int, heads: int, dk: int, dv: int, silu: bool = False) -> None:
     """Finish the input product from column ``col0`` on (q, k: heads*dk each; v, g: heads*dv each) into the float32 rows
-    [q | k | log decay | v | g] that the recurrent kernels share: the first ``rot`` elements of every query and key head
+    [q | k | log decay | v | g] that the recurrent kernels share: q, k and v through silu (``silu``), the first ``rot`` elements of every query and key head
     turned by position, the keys then times ``kscale``; every key channel of head h gets ``log_decay[h]``."""
     _dev(proj.data, log_decay, cos, sin, positions, x)
     args = _proj_args(proj, col0, 2 * heads * dk + 2 * heads * dv)
@@ -1479,7 +1507,8 @@ def retention_prepare(proj: Partials, col0: int, log_decay: torch.Tensor, cos: t
             raise KernelError("retention_prepare: cos and sin are float32 [positions, rot / 2], rot even and within the head")
         _contig("cos", cos), _contig("sin", sin)
     call("pyre_retention_prepare", *args, log_decay.data_ptr(), _ptr(cos) if rot else None, _ptr(sin) if rot else None,
-         int(rot), int(bool(neighbours)), positions.data_ptr(), float(kscale), x.data_ptr(), n, heads, dk, dv, _stream())
+         int(rot), int(bool(neighbours)), positions.data_ptr(), float(kscale), int(bool(silu)), x.data_ptr(), n, heads, dk,
+         dv, _stream())
 
 
 def route_grouped(z: Partials, correction: torch.Tensor | None, gates: torch.Tensor, n: int, top: int, groups: int,
@@ -1700,3 +1729,102 @@ def token_side_gate(z: Partials, table: torch.Tensor, first: int, ids: torch.Ten
     _contig("out", out), _i32("ids", ids, n)
     call("pyre_token_side_gate", *z._args(dim), table.data_ptr(), dtype_code(table), table.shape[1], int(first),
          ids.data_ptr(), out.data_ptr(), dtype_code(out), n, dim, _stream())
+
+
+SSM_MAX_STATE = 256      #: the largest state of a channel that the selective scan's kernels take (selective_scan.hip)
+SSM_MAX_SELECTED = 12288  #: the most columns (rank of the step sizes and twice the state) of its second product
+
+
+def _ssm_columns(what: str, p: Partials, n: int, first: int, width: int):
+    if p.bias is not None:
+        raise KernelError(f"{what}: a product with a pending bias is not taken")
+    if p.rows < n or first < 0 or first + width > p.width:
+        raise KernelError(f"{what}: columns {first}..{first + width} of {n} rows lie outside the product's [{p.rows}, {p.width}]")
+    _dev(p.data)
+    return (p.data.data_ptr(), dtype_code(p.data), p.count, p.stride)
+
+
+def _ssm_f32(what: str, **tensors) -> None:
+    for name, (t, shape) in tensors.items():
+        _dev(t), _contig(name, t)
+        if t.dtype != torch.float32 or tuple(t.shape) != tuple(shape):
+            raise KernelError(f"{what}: {name} is contiguous float32 {list(shape)}, not {t.dtype} {list(t.shape)}")
+
+
+def ssm_conv(proj: Partials, col0: int, taps_w: torch.Tensor, conv_b: torch.Tensor, conv_state: torch.Tensor | None,
+             state_slots: torch.Tensor, seq_of_token: torch.Tensor, q_start: torch.Tensor, n_seqs: int, x: torch.Tensor, n: int,
+             single: bool = False) -> None:
+    """x[n, inner] = silu(causal convolution over the request's tokens of the product's ``inner`` columns from ``col0`` on,
+    + ``conv_b``). ``taps_w`` float32 [taps, inner]; inputs before the step come from ``conv_state`` (float32 [slots, taps - 1,
+    inner]), which is brought up to date. ``single`` as for :func:`conv_qkv_write`."""
+    taps, inner = taps_w.shape
+    args = _ssm_columns("ssm_conv", proj, n, col0, inner)
+    _ssm_f32("ssm_conv", taps_w=(taps_w, (taps, inner)), conv_b=(conv_b, (inner,)))
+    if not 1 <= taps <= CONV_MAX_TAPS:
+        raise KernelError(f"ssm_conv: {taps} taps are outside 1..{CONV_MAX_TAPS}")
+    if taps > 1:
+        if conv_state is None:
+            raise KernelError("ssm_conv: more than one tap needs the requests' states")
+        _ssm_f32("ssm_conv", conv_state=(conv_state, (conv_state.shape[0], taps - 1, inner)))
+    _dev(state_slots, seq_of_token, q_start, x), _contig("x", x)
+    _i32("seq_of_token", seq_of_token, n), _i32("q_start", q_start, n_seqs + 1), _i32("state_slots", state_slots, n_seqs)
+    if x.shape[-1] != inner or x.shape[0] < n:
+        raise KernelError(f"ssm_conv: x is [>= {n}, {inner}]")
+    if single and n != n_seqs:
+        raise KernelError(f"ssm_conv: {n} tokens of {n_seqs} requests are not one token each")
+    call("pyre_ssm_conv", *args, proj.width, int(col0), taps_w.data_ptr(), taps, conv_b.data_ptr(),
+         conv_state.data_ptr() if taps > 1 else None, state_slots.data_ptr(), seq_of_token.data_ptr(), q_start.data_ptr(),
+         n_seqs, int(bool(single)), x.data_ptr(), dtype_code(x), n, inner, _stream())
+
+
+def ssm_low(sel: Partials, rank: int, out: torch.Tensor, n: int) -> None:
+    """The first ``rank`` columns of the product ``sel`` as operands of the next one: ``out`` float32 [n, padded], or
+    bfloat16 [n, 2 * padded] with what the rounding left in the second half; zeros from ``rank`` to ``padded``."""
+    args = _ssm_columns("ssm_low", sel, n, 0, rank)
+    _dev(out), _contig("out", out)
+    padded = out.shape[-1] if out.dtype == torch.float32 else out.shape[-1] // 2
+    if out.shape[0] < n or padded < rank or (out.dtype == torch.bfloat16 and out.shape[-1] % 2):
+        raise KernelError(f"ssm_low: out {tuple(out.shape)} does not hold {n} rows of {rank} columns")
+    call("pyre_ssm_low", *args, sel.width, out.data_ptr(), dtype_code(out), int(rank), int(padded), n, _stream())
+
+
+def _ssm_common(what, x, sel, rank, gate, g0, A2, D, dt_b, state, out, n, inner, n_state):
+    if not 0 < n_state <= SSM_MAX_STATE or not 0 < rank <= SSM_MAX_SELECTED - 2 * n_state:
+        raise KernelError(f"{what}: a state of {n_state} beside a rank of {rank} is not taken")
+    _ssm_f32(what, A2=(A2, (inner, n_state)), D=(D, (inner,)), dt_b=(dt_b, (inner,)), state=(state, (state.shape[0], inner, n_state)))
+    _dev(x, out), _contig("x", x)
+    if x.shape[-1] != inner or x.shape[0] < n or out.dim() != 2 or out.stride(1) != 1 or out.shape[1] < inner or out.shape[0] < n:
+        raise KernelError(f"{what}: x is [>= {n}, {inner}], out [>= {n}, >= {inner}] with contiguous rows")
+    return (_ssm_columns(what, sel, n, 0, rank + 2 * n_state), _ssm_columns(what, gate, n, g0, inner))
+
+
+def ssm_scan(z: Partials, dt_b: torch.Tensor, x: torch.Tensor, sel: Partials, rank: int, gate: Partials, g0: int,
+             A2: torch.Tensor, D: torch.Tensor, state: torch.Tensor, q_start: torch.Tensor, state_slots: torch.Tensor,
+             n_seqs: int, out_scale: float, out: torch.Tensor, n: int) -> None:
+    """The selective scan over each request's tokens of the step, from and into ``state`` [slots, inner, N] (float32):
+    dt = softplus(z + dt_b); S <- exp(dt A) S + dt x B; out = (S C + D x) * silu(gate columns from ``g0`` on) * out_scale.
+    ``sel`` holds [rank | B | C]; ``A2`` = A * log2(e), float32 [inner, N]; ``x`` [N, inner] as :func:`ssm_conv` leaves it."""
+    inner, n_state = A2.shape
+    s, g = _ssm_common("ssm_scan", x, sel, rank, gate, g0, A2, D, dt_b, state, out, n, inner, n_state)
+    zp = _ssm_columns("ssm_scan", z, n, 0, inner)
+    if z.width != inner:
+        raise KernelError("ssm_scan: the step sizes' product is as wide as the channels")
+    _i32("q_start", q_start, n_seqs + 1), _i32("state_slots", state_slots, n_seqs), _dev(q_start, state_slots)
+    call("pyre_ssm_scan", *zp, dt_b.data_ptr(), x.data_ptr(), dtype_code(x), *s, sel.width, int(rank), *g, gate.width, int(g0),
+         A2.data_ptr(), D.data_ptr(), state.data_ptr(), q_start.data_ptr(), state_slots.data_ptr(), n_seqs, float(out_scale),
+         out.data_ptr(), dtype_code(out), out.stride(0), inner, n_state, _stream())
+
+
+def ssm_step(dt_w: torch.Tensor, dt_b: torch.Tensor, x: torch.Tensor, sel: Partials, rank: int, gate: Partials, g0: int,
+             A2: torch.Tensor, D: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor, n_seqs: int, out_scale: float,
+             out: torch.Tensor) -> None:
+    """:func:`ssm_scan` for a step of one token a request (token i is request i's), the step sizes' product inside:
+    ``dt_w`` [inner, >= rank] with contiguous rows."""
+    inner, n_state = A2.shape
+    s, g = _ssm_common("ssm_step", x, sel, rank, gate, g0, A2, D, dt_b, state, out, n_seqs, inner, n_state)
+    _dev(dt_w, state_slots), _i32("state_slots", state_slots, n_seqs)
+    if dt_w.dim() != 2 or dt_w.shape[0] != inner or dt_w.shape[1] < rank or dt_w.stride(1) != 1:
+        raise KernelError(f"ssm_step: the step sizes' matrix is [{inner}, >= {rank}] with contiguous rows")
+    call("pyre_ssm_step", dt_w.data_ptr(), dtype_code(dt_w), dt_w.stride(0), dt_b.data_ptr(), x.data_ptr(), dtype_code(x), *s,
+         sel.width, int(rank), *g, gate.width, int(g0), A2.data_ptr(), D.data_ptr(), state.data_ptr(), state_slots.data_ptr(),
+         n_seqs, float(out_scale), out.data_ptr(), dtype_code(out), out.stride(0), inner, n_state, _stream())

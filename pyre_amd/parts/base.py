@@ -255,7 +255,7 @@ class Block(Part):
 # --------------------------------------------------------------------------- registry of parts
 
 _PARTS: dict[tuple[str, str], type] = {}
-ROLES = ("mixer", "feed_forward", "norm", "position", "block", "embedding", "head", "token_input")
+ROLES = ("mixer", "feed_forward", "norm", "position", "block", "embedding", "head", "token_input", "pass_input")
 
 
 def register_part(role: str, kind: str, cls: type) -> None:
@@ -315,6 +315,10 @@ class RotarySpec:
     #: positions are divided by ``factor``, those that turn more than ``fast`` times stay, those between are blended
     #: linearly by their index; cosines and sines are multiplied by 0.1 ln(factor) + 1. None: plain frequencies.
     scaling: tuple | None = None
+    #: (factor, low, high, original): frequencies changed by their wavelength 2 pi / f instead: those shorter than
+    #: original / high stay, those longer than original / low are divided by ``factor``, those between are blended linearly
+    #: in original / wavelength. None: not.
+    wave_scaling: tuple | None = None
     kind: ClassVar[str] = "rotary"
 
 
@@ -467,6 +471,16 @@ class GeluGLUSpec:
 
 
 @dataclass(frozen=True)
+class ReluGLUSpec:
+    """down(relu(gate(x)) * up(x)), no biases. Tensors: ``prefix + .gate / .up / .down``."""
+
+    hidden_size: int
+    intermediate_size: int
+    prefix: str
+    kind: ClassVar[str] = "relu_glu"
+
+
+@dataclass(frozen=True)
 class SigmoidMoESpec:
     """A mixture of ``experts`` feed-forward layers down(relu(up(x))^2) of ``expert_size`` hidden units each: every
     token goes through the ``top`` experts of largest sigmoid(router(x)), weighted by these scores over their sum
@@ -489,7 +503,7 @@ class SinkAttentionSpec:
     through a causal convolution over time, ``conv_taps`` taps per channel (0: none), whose last ``conv_taps - 1``
     inputs a request keeps as state; queries and keys are then divided by their root mean square per head, times a
     gain over ``key_dim`` that the heads share (``qk_norm``), and turned by position (``position``: either pairing).
-    The heads' outputs are multiplied element by element with sigmoid(G h) (``gated``). Tensors: ``prefix + .q / .k /
+    Scores are squashed by ``softcap * tanh(s / softcap)`` (0: not; the sink is not). The heads' outputs are multiplied element by element with sigmoid(G h) (``gated``). Tensors: ``prefix + .q / .k /
     .v / .g / .o / .sink / .q.norm / .k.norm / .q.conv / .k.conv / .v.conv``."""
 
     hidden_size: int
@@ -506,6 +520,7 @@ class SinkAttentionSpec:
     norm_eps: float = 1e-6
     sink: bool = True
     gated: bool = True
+    softcap: float = 0.0
     kind: ClassVar[str] = "sink_attention"
 
 
@@ -525,6 +540,40 @@ class RetentionSpec:
     prefix: str
     norm_eps: float = 1e-6
     kind: ClassVar[str] = "retention"
+
+
+@dataclass(frozen=True)
+class LightningAttentionSpec:
+    """Linear attention with one fixed decay per head: S <- decay_h S + k v^T, o = S^T q with S [key_dim, value_dim]
+    float32 per head and request; q, k, v = silu of their projections. The heads' o are divided by their root mean square
+    over all heads at once, times a gain over heads * value_dim, times sigmoid(G h). Tensors: ``prefix + .q / .k / .v / .g /
+    .o / .norm``."""
+
+    hidden_size: int
+    num_heads: int
+    key_dim: int
+    value_dim: int
+    decay: tuple
+    prefix: str
+    norm_eps: float = 1e-6
+    position: Any = NoPositionSpec()
+    kind: ClassVar[str] = "lightning_attention"
+
+
+@dataclass(frozen=True)
+class SelectiveScanSpec:
+    """Per channel c of ``inner`` a float32 state S [state]: S <- exp(dt_c A[c]) S + dt_c x_c B, y_c = S . C + D_c x_c.
+    [x | z] = W_in h; x goes through a short causal convolution (``conv_taps`` per channel, with a bias) and silu;
+    [low | B | C] = W_x x with ``dt_rank`` columns of low, dt = softplus(W_dt low + b); A = -exp(A_log). The result is
+    y silu(z). Tensors: ``prefix + .in / .conv / .conv.b / .x / .dt / .dt.b / .A_log / .D / .o``."""
+
+    hidden_size: int
+    inner: int
+    state: int
+    dt_rank: int
+    conv_taps: int
+    prefix: str
+    kind: ClassVar[str] = "selective_scan"
 
 
 @dataclass(frozen=True)
@@ -779,10 +828,15 @@ class HyperConnectionBlockSpec:
 
 @dataclass(frozen=True)
 class EmbeddingSpec:
+    """``places_name``: a table of ``places`` rows, of which a token's position takes one that is added as it is (None: no
+    such table); no request can then be longer than the table."""
+
     vocab_size: int
     hidden_size: int
     name: str = "model.embed_tokens.weight"
     scale: float = 1.0               #: the table's rows are multiplied by this
+    places: int = 0
+    places_name: str | None = None
     kind: ClassVar[str] = "embedding"
 
 
@@ -827,6 +881,18 @@ class LayerCall:
 
     layer: int
     cache_from: int | None = None
+    #: the residual stream goes through the model's ``pass_input`` first (the first layer of a pass of a loop)
+    enters: bool = False
+
+
+@dataclass(frozen=True)
+class PassInputSpec:
+    """What stands before a pass of looped layers: x <- W [x; x0], x the residual stream and x0 the embedding's output.
+    Tensor: ``name`` [hidden, 2 hidden]."""
+
+    hidden_size: int
+    name: str
+    kind: ClassVar[str] = "pass_input"
 
 
 @dataclass(frozen=True)
@@ -842,4 +908,6 @@ class ModelSpec:
     #: streams of the residual (blocks of hyper-connections); 0: the residual is one row a token. All streams are the
     #: embedding's output at the start, and the final norm reads their sum
     streams: int = 0
+    #: what stands before the entries of the order that say so (``LayerCall.enters``)
+    pass_input: Any = None
     extra: dict = field(default_factory=dict, compare=False)

@@ -24,6 +24,17 @@ class Hidden:
     weights: object = None
 
 
+def without_bias(ctx, pending: Partials | None) -> Partials | None:
+    """The pending term for a kernel that takes no pending bias: summed first if it has one."""
+    if pending is None or pending.bias is None:
+        return pending
+    from pyre_amd.hip import ops
+
+    full = ctx.workspace.get("block.sum", (1, ctx.n_tokens, pending.width), torch.float32)
+    ops.reduce_partials(pending, full[0], ctx.n_tokens)
+    return Partials(full, None, pending.post, pending.scale, pending.more, pending.outer)
+
+
 class PreNormBlock(Block):
     """x += mixer(norm1(x)); x += feed_forward(norm2(x)), the second half only if the layer has a feed-forward. A layer
     may have a third sublayer that reads the residual stream itself and the step's tokens (``token_input``): the kernel
@@ -81,12 +92,8 @@ class PreNormBlock(Block):
             return
         from pyre_amd.hip import ops
 
-        pending = state.pending
-        if pending is not None and pending.bias is not None:  # the kernel below takes no pending bias: summed first
-            full = ctx.workspace.get("block.sum", (1, ctx.n_tokens, state.resid.shape[1]), torch.float32)
-            ops.reduce_partials(pending, full[0], ctx.n_tokens)
-            pending = Partials(full)
-        ops.add_rms_terms(state.resid, pending, None, 0.0, h)   # the pending term joins the stream; h = the stream
+        # the pending term joins the stream; h = the stream
+        ops.add_rms_terms(state.resid, without_bias(ctx, state.pending), None, 0.0, h)
         term = self.token_input.forward(ctx, h)
         norm = self.token_input_norm
         state.pending = Partials(term.data, term.bias, PostNorm(norm.gain, norm.spec.eps, kind="rms"))

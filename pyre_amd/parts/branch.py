@@ -54,6 +54,10 @@ class BranchMixer(Mixer):
     def attend(self, ctx, proj: Partials, col0: int, cache, o: torch.Tensor, scale: float) -> None:
         raise NotImplementedError
 
+    def inner_linears(self) -> list:
+        """Products that ``attend`` runs itself."""
+        return []
+
     def cache_specs(self) -> list:
         """What the mixer keeps, one description per cache (a mixer with pages and a state of its own has two);
         ``attend`` gets the one view, or the list of them if there are several."""
@@ -82,7 +86,7 @@ class BranchMixer(Mixer):
         self.bind_others(tensors, runtime)
 
     def linears(self) -> list:
-        return [self._in, self._out]
+        return [self._in, *self.inner_linears(), self._out]
 
     def forward(self, ctx, h, cache):
         n = ctx.n_tokens
@@ -205,7 +209,8 @@ class ParallelMixer(Mixer):
             b.bind_others(tensors, runtime)
 
     def linears(self) -> list:
-        return [self.proj, *([self.out] if self.out is not None else self.outs)]
+        return [self.proj, *(lin for b in self.branches for lin in b.inner_linears()),
+                *([self.out] if self.out is not None else self.outs)]
 
     def forward(self, ctx, h, caches):
         n = ctx.n_tokens

@@ -7,12 +7,14 @@ from pyre_amd.parts.branch import ParallelMixer
 from pyre_amd.parts.capped_attention import CappedAttention
 from pyre_amd.parts.delta_rule import GatedDeltaRule
 from pyre_amd.parts.embedding import BigramEmbedding, LMHead, TokenEmbedding
-from pyre_amd.parts.feedforward import ClippedGLU, GeluGLU, PolyNormMLP, ReluSquaredMLP, SwiGLU
+from pyre_amd.parts.feedforward import ClippedGLU, GeluGLU, PolyNormMLP, ReluGLU, ReluSquaredMLP, SwiGLU
 from pyre_amd.parts.latent_attention import LatentAttention
-from pyre_amd.parts.linear_attention import GatedLinearAttention, Retention
+from pyre_amd.parts.linear_attention import GatedLinearAttention, LightningAttention, Retention
 from pyre_amd.parts.moe import GroupedSoftmaxMoE, SigmoidMoE, SoftmaxTopKMoE
 from pyre_amd.parts.norm import LayerNorm, RMSNorm, TanhNorm
+from pyre_amd.parts.pass_input import PassInput
 from pyre_amd.parts.rotary import NoPosition, RotaryEncoding
+from pyre_amd.parts.selective_scan import SelectiveScan
 from pyre_amd.parts.sink_attention import SinkAttention
 from pyre_amd.parts.streams import HyperConnectionBlock
 from pyre_amd.parts.tied_attention import TiedAttention
@@ -51,3 +53,7 @@ register_part("feed_forward", "softmax_topk_moe", SoftmaxTopKMoE)
 register_part("token_input", "token_side", TokenSide)
 register_part("feed_forward", "poly_norm_mlp", PolyNormMLP)
 register_part("block", "hyper_connections", HyperConnectionBlock)
+register_part("mixer", "lightning_attention", LightningAttention)
+register_part("mixer", "selective_scan", SelectiveScan)
+register_part("feed_forward", "relu_glu", ReluGLU)
+register_part("pass_input", "pass_input", PassInput)

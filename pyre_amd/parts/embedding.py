@@ -10,19 +10,32 @@ from pyre_amd.parts.linear import Linear
 
 
 class TokenEmbedding(Part):
+    """table[token] * scale, joined by a learned row per position if the description names a table of them."""
+
     def __init__(self, spec: EmbeddingSpec):
+        if (spec.places_name is not None) != (spec.places > 0):
+            raise ValueError("embedding: a table of positions needs a name and rows")
         self.spec = spec
-        self.table = None
+        self.table = self.places = None
+
+    @property
+    def max_positions(self) -> int:
+        """Positions that the tables have rows for (0: no such bound); the engine takes no longer request."""
+        return self.spec.places
 
     def tensor_specs(self) -> list[TensorSpec]:
-        return [TensorSpec(self.spec.name, (self.spec.vocab_size, self.spec.hidden_size))]
+        s = self.spec
+        specs = [TensorSpec(s.name, (s.vocab_size, s.hidden_size))]
+        return specs + ([TensorSpec(s.places_name, (s.places, s.hidden_size))] if s.places_name else [])
 
     def bind(self, tensors, runtime) -> None:
         self.table = tensors[self.spec.name].contiguous()
+        if self.spec.places_name:
+            self.places = tensors[self.spec.places_name].to(self.table.dtype).contiguous()
 
     def forward(self, ctx, resid: torch.Tensor) -> None:
-        """resid[n] = float32(table[token n]) * scale: the residual stream starts here."""
-        ops.embed(self.table, ctx.tokens, resid, self.spec.scale)
+        """resid[n] = float32(table[token n]) * scale (+ the position's row): the residual stream starts here."""
+        ops.embed(self.table, ctx.tokens, resid, self.spec.scale, ctx.positions, self.places)
 
 
 class BigramEmbedding(Part):

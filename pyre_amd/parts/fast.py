@@ -94,7 +94,8 @@ LIBRARY_F32_ROLES = frozenset({"attn.qkv", "attn.out", "mix.in", "mix.out", "cat
                                "moe.down", "mix.out0", "mix.out1", "sattn.in", "sattn.out", "ret.in", "ret.out",
                                "relu2.down", "gmoe.router", "gmoe.down", "wattn.in", "wattn.out", "gdr.in", "gdr.out",
                                "stmoe.router", "stmoe.down", "side.gate", "side.proj", "lattn.q_up", "poly.up",
-                               "poly.down"})
+                               "poly.down", "light.in", "light.out", "ssm.in", "ssm.out", "ssm.x", "ssm.dt", "reglu.down",
+                               "pass.start", "pass.stream"})
 
 
 def _is_bf16(ctx, lin, x) -> bool:

@@ -6,8 +6,8 @@ import torch
 
 from pyre_amd.hip import ops
 from pyre_amd.parts import fast
-from pyre_amd.parts.base import (ClippedGLUSpec, FeedForward, GeluGLUSpec, PolyNormMLPSpec, ReluSquaredMLPSpec, SwiGLUSpec,
-                                 TensorSpec, take)
+from pyre_amd.parts.base import (ClippedGLUSpec, FeedForward, GeluGLUSpec, PolyNormMLPSpec, ReluGLUSpec, ReluSquaredMLPSpec,
+                                 SwiGLUSpec, TensorSpec, take)
 from pyre_amd.parts.linear import Linear, linear_specs
 
 
@@ -88,11 +88,12 @@ class GeluGLU(FeedForward):
     few rows finishes the unit in that product's epilogue."""
 
     UNIT = (0.0, ops.GELU_TANH_SLOPE, 0.0, ops.GELU_TANH_CUBIC)  #: no clipping, no shift
+    DOWN_ROLE = "geglu.down"
 
     def __init__(self, spec: GeluGLUSpec):
         self.spec = spec
         self.gate_up = Linear(spec.hidden_size, 2 * spec.intermediate_size, "ffn.gate_up")
-        self.down = Linear(spec.intermediate_size, spec.hidden_size, "geglu.down")
+        self.down = Linear(spec.intermediate_size, spec.hidden_size, self.DOWN_ROLE)
 
     def tensor_specs(self) -> list[TensorSpec]:
         s, p = self.spec, self.spec.prefix
@@ -119,6 +120,16 @@ class GeluGLU(FeedForward):
             limit, slope, shift, cubic = self.UNIT
             ops.clipped_glu(gu, act, n, limit, slope, shift, cubic)
         return self.down.forward(ctx, act, n)
+
+
+class ReluGLU(GeluGLU):
+    """down(relu(gate(x)) * up(x)): the same with the unit whose sigmoid is a step."""
+
+    UNIT = (0.0, ops.RELU_SLOPE, 0.0, 0.0)
+    DOWN_ROLE = "reglu.down"
+
+    def __init__(self, spec: ReluGLUSpec):
+        super().__init__(spec)
 
 
 class ReluSquaredMLP(FeedForward):

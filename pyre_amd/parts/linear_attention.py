@@ -7,7 +7,8 @@ import torch
 from pyre_amd.hip import ops
 import math
 
-from pyre_amd.parts.base import GatedLinearAttentionSpec, RetentionSpec, StateCacheSpec, TensorSpec, make_part, take
+from pyre_amd.parts.base import (GatedLinearAttentionSpec, LightningAttentionSpec, RetentionSpec, StateCacheSpec, TensorSpec,
+                                 make_part, take)
 from pyre_amd.parts.branch import BranchMixer
 
 #: columns of the decay's low-rank product that the random-weights mode draws when a description leaves them to the file
@@ -87,10 +88,10 @@ class Retention(BranchMixer):
 
     def __init__(self, spec: RetentionSpec):
         if not (0 < spec.key_dim <= ops.GLA_MAX_KEY_HEAD and 0 < spec.value_dim <= ops.GLA_MAX_VALUE_HEAD):
-            raise ValueError(f"retention: head sizes {spec.key_dim} / {spec.value_dim} are outside "
+            raise ValueError(f"{spec.kind}: head sizes {spec.key_dim} / {spec.value_dim} are outside "
                              f"1..{ops.GLA_MAX_KEY_HEAD} / 1..{ops.GLA_MAX_VALUE_HEAD}")
         if spec.num_heads <= 0 or len(spec.decay) != spec.num_heads or not all(0.0 < float(d) <= 1.0 for d in spec.decay):
-            raise ValueError("retention: one decay in (0, 1] per head")
+            raise ValueError(f"{spec.kind}: one decay in (0, 1] per head")
         self.spec = spec
         self.hidden_size = spec.hidden_size
         self.inner = spec.num_heads * spec.value_dim
@@ -123,12 +124,44 @@ class Retention(BranchMixer):
         shape = (s.num_heads, s.key_dim, s.value_dim)
         x = ws.get("ret.x", (n, ops.gla_row_width(*shape)), torch.float32)
         raw = ws.get("ret.raw", (n, s.num_heads * s.value_dim), torch.float32)
-        cos, sin, rot = self.position.rotary(ctx.runtime)
-        ops.retention_prepare(proj, col0, self.log_decay, cos, sin, rot, self.neighbours, ctx.positions,
-                              s.key_dim ** -0.5, x, n, *shape)
+        self.prepare(ctx, proj, col0, x, n, shape)
         pairs = None
         if ctx.host.max_q_len > 1:
             pairs = ws.get("ret.chunks", (ops.gla_chunks_scratch(n, ctx.n_seqs, *shape),), torch.float32)
         ops.gla_scan(x, cache.tensor, raw, ctx.q_start, cache.slots, ctx.n_seqs, *shape, 1.0, chunks=pairs,
                      max_tokens=ctx.host.max_q_len, decay=self.decay)
-        ops.gla_finish(raw, x, None, s.norm_eps, scale, o, n, *shape)
+        self.finish(raw, x, scale, o, n, shape)
+
+    def prepare(self, ctx, proj, col0, x, n, shape) -> None:
+        cos, sin, rot = self.position.rotary(ctx.runtime)
+        ops.retention_prepare(proj, col0, self.log_decay, cos, sin, rot, self.neighbours, ctx.positions,
+                              self.spec.key_dim ** -0.5, x, n, *shape)
+
+    def finish(self, raw, x, scale, o, n, shape) -> None:
+        ops.gla_finish(raw, x, None, self.spec.norm_eps, scale, o, n, *shape)
+
+
+class LightningAttention(Retention):
+    """The same recurrence behind silu on queries, keys and values, without positions and without a scale; all heads' o
+    are normed together (one gain over all of them) and multiplied by sigmoid(G h)."""
+
+    role = "light"
+
+    def __init__(self, spec: LightningAttentionSpec):
+        super().__init__(spec)
+        self.gain = None
+
+    def other_tensors(self):
+        return [TensorSpec(f"{self.spec.prefix}.norm", (self.inner,), init="gain")]
+
+    def bind_others(self, tensors, runtime) -> None:
+        super().bind_others(tensors, runtime)
+        self.gain = take(tensors, f"{self.spec.prefix}.norm").contiguous()
+
+    def prepare(self, ctx, proj, col0, x, n, shape) -> None:
+        cos, sin, rot = self.position.rotary(ctx.runtime)
+        ops.retention_prepare(proj, col0, self.log_decay, cos, sin, rot, self.neighbours, ctx.positions, 1.0, x, n, *shape,
+                              silu=True)
+
+    def finish(self, raw, x, scale, o, n, shape) -> None:
+        ops.gla_finish_wide(raw, x, self.gain, self.spec.norm_eps, scale, o, n, *shape)

@@ -27,7 +27,10 @@ class LayeredModel(Part):
                     any(c.streams != spec.streams for c in getattr(b, "connections", ())):
                 raise ValueError(f"a layer's connections do not fit the model's {spec.streams} streams")
         self.head = make_part("head", spec.head)
+        self.pass_input = make_part("pass_input", spec.pass_input) if spec.pass_input is not None else None
         self.schedule = list(spec.schedule)
+        if any(call.enters for call in self.schedule) and (self.pass_input is None or spec.streams):
+            raise ValueError("an entry of the order that enters a pass needs the model's pass_input and a residual of one row")
         for pos, call in enumerate(self.schedule):
             if not (0 <= call.layer < len(self.layers)):
                 raise ValueError(f"order entry {pos} names layer {call.layer}, there are {len(self.layers)}")
@@ -35,7 +38,8 @@ class LayeredModel(Part):
                 raise ValueError(f"order entry {pos} reads the cache of entry {call.cache_from}, which does not precede it")
 
     def parts(self):
-        return (self.embedding, *self.layers, self.final_norm, self.head)
+        passes = () if self.pass_input is None else (self.pass_input,)
+        return (self.embedding, *passes, *self.layers, self.final_norm, self.head)
 
     def tensor_specs(self) -> list[TensorSpec]:
         seen: dict[str, TensorSpec] = {}
@@ -106,7 +110,10 @@ class LayeredModel(Part):
         else:
             self.embedding.forward(ctx, resid)
         state = Hidden(resid, streams=self.spec.streams)
+        start = self.pass_input.start(ctx, state) if self.pass_input is not None else None
         for pos, call in enumerate(self.schedule):
+            if call.enters:
+                self.pass_input.enter(ctx, state, start)
             self.layers[call.layer].forward(ctx, state, caches[pos])
             if tap is not None:
                 tap(pos, self._hidden_rows(ctx, state))

@@ -32,15 +32,29 @@ def scaled_frequencies(inv: torch.Tensor, rotary_dim: int, theta: float, scaling
     return inv / factor * ramp + inv * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
 
 
+def wave_scaled_frequencies(inv: torch.Tensor, scaling: tuple) -> torch.Tensor:
+    """The frequencies ``inv`` (float64, one per pair) changed by their wavelength l = 2 pi / f: kept where l < original /
+    high, divided by ``factor`` where l > original / low; between the two (1 - s) f / factor + s f with s = (original / l -
+    low) / (high - low)."""
+    factor, low, high, original = (float(x) for x in scaling)
+    wave = 2.0 * math.pi / inv
+    s = (original / wave - low) / (high - low) if high != low else torch.zeros_like(inv)
+    mixed = (1.0 - s) * inv / factor + s * inv
+    return torch.where(wave < original / high, inv, torch.where(wave > original / low, inv / factor, mixed))
+
+
 def rotary_tables(rotary_dim: int, theta: float, n_positions: int, exact: bool = False,
-                  scaling: tuple | None = None) -> tuple[torch.Tensor, torch.Tensor]:
+                  scaling: tuple | None = None, wave_scaling: tuple | None = None) -> tuple[torch.Tensor, torch.Tensor]:
     """cos, sin of shape [n_positions, rotary_dim / 2], float32, on the CPU. ``exact``: the angles are formed in
-    float64 and only their cosines and sines are rounded. ``scaling`` (always exact): see :func:`scaled_frequencies`."""
-    if exact or scaling is not None:
+    float64 and only their cosines and sines are rounded. ``scaling`` (always exact): see :func:`scaled_frequencies`;
+    ``wave_scaling`` (likewise): see :func:`wave_scaled_frequencies`."""
+    if exact or scaling is not None or wave_scaling is not None:
         inv = theta ** (-torch.arange(0, rotary_dim, 2, dtype=torch.float64) / rotary_dim)
         mag = 1.0
         if scaling is not None:
             inv, mag = scaled_frequencies(inv, rotary_dim, theta, scaling)
+        if wave_scaling is not None:
+            inv = wave_scaled_frequencies(inv, wave_scaling)
         freqs = torch.outer(torch.arange(n_positions, dtype=torch.float64), inv)
         return (freqs.cos() * mag).float(), (freqs.sin() * mag).float()
     inv_freq = 1.0 / (theta ** (torch.arange(0, rotary_dim, 2, dtype=torch.float32) / rotary_dim))
@@ -60,7 +74,8 @@ class RotaryEncoding(PositionEncoding):
     def rotary(self, runtime):
         n = runtime.max_positions  # the engine's longest request decides, as the reference's table grows on demand
         if self._tables is None or self._tables[0].shape[0] < n or self._tables[0].device != runtime.device:
-            cos, sin = rotary_tables(self.rotary_dim, self.spec.theta, n, self.spec.exact, getattr(self.spec, "scaling", None))
+            cos, sin = rotary_tables(self.rotary_dim, self.spec.theta, n, self.spec.exact, getattr(self.spec, "scaling", None),
+                                     getattr(self.spec, "wave_scaling", None))
             self._tables = (cos.to(runtime.device).contiguous(), sin.to(runtime.device).contiguous())
         return self._tables[0], self._tables[1], self.rotary_dim
 

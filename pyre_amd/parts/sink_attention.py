@@ -14,7 +14,8 @@ from pyre_amd.parts.branch import BranchMixer
 
 class SinkAttention(BranchMixer):
     """q, k, v, g = split(h W^T); q, k, v <- conv over time; q, k <- RMS norm per head, turned by position;
-    out = softmax over (the window's keys and a sink) of (q k^T scale) v, times sigmoid(g); then the output matrix.
+    out = softmax over (the window's keys and a sink) of (q k^T scale, squashed if a cap is given) v, times sigmoid(g);
+    then the output matrix.
 
     Keeps two things per request: pages of keys (normed and turned) and values (after the convolution), of which
     those that the window has passed go back to the pool, and the last ``taps - 1`` projected rows, which the
@@ -30,6 +31,8 @@ class SinkAttention(BranchMixer):
                 raise ValueError(f"sink attention: {name} {v} is outside 1..{ops.ATTN_MAX_HEAD_DIM}")
         if spec.window < 0 or not (0 <= spec.conv_taps <= ops.CONV_MAX_TAPS):
             raise ValueError(f"sink attention: the window must not be negative, the taps lie in 0..{ops.CONV_MAX_TAPS}")
+        if spec.softcap < 0:
+            raise ValueError("sink attention: the cap on the scores must not be negative")
         self.spec = spec
         self.hidden_size = spec.hidden_size
         self.inner = spec.num_heads * spec.value_dim
@@ -100,8 +103,8 @@ class SinkAttention(BranchMixer):
                            ctx.seq_of_token, ctx.q_start, ctx.n_seqs, self.q_gain, self.k_gain, s.norm_eps, cos, sin, rot,
                            self.neighbours, ctx.positions, q, k_pages if pages.writes else None,
                            v_pages if pages.writes else None, gate, pages.slots, n, s.num_heads, s.num_kv_heads, s.key_dim,
-                           s.value_dim, pages.page_size)
-        shape = (s.num_heads, s.num_kv_heads, s.key_dim, s.value_dim, pages.page_size, s.scale, 0.0, None, 0, s.window, 0)
+                           s.value_dim, pages.page_size, single=ctx.host.max_q_len == 1 and n == ctx.n_seqs)
+        shape = (s.num_heads, s.num_kv_heads, s.key_dim, s.value_dim, pages.page_size, s.scale, s.softcap, None, 0, s.window, 0)
         extra = dict(sink=self.sink, gate_dim=s.value_dim if s.gated else 1)
         tiles = ctx.host.arrays["attention.prefill_tiles"]
         singles = ctx.host.arrays["attention.decode_tokens"]
