@@ -386,9 +386,10 @@ int pyre_gla_finish_wide(const float* o, const float* x, const void* gain, int g
 
 // ---- a selective scan (selective_scan.hip) ----
 // x[n, inner] = silu(conv over time of the product's columns from col0 on + conv_b); state [slots][taps - 1][inner] is
-// brought up to date. `single`: the step brings one token a request.
-int pyre_ssm_conv(const void* proj, int proj_dt, int n_partials, long partial_stride, int ld, int col0, const float* taps_w,
-                  int taps, const float* conv_b, float* conv_state, const int* state_slots, const int* seq_of_token,
+// brought up to date. `single`: the step brings one token a request. proj_bias (here and below): float32 over all of the
+// product's columns, or null.
+int pyre_ssm_conv(const void* proj, int proj_dt, int n_partials, long partial_stride, int ld, int col0, const float* proj_bias,
+                  const float* taps_w,                  int taps, const float* conv_b, float* conv_state, const int* state_slots, const int* seq_of_token,
                   const int* q_start, int n_seqs, int single, void* x, int x_dt, int n, int inner, hipStream_t stream);
 // out[n] = the product's first `rank` columns as operands of the next product: float32 [n, padded], or bfloat16
 // [n, 2 padded], rounded to bfloat16 and what the rounding left; zeros from `rank` to `padded`.
@@ -399,14 +400,14 @@ int pyre_ssm_low(const void* sel, int sel_dt, int n_partials, long partial_strid
 // A2 [inner][state] = A log2(e); S float32 [slots][inner][state].
 int pyre_ssm_scan(const void* z, int z_dt, int z_partials, long z_stride, const float* dt_b, const void* x, int x_dt,
                   const void* sel, int sel_dt, int sel_partials, long sel_stride, int sel_ld, int b0, const void* proj,
-                  int proj_dt, int proj_partials, long proj_stride, int proj_ld, int g0, const float* A2, const float* D,
-                  float* state, const int* q_start, const int* state_slots, int n_seqs, float out_scale, void* out, int out_dt,
+                  int proj_dt, int proj_partials, long proj_stride, int proj_ld, const float* proj_bias, int g0, const float* A2,
+                  const float* D, float* state, const int* q_start, const int* state_slots, int n_seqs, float out_scale, void* out, int out_dt,
                   long out_ld, int inner, int n_state, hipStream_t stream);
 // The same for steps of one token a request, the step size's product included: z = dt_w [inner][rank, rows dt_ld apart] sel[0 .. rank).
 int pyre_ssm_step(const void* dt_w, int dt_w_dt, long dt_ld, const float* dt_b, const void* x, int x_dt, const void* sel,
                   int sel_dt, int sel_partials, long sel_stride, int sel_ld, int rank, const void* proj, int proj_dt,
-                  int proj_partials, long proj_stride, int proj_ld, int g0, const float* A2, const float* D, float* state,
-                  const int* state_slots, int n_seqs, float out_scale, void* out, int out_dt, long out_ld, int inner,
+                  int proj_partials, long proj_stride, int proj_ld, const float* proj_bias, int g0, const float* A2, const float* D,
+                  float* state, const int* state_slots, int n_seqs, float out_scale, void* out, int out_dt, long out_ld, int inner,
                   int n_state, hipStream_t stream);
 
 int pyre_route_grouped(const void* z, int z_dt, int n_partials, long partial_stride, const void* bias, int bias_dt,

@@ -47,12 +47,13 @@ struct Columns {
   int dt, n_partials;
   size_t stride;
   int ld, col0;
+  const float* bias = nullptr;  // over all of the product's columns, or null
 };
 __device__ inline float column(const Columns& p, size_t row, int col) {
   const size_t at = row * p.ld + p.col0 + col;
   float v = load_as_float(p.data, p.dt, at);
   for (int i = 1; i < p.n_partials; ++i) v += load_as_float(p.data, p.dt, i * p.stride + at);
-  return v;
+  return p.bias ? v + p.bias[p.col0 + col] : v;
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -270,7 +271,7 @@ int check_scan(const char* what, const ScanArgs& a, int n_seqs) {
 }  // namespace
 
 extern "C" int pyre_ssm_conv(const void* proj, int proj_dt, int n_partials, long partial_stride, int ld, int col0,
-                             const float* taps_w, int taps, const float* conv_b, float* conv_state, const int* state_slots,
+                             const float* proj_bias, const float* taps_w, int taps, const float* conv_b, float* conv_state, const int* state_slots,
                              const int* seq_of_token, const int* q_start, int n_seqs, int single, void* x, int x_dt, int n,
                              int inner, hipStream_t stream) {
   PYRE_REQUIRE(known_dtype(proj_dt) && known_dtype(x_dt) && n_partials >= 1, "ssm_conv: bad dtypes");
@@ -278,9 +279,10 @@ extern "C" int pyre_ssm_conv(const void* proj, int proj_dt, int n_partials, long
                "ssm_conv: %d taps (of at most %d) need their weights, the bias and, beyond one, the state", taps, kMaxTaps);
   PYRE_REQUIRE(state_slots && seq_of_token && q_start && n_seqs >= 0 && n_seqs <= 65535, "ssm_conv: the step's arrays are needed");
   if (n <= 0) return 0;
-  const ConvIn in{proj, proj_dt, n_partials, static_cast<size_t>(partial_stride), ld, col0, taps_w, taps, conv_state, inner};
+  const ConvIn in{proj, proj_dt, n_partials, static_cast<size_t>(partial_stride), ld, col0, taps_w, taps, conv_state, inner,
+                  proj_bias};
   if (taps <= kConvVecTaps && inner % 4 == 0 && ld % 4 == 0 && col0 % 4 == 0 && partial_stride % 4 == 0 && on16(proj) &&
-      on16(x) && on16(taps_w) && on16(conv_b) && on16(conv_state)) {
+      on16(x) && on16(taps_w) && on16(conv_b) && on16(conv_state) && on16(proj_bias)) {
     const dim3 grid(n, (inner / 4 + kThreads - 1) / kThreads);
     PYRE_DISPATCH(proj_dt, TP, PYRE_DISPATCH(x_dt, TX,
         hipLaunchKernelGGL((ssm_conv_vec_kernel<TP, TX>), grid, dim3(kThreads), 0, stream, in, conv_b, state_slots,
@@ -331,13 +333,14 @@ extern "C" int pyre_ssm_low(const void* sel, int sel_dt, int n_partials, long pa
 
 extern "C" int pyre_ssm_scan(const void* z, int z_dt, int z_partials, long z_stride, const float* dt_b, const void* x, int x_dt,
                              const void* sel, int sel_dt, int sel_partials, long sel_stride, int sel_ld, int b0,
-                             const void* proj, int proj_dt, int proj_partials, long proj_stride, int proj_ld, int g0,
+                             const void* proj, int proj_dt, int proj_partials, long proj_stride, int proj_ld, const float* proj_bias,
+                             int g0,
                              const float* A2, const float* D, float* state, const int* q_start, const int* state_slots,
                              int n_seqs, float out_scale, void* out, int out_dt, long out_ld, int inner, int n_state,
                              hipStream_t stream) {
   const ScanArgs a{{z, z_dt, z_partials, static_cast<size_t>(z_stride), inner, 0}, dt_b, x, x_dt,
                    {sel, sel_dt, sel_partials, static_cast<size_t>(sel_stride), sel_ld, b0},
-                   {proj, proj_dt, proj_partials, static_cast<size_t>(proj_stride), proj_ld, g0},
+                   {proj, proj_dt, proj_partials, static_cast<size_t>(proj_stride), proj_ld, g0, proj_bias},
                    A2, D, state, out, out_dt, static_cast<size_t>(out_ld), out_scale, inner, n_state};
   if (int rc = check_scan("ssm_scan", a, n_seqs)) return rc;
   PYRE_REQUIRE(z && known_dtype(z_dt) && z_partials >= 1 && q_start && state_slots, "ssm_scan: the step sizes' product and the step's arrays are needed");
@@ -351,12 +354,13 @@ extern "C" int pyre_ssm_scan(const void* z, int z_dt, int z_partials, long z_str
 
 extern "C" int pyre_ssm_step(const void* dt_w, int dt_w_dt, long dt_ld, const float* dt_b, const void* x, int x_dt,
                              const void* sel, int sel_dt, int sel_partials, long sel_stride, int sel_ld, int rank,
-                             const void* proj, int proj_dt, int proj_partials, long proj_stride, int proj_ld, int g0,
+                             const void* proj, int proj_dt, int proj_partials, long proj_stride, int proj_ld, const float* proj_bias,
+                             int g0,
                              const float* A2, const float* D, float* state, const int* state_slots, int n_seqs,
                              float out_scale, void* out, int out_dt, long out_ld, int inner, int n_state, hipStream_t stream) {
   const ScanArgs a{{nullptr, kF32, 1, 0, inner, 0}, dt_b, x, x_dt,
                    {sel, sel_dt, sel_partials, static_cast<size_t>(sel_stride), sel_ld, 0},
-                   {proj, proj_dt, proj_partials, static_cast<size_t>(proj_stride), proj_ld, g0},
+                   {proj, proj_dt, proj_partials, static_cast<size_t>(proj_stride), proj_ld, g0, proj_bias},
                    A2, D, state, out, out_dt, static_cast<size_t>(out_ld), out_scale, inner, n_state};
   if (int rc = check_scan("ssm_step", a, n_seqs)) return rc;
   PYRE_REQUIRE(dt_w && known_dtype(dt_w_dt) && rank > 0 && dt_ld >= rank && rank + 2 * n_state <= kMaxSelected && state_slots,

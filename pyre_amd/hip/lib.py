@@ -85,10 +85,10 @@ _SIGNATURES = {
                             I, I, I, I, P],
     "pyre_retention_prepare": [P, I, I, L, I, I, P, P, P, I, I, P, F, I, P, I, I, I, I, P],
     "pyre_gla_finish_wide": [P, P, P, I, F, F, P, I, L, I, I, I, I, P],
-    "pyre_ssm_conv": [P, I, I, L, I, I, P, I, P, P, P, P, P, I, I, P, I, I, I, P],
+    "pyre_ssm_conv": [P, I, I, L, I, I, P, P, I, P, P, P, P, P, I, I, P, I, I, I, P],
     "pyre_ssm_low": [P, I, I, L, I, P, I, I, I, I, P],
-    "pyre_ssm_scan": [P, I, I, L, P, P, I, P, I, I, L, I, I, P, I, I, L, I, I, P, P, P, P, P, I, F, P, I, L, I, I, P],
-    "pyre_ssm_step": [P, I, L, P, P, I, P, I, I, L, I, I, P, I, I, L, I, I, P, P, P, P, I, F, P, I, L, I, I, P],
+    "pyre_ssm_scan": [P, I, I, L, P, P, I, P, I, I, L, I, I, P, I, I, L, I, P, I, P, P, P, P, P, I, F, P, I, L, I, I, P],
+    "pyre_ssm_step": [P, I, L, P, P, I, P, I, I, L, I, I, P, I, I, L, I, P, I, P, P, P, P, I, F, P, I, L, I, I, P],
     "pyre_route_grouped": [P, I, I, L, P, I, P, P, I, I, I, I, I, P],
     "pyre_expert_glu_act": [P, I, I, L, P, L, P, I, I, I, I, I, I, P],
     "pyre_add_weighted_rows": [P, P, I, L, P, L, I, I, I, I, P],

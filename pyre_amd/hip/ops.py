@@ -1735,12 +1735,13 @@ SSM_MAX_STATE = 256      #: the largest state of a channel that the selective sc
 SSM_MAX_SELECTED = 12288  #: the most columns (rank of the step sizes and twice the state) of its second product
 
 
-def _ssm_columns(what: str, p: Partials, n: int, first: int, width: int):
-    if p.bias is not None:
-        raise KernelError(f"{what}: a product with a pending bias is not taken")
+def _ssm_columns(what: str, p: Partials, n: int, first: int, width: int, biased: bool = False):
+    bias = p.bias
+    if bias is not None and not (biased and bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() == p.width):
+        raise KernelError(f"{what}: a pending bias is taken with the input product alone, contiguous float32 [{p.width}]")
     if p.rows < n or first < 0 or first + width > p.width:
         raise KernelError(f"{what}: columns {first}..{first + width} of {n} rows lie outside the product's [{p.rows}, {p.width}]")
-    _dev(p.data)
+    _dev(p.data, bias)
     return (p.data.data_ptr(), dtype_code(p.data), p.count, p.stride)
 
 
@@ -1758,7 +1759,7 @@ def ssm_conv(proj: Partials, col0: int, taps_w: torch.Tensor, conv_b: torch.Tens
     + ``conv_b``). ``taps_w`` float32 [taps, inner]; inputs before the step come from ``conv_state`` (float32 [slots, taps - 1,
     inner]), which is brought up to date. ``single`` as for :func:`conv_qkv_write`."""
     taps, inner = taps_w.shape
-    args = _ssm_columns("ssm_conv", proj, n, col0, inner)
+    args = _ssm_columns("ssm_conv", proj, n, col0, inner, biased=True)
     _ssm_f32("ssm_conv", taps_w=(taps_w, (taps, inner)), conv_b=(conv_b, (inner,)))
     if not 1 <= taps <= CONV_MAX_TAPS:
         raise KernelError(f"ssm_conv: {taps} taps are outside 1..{CONV_MAX_TAPS}")
@@ -1772,7 +1773,7 @@ def ssm_conv(proj: Partials, col0: int, taps_w: torch.Tensor, conv_b: torch.Tens
         raise KernelError(f"ssm_conv: x is [>= {n}, {inner}]")
     if single and n != n_seqs:
         raise KernelError(f"ssm_conv: {n} tokens of {n_seqs} requests are not one token each")
-    call("pyre_ssm_conv", *args, proj.width, int(col0), taps_w.data_ptr(), taps, conv_b.data_ptr(),
+    call("pyre_ssm_conv", *args, proj.width, int(col0), _ptr(proj.bias), taps_w.data_ptr(), taps, conv_b.data_ptr(),
          conv_state.data_ptr() if taps > 1 else None, state_slots.data_ptr(), seq_of_token.data_ptr(), q_start.data_ptr(),
          n_seqs, int(bool(single)), x.data_ptr(), dtype_code(x), n, inner, _stream())
 
@@ -1795,7 +1796,7 @@ def _ssm_common(what, x, sel, rank, gate, g0, A2, D, dt_b, state, out, n, inner,
     _dev(x, out), _contig("x", x)
     if x.shape[-1] != inner or x.shape[0] < n or out.dim() != 2 or out.stride(1) != 1 or out.shape[1] < inner or out.shape[0] < n:
         raise KernelError(f"{what}: x is [>= {n}, {inner}], out [>= {n}, >= {inner}] with contiguous rows")
-    return (_ssm_columns(what, sel, n, 0, rank + 2 * n_state), _ssm_columns(what, gate, n, g0, inner))
+    return (_ssm_columns(what, sel, n, 0, rank + 2 * n_state), _ssm_columns(what, gate, n, g0, inner, biased=True))
 
 
 def ssm_scan(z: Partials, dt_b: torch.Tensor, x: torch.Tensor, sel: Partials, rank: int, gate: Partials, g0: int,
@@ -1810,8 +1811,8 @@ def ssm_scan(z: Partials, dt_b: torch.Tensor, x: torch.Tensor, sel: Partials, ra
     if z.width != inner:
         raise KernelError("ssm_scan: the step sizes' product is as wide as the channels")
     _i32("q_start", q_start, n_seqs + 1), _i32("state_slots", state_slots, n_seqs), _dev(q_start, state_slots)
-    call("pyre_ssm_scan", *zp, dt_b.data_ptr(), x.data_ptr(), dtype_code(x), *s, sel.width, int(rank), *g, gate.width, int(g0),
-         A2.data_ptr(), D.data_ptr(), state.data_ptr(), q_start.data_ptr(), state_slots.data_ptr(), n_seqs, float(out_scale),
+    call("pyre_ssm_scan", *zp, dt_b.data_ptr(), x.data_ptr(), dtype_code(x), *s, sel.width, int(rank), *g, gate.width,
+         _ptr(gate.bias), int(g0), A2.data_ptr(), D.data_ptr(), state.data_ptr(), q_start.data_ptr(), state_slots.data_ptr(), n_seqs, float(out_scale),
          out.data_ptr(), dtype_code(out), out.stride(0), inner, n_state, _stream())
 
 
@@ -1826,5 +1827,5 @@ def ssm_step(dt_w: torch.Tensor, dt_b: torch.Tensor, x: torch.Tensor, sel: Parti
     if dt_w.dim() != 2 or dt_w.shape[0] != inner or dt_w.shape[1] < rank or dt_w.stride(1) != 1:
         raise KernelError(f"ssm_step: the step sizes' matrix is [{inner}, >= {rank}] with contiguous rows")
     call("pyre_ssm_step", dt_w.data_ptr(), dtype_code(dt_w), dt_w.stride(0), dt_b.data_ptr(), x.data_ptr(), dtype_code(x), *s,
-         sel.width, int(rank), *g, gate.width, int(g0), A2.data_ptr(), D.data_ptr(), state.data_ptr(), state_slots.data_ptr(),
+         sel.width, int(rank), *g, gate.width, _ptr(gate.bias), int(g0), A2.data_ptr(), D.data_ptr(), state.data_ptr(), state_slots.data_ptr(),
          n_seqs, float(out_scale), out.data_ptr(), dtype_code(out), out.stride(0), inner, n_state, _stream())
