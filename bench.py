@@ -2,7 +2,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--context 4096] [--model qwen2.5-7b]
     python bench.py --workload serve [--model qwen2.5-1.5b] [--requests 256] [--max-batch 256]
-    python bench.py --workload designs [--shapes 1.5b,7b] [--layers 4] [--designs qwen2,mafurax,nurasun,durelix,zorulix,rukosun]
+    python bench.py --workload designs [--shapes 1.5b,7b] [--layers 4] [--designs qwen2,mafurax,nurasun,durelix,zorulix,rukosun,pinozen]
 
 A step is one decode step of the scheduler: every running request gets one new
 token (plan, one engine step over the paged cache, greedy sampling, token fed
@@ -43,7 +43,10 @@ and the Zorulix design, whose layers alternate between attention over a window o
 reading the keys and values of the one before) and windowed attention beside the gated delta rule at the same split of
 the heads, every layer with the mixture of 8 gated experts and a shared one and with 64 columns of a second token table,
 and the Rukosun design, whose layers alternate between its two kinds of latent attention (the same heads over rows of
-512 + 64 elements and a window of 1,024 tokens) with a dense feed-forward of the same width and two residual streams.
+512 + 64 elements and a window of 1,024 tokens) with a dense feed-forward of the same width and two residual streams,
+and the Pinozen design, three of whose four layers have causal attention (no window) at the Mafurax design's split of the
+heads beside a selective scan over as many channels as the width with a state of 16, the fourth lightning attention of all
+heads, a dense feed-forward of the same width, the last three layers a pass of a loop that runs once.
 For each:
 the prefill of a 2,048-token prompt, decode steps at 8 and 64 requests with contexts of 4,096, and
 the device time of every kernel of a prefill step and of a decode step at 8 requests.
@@ -304,7 +307,24 @@ def designs(args) -> dict:
                    "max_positions": 32768, "embedding": {"bigram": {"buckets": 65521, "mul_prev": 1000003, "mul_cur": 31}},
                    "layers": [{"type": "latent_attention" if i % 2 else "latent_attention_2", "mlp": {"kind": "dense", "ff": sh["ff"]},
                                "mixer": dict(rrow, q_rank=3 * sh["width"] // 8) if i % 2 else rrow} for i in range(layers)]}
-        made = {"qwen2": qwen, "mafurax": mafurax, "nurasun": nurasun, "durelix": durelix, "zorulix": zorulix, "rukosun": rukosun}
+        # Pinozen: three layers of four have causal attention over everything before (half of the heads, half of each
+        # turned with stretched frequencies, a convolution of four taps, capped scores) beside a selective scan (as many
+        # channels as the width, a state of 16, step sizes of a sixteenth of the width, four taps), the fourth lightning
+        # attention of all heads with decays from 0.9 to 0.9999; the layers behind the first are a pass of a loop that runs once
+        pleft = {"heads": sh["heads"] // 2, "kv_heads": max(1, sh["kv_heads"] // 2), "dim": sh["head"], "vdim": sh["head"],
+                 "scale": sh["head"] ** -0.5, "softcap": 50.0, "conv": 4,
+                 "rot": {"base": 2.5e5, "dims": sh["head"] // 2, "scaling": {"factor": 4.0, "low": 1.0, "high": 4.0, "original": 1024}}}
+        pright = {"inner": sh["width"], "state": 16, "dt_rank": sh["width"] // 16, "conv": 4}
+        plight = {"heads": sh["heads"], "dim": sh["head"], "vdim": sh["head"],
+                  "decay": [0.9 + 0.0999 * i / max(1, sh["heads"] - 1) for i in range(sh["heads"])]}
+        pinozen = {"architecture": "Pinozen", "vocab": sh["vocab"], "width": sh["width"], "norm": {"eps": 1e-6},
+                   "embedding": {"scale": 1.0}, "logit_scale": 1.0, "max_positions": 32768,
+                   "layers": [{"type": "lightning", "mixer": plight, "mlp": dense} if i % 4 == 2 else
+                              {"type": "parallel", "mixer": {"left": pleft, "right": pright}, "mlp": dense} for i in range(layers)]}
+        if layers > 1:
+            pinozen["loop"] = {"start": 1, "stop": layers, "times": 1}
+        made = {"qwen2": qwen, "mafurax": mafurax, "nurasun": nurasun, "durelix": durelix, "zorulix": zorulix, "rukosun": rukosun,
+                "pinozen": pinozen}
         return {name: config_from_dict(made[name]) for name in args.designs.split(",") if name}
 
     def kernels_of(run, per: int) -> dict:
@@ -453,8 +473,8 @@ def main() -> int:
     ap.add_argument("--model", default=None, help="preset shape (qwen2.5-7b; for --workload serve qwen2.5-1.5b)")
     ap.add_argument("--workload", default="decode", choices=["decode", "serve", "designs"])
     ap.add_argument("--shapes", default="1.5b,7b", help="designs: the layer sizes to compare at (1.5b, 7b)")
-    ap.add_argument("--designs", default="qwen2,mafurax,nurasun,durelix,zorulix,rukosun",
-                    help="designs: which of qwen2, mafurax, nurasun, durelix, zorulix, rukosun to measure")
+    ap.add_argument("--designs", default="qwen2,mafurax,nurasun,durelix,zorulix,rukosun,pinozen",
+                    help="designs: which of qwen2, mafurax, nurasun, durelix, zorulix, rukosun, pinozen to measure")
     ap.add_argument("--requests", type=int, default=256, help="serve: number of requests")
     ap.add_argument("--max-batch", type=int, default=256, help="serve: requests that run at a time")
     ap.add_argument("--seed", type=int, default=0, help="serve: seed of the lengths and token ids")

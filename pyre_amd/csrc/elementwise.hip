@@ -4,6 +4,7 @@
 #include "pyre_api.h"
 #include "pyre_common.h"
 #include "pyre_vec.h"
+#include "pyre_vec4.h"
 
 using namespace pyre;
 
@@ -26,12 +27,56 @@ __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict_
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) o[i] = to_float(row[i]) * scale;
 }
 
+// The same with four elements to a load, a row's all asked for at once (rows of at most 4 x 256 x ITEMS elements, whose
+// number is a multiple of four): at few tokens the kernel is one trip to memory and not one per 256 elements.
+template <typename T, int ITEMS>
+__global__ __launch_bounds__(256) void embed_vec_kernel(const T* __restrict__ table, const int* __restrict__ ids,
+                                                        const int* __restrict__ positions, const T* __restrict__ places,
+                                                        int n_places, float* __restrict__ out, int hidden, float scale) {
+  const int n = blockIdx.x;
+  const T* row = table + static_cast<size_t>(ids[n]) * hidden;
+  const T* place = places ? places + static_cast<size_t>(min(positions[n], n_places - 1)) * hidden : nullptr;
+  float* o = out + static_cast<size_t>(n) * hidden;
+  float4 v[ITEMS], p[ITEMS];
+#pragma unroll
+  for (int k = 0; k < ITEMS; ++k) {
+    const int i = 4 * (threadIdx.x + k * 256);
+    if (i >= hidden) continue;
+    v[k] = Vec4<T>::load(row + i);
+    if (place) p[k] = Vec4<T>::load(place + i);
+  }
+#pragma unroll
+  for (int k = 0; k < ITEMS; ++k) {
+    const int i = 4 * (threadIdx.x + k * 256);
+    if (i >= hidden) continue;
+    if (place) {
+      Vec4<float>::store(o + i, float4{fmaf(v[k].x, scale, p[k].x), fmaf(v[k].y, scale, p[k].y), fmaf(v[k].z, scale, p[k].z),
+                                       fmaf(v[k].w, scale, p[k].w)});
+    } else {
+      Vec4<float>::store(o + i, float4{v[k].x * scale, v[k].y * scale, v[k].z * scale, v[k].w * scale});
+    }
+  }
+}
+
 extern "C" int pyre_embed(const void* table, int table_dt, const int* ids, const int* positions, const void* places,
                           int n_places, float* out, int n, int hidden, float scale, hipStream_t stream) {
   PYRE_REQUIRE(!places || (positions && n_places > 0), "embed: a table of positions needs rows and the tokens' positions");
   PYRE_REQUIRE(known_dtype(table_dt), "embed: unknown table dtype %d", table_dt);
   PYRE_REQUIRE(n >= 0 && hidden > 0, "embed: bad sizes n=%d hidden=%d", n, hidden);
   if (n == 0) return 0;
+  const auto a16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  if (hidden % 4 == 0 && hidden <= 4 * 256 * 8 && a16(table) && a16(places) && a16(out)) {
+#define PYRE_EMBED(ITEMS)                                                                                                   \
+  hipLaunchKernelGGL((embed_vec_kernel<T, ITEMS>), dim3(n), dim3(256), 0, stream, static_cast<const T*>(table), ids, positions, \
+                     static_cast<const T*>(places), n_places, out, hidden, scale)
+    PYRE_DISPATCH(table_dt, T, {
+      if (hidden <= 1024) PYRE_EMBED(1);
+      else if (hidden <= 4096) PYRE_EMBED(4);
+      else PYRE_EMBED(8);
+    });
+#undef PYRE_EMBED
+    return check_launch("embed");
+  }
   PYRE_DISPATCH(table_dt, T,
                 hipLaunchKernelGGL(embed_kernel<T>, dim3(n), dim3(256), 0, stream,
                                    static_cast<const T*>(table), ids, positions, static_cast<const T*>(places), n_places,

@@ -11,17 +11,19 @@
 // ssm_low    the columns `low` as operands of the product that makes the step sizes: float32 as they are, or in 16-bit mode
 //            as two bfloat16 numbers side by side, the rounded one and what the rounding left: against [W_dt | W_dt]
 //            the product is then that of the unrounded numbers to 2^-17, since step sizes are 32-bit numbers.
-// ssm_scan   the recurrence over each request's tokens of the step in their order. A block: one request, 32 channels, eight
-//            neighbouring lanes to a channel, lane l keeping the state's elements l NS .. l NS + NS - 1 in registers. The
-//            tokens' numbers come 32 tokens at a time: while a tile is walked, the next one's are on their way into
-//            registers; a tile's step sizes are made once (not by every lane) on the way into LDS, and what leaves it (D x,
-//            the gate) is finished for the whole tile. The chain from token to token is one multiply-add: the exponentials do
-//            not depend on it. A token's sum over the state is joined by exchanges inside the vector unit.
+// ssm_scan   the recurrence over each request's tokens of the step in their order. A block: one request, 32 or 16 channels,
+//            eight or sixteen neighbouring lanes to a channel, lane l keeping the state's elements l NS .. l NS + NS - 1 in
+//            registers. The tokens' numbers come 32 tokens at a time through LDS, brought and finished by waves of their
+//            own; a tile's step sizes are made once (not by every lane) on the way there. The chain from token to token is
+//            one multiply-add: the exponentials do not depend on it, and eight tokens are one piece of code without a
+//            branch, so that they overlap. A token's sum over the state is joined by exchanges inside the vector unit.
 // ssm_step   the same for steps of one token a request, with the step size's product inside: the eight lanes of a channel
 //            share its row of W_dt, the second product's columns lie in LDS.
 //
 // A token's numbers are added in an order that its own sizes fix, and the state is walked token by token whatever the step
 // holds, so a result does not depend on where a step begins. All arithmetic float32; exponentials of dt A as powers of two.
+#include <type_traits>
+
 #include "pyre_api.h"
 #include "pyre_common.h"
 #include "pyre_conv.h"
@@ -38,8 +40,18 @@ constexpr int kTile = 32;                    // tokens of a tile
 constexpr int kMaxState = 256;
 constexpr int kMaxSelected = 12288;          // floats of LDS for the second product's columns of a token
 
-__device__ inline float silu_of(float z) { return z / (1.f + expf(-z)); }
-__device__ inline float softplus_of(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+__device__ inline float silu_of(float z) { return z * __builtin_amdgcn_rcpf(1.f + expf(-z)); }
+
+// log(1 + e^z) = max(z, 0) + log(1 + u), u = e^-|z| in (0, 1]; log(1 + u) = 2 atanh(s) with s = u / (2 + u) <= 1/3, whose
+// power series 2 s (1 + s^2 / 3 + s^4 / 5 + ..) is cut behind s^16 (the rest is below 2^-29 of it): accurate to a few units in
+// the last place however small u is, and without a branch.
+__device__ inline float softplus_of(float z) {
+  const float u = expf(-fabsf(z)), s = u * __builtin_amdgcn_rcpf(2.f + u), q = s * s;
+  float p = 1.f / 17.f;
+  p = fmaf(p, q, 1.f / 15.f), p = fmaf(p, q, 1.f / 13.f), p = fmaf(p, q, 1.f / 11.f), p = fmaf(p, q, 1.f / 9.f);
+  p = fmaf(p, q, 1.f / 7.f), p = fmaf(p, q, 1.f / 5.f), p = fmaf(p, q, 1.f / 3.f), p = fmaf(p, q, 1.f);
+  return fmaf(2.f * s, p, fmaxf(z, 0.f));
+}
 
 // A product as its partial sums; `col` counts from the first column of the part that is meant.
 struct Columns {
@@ -49,10 +61,26 @@ struct Columns {
   int ld, col0;
   const float* bias = nullptr;  // over all of the product's columns, or null
 };
+// The partial sums are added in their order, six of them asked for together.
 __device__ inline float column(const Columns& p, size_t row, int col) {
+  constexpr int kTogether = 6;
   const size_t at = row * p.ld + p.col0 + col;
-  float v = load_as_float(p.data, p.dt, at);
-  for (int i = 1; i < p.n_partials; ++i) v += load_as_float(p.data, p.dt, i * p.stride + at);
+  float v = 0.f;
+  if (p.dt == kF32) {
+    const float* src = static_cast<const float*>(p.data) + at;
+#pragma unroll 1
+    for (int i = 0; i < p.n_partials; i += kTogether) {
+      float part[kTogether];
+#pragma unroll
+      for (int u = 0; u < kTogether; ++u) part[u] = i + u < p.n_partials ? src[(i + u) * p.stride] : 0.f;
+#pragma unroll
+      for (int u = 0; u < kTogether; ++u)
+        if (i + u < p.n_partials) v += part[u];
+    }
+  } else {
+#pragma unroll 1
+    for (int i = 0; i < p.n_partials; ++i) v += to_float(static_cast<const bf16*>(p.data)[i * p.stride + at]);
+  }
   return p.bias ? v + p.bias[p.col0 + col] : v;
 }
 
@@ -116,20 +144,118 @@ struct ScanArgs {
   int inner, n_state;
 };
 
-template <int NS>
-__global__ __launch_bounds__(kThreads) void ssm_scan_kernel(ScanArgs a, const int* __restrict__ q_start,
-                                                            const int* __restrict__ state_slots) {
-  constexpr int kMine = kTile * kChannels / kThreads;    // (token, channel) pairs of a thread: tokens t, t + 8, ..
-  constexpr int kRow = 2 * NS * kLanes;                  // a token's B and C: [lane][B of NS elements | C of NS elements]
-  __shared__ __attribute__((aligned(16))) float2 steps[kTile][kChannels];  // dt, dt x
-  __shared__ __attribute__((aligned(16))) float bc[kTile][kRow];
-  __shared__ float ys[kTile][kChannels + 1];
-  const int s = blockIdx.y, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
-  const int part = lane % kLanes, mine = wave * (kWave / kLanes) + lane / kLanes;  // the walk: this lane's part of channel `mine`
-  const int c0 = blockIdx.x * kChannels, ch = c0 + mine;
-  const int t_begin = q_start[s], t_end = q_start[s + 1];
+// The sum over a group of L neighbouring lanes, in every lane of it (eight or sixteen).
+template <int L>
+__device__ inline float group_sum(float v) {
+  v = lanes_sum<8>(v);
+  if constexpr (L == 16) v += lane_exchange<0x140>(v);  // row_mirror: the other eight of a row of sixteen
+  return v;
+}
+
+__device__ inline void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+// A block: four waves that walk and four that do everything else, a tile ahead of them and a tile behind (they share the
+// compute unit's four schedulers in pairs). In the round of tile i the walking waves turn its numbers in LDS into its sums;
+// the others finish tile i - 1 (its sums, D x, the gate), put tile i + 1 into LDS (its step sizes made on the way) and send
+// for tile i + 2. The two meet at one barrier a round, which waits for LDS alone.
+// PLAIN: the usual case of many tokens, every product one float32 array without a bias, x and out bfloat16: the loads of a
+// tile are then nothing but loads (addresses held inside the arrays, what is not there replaced by zero when it is used),
+// so that all of them are on their way together.
+template <int L, int NS, bool PLAIN>
+__global__ __launch_bounds__(2 * kThreads) void ssm_scan_kernel(ScanArgs a, const int* __restrict__ q_start,
+                                                                const int* __restrict__ state_slots) {
+  constexpr int kCh = kThreads / L;                      // channels of a block
+  constexpr int kStep = kThreads / kCh;                  // tokens that the helping waves cover at once
+  constexpr int kMine = kTile / kStep;                   // (token, channel) pairs of a helping thread: tokens t, t + kStep, ..
+  constexpr int kPad = NS * L;                           // elements of the state, padded
+  constexpr int kBc = kTile * 2 * kPad / kThreads;       // numbers of B and C that a helping thread brings per tile
+  constexpr int kHalf = (NS + 1) / 2;
+  constexpr int kUnroll = NS <= 4 ? 8 : NS <= 8 ? 4 : 2;
+  static_assert(kTile % 8 == 0 && kTile % kStep == 0 && kTile * 2 * kPad % kThreads == 0, "a tile is dealt evenly");
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  float2(*steps)[kTile][kCh] = reinterpret_cast<float2(*)[kTile][kCh]>(lds);            // [2]: dt, dt x
+  float(*bc)[kTile][2 * kPad] = reinterpret_cast<float(*)[kTile][2 * kPad]>(lds + 2 * 2 * kTile * kCh);  // [2], [lane][B | C]
+  float(*ys)[kTile][kCh + 1] = reinterpret_cast<float(*)[kTile][kCh + 1]>(lds + 2 * 2 * kTile * kCh + 2 * kTile * 2 * kPad);  // [2]
+  const int s = blockIdx.y, c0 = blockIdx.x * kCh, tid = threadIdx.x % kThreads;
+  const int t_begin = q_start[s], t_end = q_start[s + 1], N = a.n_state;
   if (t_begin >= t_end) return;
-  const int N = a.n_state;
+  const int n_tiles = (t_end - t_begin + kTile - 1) / kTile;
+
+  if (threadIdx.x >= kThreads) {  // the helping waves: thread -> channel fc, tokens ft, ft + kStep, ..
+    const int fc = tid % kCh, ft = tid / kCh, fch = c0 + fc, fch_in = min(fch, a.inner - 1);
+    const bool fin = fch < a.inner;
+    const float dt_b = fin ? a.dt_b[fch] : 0.f, skip = fin ? a.D[fch] : 0.f;
+    float z[kMine], g[kMine], b[kBc];                     // of the tile that is on its way
+    typename std::conditional<PLAIN, bf16, float>::type x[kMine];
+    float x1[kMine], g1[kMine], x0[kMine], g0[kMine];     // of the tile in LDS next, of the tile that is walked
+    auto ask = [&](int tile) {
+      const int t0 = t_begin + tile * kTile;
+#pragma unroll
+      for (int k = 0; k < kMine; ++k) {
+        const size_t t = min(t0 + ft + k * kStep, t_end - 1);
+        if constexpr (PLAIN) {
+          z[k] = static_cast<const float*>(a.z.data)[t * a.z.ld + a.z.col0 + fch_in];
+          x[k] = static_cast<const bf16*>(a.x)[t * a.inner + fch_in];
+          g[k] = static_cast<const float*>(a.gate.data)[t * a.gate.ld + a.gate.col0 + fch_in];
+        } else {
+          z[k] = column(a.z, t, fch_in);
+          x[k] = load_as_float(a.x, a.x_dt, t * a.inner + fch_in);
+          g[k] = column(a.gate, t, fch_in);
+        }
+      }
+#pragma unroll
+      for (int k = 0; k < kBc; ++k) {
+        const int i = tid + k * kThreads, col = i % (2 * kPad), n = min(col % kPad, N - 1);  // B of all elements, then C
+        const size_t t = min(t0 + i / (2 * kPad), t_end - 1);
+        if constexpr (PLAIN) b[k] = static_cast<const float*>(a.sel.data)[t * a.sel.ld + a.sel.col0 + (col < kPad ? n : N + n)];
+        else b[k] = column(a.sel, t, col < kPad ? n : N + n);
+      }
+    };
+    auto put = [&](int tile) {  // the tile that was on its way goes to LDS
+      const int buf = tile & 1, left = t_end - t_begin - tile * kTile;
+#pragma unroll
+      for (int k = 0; k < kMine; ++k) {
+        const int t = ft + k * kStep;
+        x1[k] = to_float(x[k]), g1[k] = g[k];
+        const float dt = t < left ? softplus_of(z[k] + dt_b) : 0.f;  // behind the last token: S times one, plus zero
+        steps[buf][t][fc] = float2{dt, dt * x1[k]};
+      }
+#pragma unroll
+      for (int k = 0; k < kBc; ++k) {
+        const int i = tid + k * kThreads, t = i / (2 * kPad), col = i % (2 * kPad), n = col % kPad;
+        bc[buf][t][(n / NS) * 2 * NS + n % NS + (col < kPad ? 0 : NS)] = n < N ? b[k] : 0.f;
+      }
+    };
+    auto finish = [&](int tile, const float (&xs)[kMine], const float (&gs)[kMine]) {
+      const int t0 = t_begin + tile * kTile;
+#pragma unroll
+      for (int k = 0; k < kMine; ++k) {
+        const int t = ft + k * kStep;
+        const float y = fmaf(skip, xs[k], ys[tile & 1][t][fc]) * silu_of(gs[k]) * a.out_scale;
+        const size_t at = static_cast<size_t>(t0 + t) * a.out_ld + fch;
+        if (fin && t0 + t < t_end) {
+          if constexpr (PLAIN) static_cast<bf16*>(a.out)[at] = from_float<bf16>(y);
+          else store_from_float(a.out, a.out_dt, at, y);
+        }
+      }
+    };
+    ask(0);
+    put(0);
+    if (n_tiles > 1) ask(1);
+    lds_barrier();
+    for (int i = 0; i < n_tiles; ++i) {
+      if (i > 0) finish(i - 1, x0, g0);
+#pragma unroll
+      for (int k = 0; k < kMine; ++k) x0[k] = x1[k], g0[k] = g1[k];
+      if (i + 1 < n_tiles) put(i + 1);
+      if (i + 2 < n_tiles) ask(i + 2);
+      lds_barrier();
+    }
+    finish(n_tiles - 1, x0, g0);
+    return;
+  }
+
+  const int lane = tid & 63, part = lane % L, mine = (tid >> 6) * (kWave / L) + lane / L, ch = c0 + mine;
   float* st = a.state + (static_cast<size_t>(state_slots[s]) * a.inner + ch) * N;
   float S[NS], A2[NS];
 #pragma unroll
@@ -139,71 +265,50 @@ __global__ __launch_bounds__(kThreads) void ssm_scan_kernel(ScanArgs a, const in
     S[j] = there ? st[n] : 0.f;
     A2[j] = there ? a.A2[static_cast<size_t>(ch) * N + n] : 0.f;
   }
-  // the finishing of tiles: thread -> channel fc, tokens ft, ft + 8, ..
-  const int fc = tid % kChannels, ft = tid / kChannels, fch = c0 + fc;
-  const bool fin = fch < a.inner;
-  const float dt_b = fin ? a.dt_b[fch] : 0.f, skip = fin ? a.D[fch] : 0.f;
-  float z_next[kMine], x_next[kMine], g_next[kMine], bc_next[2 * NS];
-  auto ask = [&](int t0) {
+  lds_barrier();
+  for (int i = 0; i < n_tiles; ++i) {
+    const int buf = i & 1, nt = min(kTile, t_end - t_begin - i * kTile);
+    for (int t8 = 0; t8 < nt; t8 += 8) {
+      float keep = 0.f;  // lane part of a channel keeps the sum of token t8 + part: no branch between the tokens
+#pragma unroll kUnroll
+      for (int u = 0; u < 8; ++u) {
+        const float2 step = steps[buf][t8 + u][mine];
+        const float* row = &bc[buf][t8 + u][part * 2 * NS];
+        float y0 = 0.f, y1 = 0.f;  // two halves of the lane's elements: with twice the lanes each is a lane's own
 #pragma unroll
-    for (int k = 0; k < kMine; ++k) {
-      const int t = t0 + ft + k * (kThreads / kChannels);
-      const bool there = fin && t < t_end;
-      z_next[k] = there ? column(a.z, t, fch) : 0.f;
-      x_next[k] = there ? load_as_float(a.x, a.x_dt, static_cast<size_t>(t) * a.inner + fch) : 0.f;
-      g_next[k] = there ? column(a.gate, t, fch) : 0.f;
-    }
-#pragma unroll
-    for (int k = 0; k < 2 * NS; ++k) {  // kTile * kRow / kThreads = 2 NS numbers a thread
-      const int i = tid + k * kThreads, t = t0 + i / kRow, col = i % kRow;  // col: B of all elements, then C
-      const int n = col % (NS * kLanes);
-      bc_next[k] = t < t_end && n < N ? column(a.sel, t, col < NS * kLanes ? n : N + n) : 0.f;
-    }
-  };
-  ask(t_begin);
-  for (int t0 = t_begin; t0 < t_end; t0 += kTile) {
-    const int nt = min(kTile, t_end - t0);
-    float x_now[kMine], g_now[kMine];
-#pragma unroll
-    for (int k = 0; k < kMine; ++k) {
-      x_now[k] = x_next[k], g_now[k] = g_next[k];
-      const float dt = softplus_of(z_next[k] + dt_b);
-      steps[ft + k * (kThreads / kChannels)][fc] = float2{dt, dt * x_now[k]};
-    }
-#pragma unroll
-    for (int k = 0; k < 2 * NS; ++k) {
-      const int i = tid + k * kThreads, t = i / kRow, col = i % kRow, n = col % (NS * kLanes);
-      bc[t][(n / NS) * 2 * NS + n % NS + (col < NS * kLanes ? 0 : NS)] = bc_next[k];
-    }
-    __syncthreads();
-    if (t0 + kTile < t_end) ask(t0 + kTile);
-#pragma unroll 4
-    for (int t = 0; t < nt; ++t) {
-      const float2 step = steps[t][mine];
-      const float* row = &bc[t][part * 2 * NS];
-      float y = 0.f;
-#pragma unroll
-      for (int j = 0; j < NS; ++j) {
-        S[j] = fmaf(__builtin_amdgcn_exp2f(step.x * A2[j]), S[j], step.y * row[j]);
-        y = fmaf(S[j], row[NS + j], y);
+        for (int j = 0; j < NS; ++j) {
+          S[j] = fmaf(__builtin_amdgcn_exp2f(step.x * A2[j]), S[j], step.y * row[j]);
+          if (j < kHalf || L == 16) y0 = fmaf(S[j], row[NS + j], y0);
+          else y1 = fmaf(S[j], row[NS + j], y1);
+        }
+        const float y = group_sum<L>(L == 16 || NS == 1 ? y0 : y0 + y1);
+        keep = (part & 7) == u ? y : keep;
       }
-      y = lanes_sum<kLanes>(y);
-      if (part == 0) ys[t][mine] = y;
+      if (L == 8 || part < 8) ys[buf][t8 + (part & 7)][mine] = keep;
     }
-    __syncthreads();
-#pragma unroll
-    for (int k = 0; k < kMine; ++k) {
-      const int t = ft + k * (kThreads / kChannels);
-      if (fin && t < nt)
-        store_from_float(a.out, a.out_dt, static_cast<size_t>(t0 + t) * a.out_ld + fch,
-                         fmaf(skip, x_now[k], ys[t][fc]) * silu_of(g_now[k]) * a.out_scale);
-    }
+    lds_barrier();
   }
 #pragma unroll
   for (int j = 0; j < NS; ++j) {
     const int n = part * NS + j;
     if (ch < a.inner && n < N) st[n] = S[j];
   }
+}
+template <int L, int NS, bool PLAIN>
+int launch_scan(const ScanArgs& a, const int* q_start, const int* state_slots, int n_seqs, hipStream_t stream) {
+  constexpr int kCh = kThreads / L;
+  constexpr size_t lds = sizeof(float) * 2 * kTile * (2 * kCh + 2 * NS * L + kCh + 1);
+  static_assert(lds <= 160 * 1024, "a compute unit has 160 KB of LDS");
+  static bool raised = lds <= 64 * 1024;
+  if (!raised) {
+    if (hipFuncSetAttribute(reinterpret_cast<const void*>(&ssm_scan_kernel<L, NS, PLAIN>),
+                            hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)) != hipSuccess)
+      return fail("ssm_scan: the device refuses %zu bytes of LDS", lds);
+    raised = true;
+  }
+  hipLaunchKernelGGL((ssm_scan_kernel<L, NS, PLAIN>), dim3((a.inner + kCh - 1) / kCh, n_seqs), dim3(2 * kThreads), lds, stream, a,
+                     q_start, state_slots);
+  return 0;
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -345,9 +450,26 @@ extern "C" int pyre_ssm_scan(const void* z, int z_dt, int z_partials, long z_str
   if (int rc = check_scan("ssm_scan", a, n_seqs)) return rc;
   PYRE_REQUIRE(z && known_dtype(z_dt) && z_partials >= 1 && q_start && state_slots, "ssm_scan: the step sizes' product and the step's arrays are needed");
   if (n_seqs <= 0) return 0;
-  const dim3 grid((inner + kChannels - 1) / kChannels, n_seqs);
-#define PYRE_SCAN(NS) hipLaunchKernelGGL(ssm_scan_kernel<NS>, grid, dim3(kThreads), 0, stream, a, q_start, state_slots)
-  PYRE_SSM_FORMS(n_state, PYRE_SCAN);
+  // eight lanes to a channel, or sixteen where blocks of the former would leave half of the compute units idle (a token
+  // of a wave is then shorter; the same sums in the same order)
+  const int blocks8 = (inner + kThreads / 8 - 1) / (kThreads / 8);
+  const bool wide = static_cast<long>(blocks8) * n_seqs <= compute_units() / 2;
+  const bool plain = z_dt == kF32 && sel_dt == kF32 && proj_dt == kF32 && z_partials == 1 && sel_partials == 1 &&
+                     proj_partials == 1 && !proj_bias && x_dt == kBF16 && out_dt == kBF16;
+#define PYRE_SCAN(L, NS)                                                                                            \
+  do {                                                                                                              \
+    if (int rc = plain ? launch_scan<L, NS, true>(a, q_start, state_slots, n_seqs, stream)                          \
+                       : launch_scan<L, NS, false>(a, q_start, state_slots, n_seqs, stream))                        \
+      return rc;                                                                                                    \
+  } while (0)
+#define PYRE_SCAN8(NS) PYRE_SCAN(8, NS)
+  if (wide && n_state > 8 && n_state <= 16) PYRE_SCAN(16, 1);
+  else if (wide && n_state > 24 && n_state <= 32) PYRE_SCAN(16, 2);
+  else if (wide && n_state > 48 && n_state <= 64) PYRE_SCAN(16, 4);
+  else if (wide && n_state > 64 && n_state <= 128) PYRE_SCAN(16, 8);
+  else if (wide && n_state > 128) PYRE_SCAN(16, 16);
+  else PYRE_SSM_FORMS(n_state, PYRE_SCAN8);
+#undef PYRE_SCAN8
 #undef PYRE_SCAN
   return check_launch("ssm_scan");
 }

@@ -480,7 +480,8 @@ def close(got, want, tol):
 
 @pytest.mark.parametrize("inner,N,rank,parts", [(32, 16, 8, 1), (5, 1, 1, 2), (33, 5, 3, 1), (64, 8, 16, 3), (40, 9, 7, 1), (96, 17, 12, 2), (24, 24, 40, 1),
                                                 (70, 25, 4, 1), (32, 32, 224, 4), (31, 48, 9, 1), (32, 64, 10, 1), (16, 65, 33, 2), (20, 128, 8, 1),
-                                                (12, 129, 16, 1), (8, 256, 100, 1), (300, 16, 24, 1)])
+                                                (12, 129, 16, 1), (8, 256, 100, 1), (900, 16, 24, 1),
+                                                (831, 27, 6, 1), (850, 60, 8, 1)])
 def test_the_selective_scan_kernels(inner, N, rank, parts):
     """The scan over requests of 0 to 75 tokens, cut in two and whole the same bits, and the step of single tokens, from
     states in slots of no order, against float64."""
@@ -510,13 +511,16 @@ def test_the_selective_scan_kernels(inner, N, rank, parts):
     d = lambda t: t.contiguous().to(DEV)  # noqa: E731
     zs, ss, gs = z.double().sum(0), sel.double().sum(0), gate.double().sum(0)
 
-    def run(kernel_lens, first, st, out):
+    def run(kernel_lens, first, st, out, only=None):
+        if only is not None and not kernel_lens[only]:
+            return
         rows = [range(int(q_start[i]) + first[i], int(q_start[i]) + first[i] + kernel_lens[i]) for i in range(S)]
         pick = torch.tensor([r for rr in rows for r in rr], dtype=torch.long)
         qs = torch.tensor([0, *np.cumsum(kernel_lens)], dtype=torch.int32)
         o = torch.full((len(pick), inner + 3), 9.0, device=DEV)
         ops.ssm_scan(ops.Partials(d(z[:, pick])), d(dt_b), d(x[pick]), ops.Partials(d(sel[:, pick])), rank, ops.Partials(d(gate[:, pick])), g0,
-                     d(A2), d(D), st, d(qs), d(slots), S, 0.7, o, len(pick))
+                     d(A2), d(D), st, d(qs) if only is None else d(torch.tensor([0, kernel_lens[only]], dtype=torch.int32)),
+                     d(slots) if only is None else d(slots[only:only + 1]), S if only is None else 1, 0.7, o, len(pick))
         assert bool((o[:, inner:] == 9.0).all())
         out[pick] = o[:, :inner].cpu()
 
@@ -526,6 +530,11 @@ def test_the_selective_scan_kernels(inner, N, rank, parts):
     run(half, [0] * S, st2, cut_out)
     run([k - h for k, h in zip(lens, half)], half, st2, cut_out)
     assert torch.equal(whole_out, cut_out) and torch.equal(st, st2)
+    # a request alone (where few channels make few blocks, sixteen lanes to a channel instead of eight): the same bits
+    alone, st3 = torch.zeros(n, inner), d(state)
+    for i in range(S):
+        run([k if j == i else 0 for j, k in enumerate(lens)], [0] * S, st3, alone, only=i)
+    assert torch.equal(whole_out, alone) and torch.equal(st, st3)
     for i in range(S):
         a, b = int(q_start[i]), int(q_start[i + 1])
         want, S1 = plain(zs[a:b], x[a:b].double(), ss[a:b], gs[a:b], state[slots[i]].double())
@@ -684,10 +693,11 @@ def test_an_embedding_with_a_factor_and_places():
 
     g = torch.Generator().manual_seed(8)
     ids, pos = [3, 19, 0, 7], [0, 5, 8, 2]
-    for dtype in (torch.float32, torch.bfloat16):
-        table, places = torch.randn(20, 300, generator=g).to(dtype), torch.randn(9, 300, generator=g).to(dtype)
+    for dtype, width in ((torch.float32, 300), (torch.bfloat16, 300), (torch.bfloat16, 37), (torch.float32, 3584), (torch.bfloat16, 5124),
+                         (torch.bfloat16, 9000)):
+        table, places = torch.randn(20, width, generator=g).to(dtype), torch.randn(9, width, generator=g).to(dtype)
         i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=DEV)  # noqa: E731
-        out = torch.zeros(4, 300, device=DEV)
+        out = torch.zeros(4, width, device=DEV)
         ops.embed(table.to(DEV), i32(ids), out, 0.3, i32(pos), places.to(DEV))
         assert close(out, table[ids].double() * 0.3 + places[pos].double(), 1e-6)
         ops.embed(table.to(DEV), i32(ids), out, 0.3)
