@@ -404,7 +404,7 @@ __global__ __launch_bounds__(kThreads) void attn_biased_tile_kernel(
 // p = p1 + p2 + p3 (p1 = bf16(p), p2 = bf16(p - p1), p3 = p - p1 - p2, which has eight bits left: exact), each
 // multiplied with the values and added in float32: scores and weights stay 32-bit. 32 such instructions a chunk and
 // head of 128 where the float32 form has 128, keys, queries and values as bfloat16 in LDS (a third of the space, so
-// that three blocks share a compute unit). Head sizes are multiples of eight; the caches start on 16 bytes.
+// that three blocks share a compute unit). Head sizes are multiples of eight, the pages' size is a power of two; the caches start on 16 bytes.
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 constexpr int kPad16 = 8;            // bfloat16 elements of padding behind a row of keys, queries or transposed values
 
@@ -412,14 +412,47 @@ constexpr int kPad16 = 8;            // bfloat16 elements of padding behind a ro
 // instruction (kk = 16 a + 4 h + u and 16 a + 8 + 4 h + u, u < 4) side by side, one 16-byte read.
 __device__ inline int vt_slot(int kk) { return (kk & 16) + 8 * ((kk >> 2) & 1) + 4 * ((kk >> 3) & 1) + (kk & 3); }
 
-template <int NV>
-__global__ __launch_bounds__(kThreads) void attn_biased_tile16_kernel(
+//
+// Scores are kept times log2(e), so that every exponential is the hardware's power of two; the cap's tanh is formed of one as
+// well (absolute errors of a few 1e-7 of the cap, float32 rounding beside values that come from bfloat16 keys).
+//
+// With `part` a tile's chunks are dealt to `gridDim.z` blocks, `per` chunks each (the last takes what is left): a tile of no more than `per` chunks is
+// finished by its first block; of a longer one every block leaves its sums, maximum (of scores times log2(e)) and sum of
+// weights at part [token][head][block][dv + 4], and attn_tile_join_kernel adds them up.
+struct TileChunks {
+  int n_first, chunk_b, n_chunks;
+};
+// The chunks of a tile: those that hold the kept first tokens which the window has passed, then the window's.
+__device__ inline TileChunks tile_chunks(int pos0, int ntok, int window, int keep_first, int chunk) {
+  const int lo_all = first_seen(pos0, window, chunk);  // rises with the position: the tile's first token sees furthest back
+  const int kept_end = min(window > 0 ? keep_first : 0, lo_all);  // keys 0 .. kept_end - 1 lie before every window
+  TileChunks r;
+  r.n_first = kept_end > 0 ? (kept_end - 1) / kKeys + 1 : 0;
+  r.chunk_b = max(lo_all / kKeys, r.n_first);
+  r.n_chunks = r.n_first + ((pos0 + ntok - 1) / kKeys - r.chunk_b + 1);
+  return r;
+}
+constexpr float kLog2e = 1.44269504088896340736f;
+// The same for a maximum and a sink in powers of two.
+__device__ inline float softmax_factor2(float m, float l, const float* sink, int head) {
+  if (!sink) return l > 0.f ? 1.f / l : 0.f;
+  const float sk = sink[head] * kLog2e, M = fmaxf(m, sk);
+  const float a = m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m - M);
+  return a / (l * a + __builtin_amdgcn_exp2f(sk - M));
+}
+
+// Where a pair of neighbouring keys (2 p, 2 p + 1) lies in a row of transposed values, in 32-bit words.
+__device__ inline int vt_pair(int p) { return vt_slot(2 * p) / 2; }
+
+// TAB: the request's block table lies in LDS.
+template <int NV, bool TAB>
+__global__ __launch_bounds__(kThreads, NV <= 4 ? 2 : 1) void attn_biased_tile16_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ k_cache, const bf16* __restrict__ v_cache, bf16* __restrict__ out,
     int out_ld, const float* __restrict__ gate, float out_scale, const int* __restrict__ tiles,
     const int* __restrict__ positions, const int* __restrict__ seq_of_token, const int* __restrict__ block_table,
-    int table_stride, int nq, int nkv, int dk, int dkp, int dv, int page_size, float scale, float cap,
+    int table_stride, int nq, int nkv, int dk, int dkp, int dv, int page_shift, float scale, float cap,
     const float* __restrict__ bias, int far, int window, int keep_first, int chunk, int tab_lds, int bias_lds,
-    const float* __restrict__ sink, int gate_dim) {
+    const float* __restrict__ sink, int gate_dim, float* __restrict__ part, int per) {
   extern __shared__ __attribute__((aligned(16))) unsigned char lds_raw[];
   const int ldk = dkp + kPad16, ldv = kKeys + kPad16;
   bf16* Ks = reinterpret_cast<bf16*>(lds_raw);                 // [kKeys][ldk]
@@ -427,7 +460,6 @@ __global__ __launch_bounds__(kThreads) void attn_biased_tile16_kernel(
   bf16* Vt = Qs + 4 * 32 * ldk;                                // [32 NV][ldv], keys in the order of vt_slot
   int* tab_s = reinterpret_cast<int*>(Vt + 32 * NV * ldv);     // [tab_lds]: the request's block table, if it fits
   float* bias_s = reinterpret_cast<float*>(tab_s + tab_lds);   // [4][far + 1]: the four heads' biases, if they fit
-  __shared__ int page_s[2][kKeys];
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = lane >> 5, c = lane & 31;
   const int n_rep = nq / nkv, hgroups = (n_rep + 3) / 4;
   const int kvh = blockIdx.y / hgroups, hin = (blockIdx.y % hgroups) * 4 + wave;
@@ -436,6 +468,9 @@ __global__ __launch_bounds__(kThreads) void attn_biased_tile16_kernel(
   const int t0 = tiles[2 * blockIdx.x], ntok = tiles[2 * blockIdx.x + 1];
   if (ntok <= 0) return;
   const int pos0 = positions[t0];
+  const TileChunks tc = tile_chunks(pos0, ntok, window, keep_first, chunk);
+  const int n_first = tc.n_first, chunk_b = tc.chunk_b, n_chunks = tc.n_chunks;
+  if (part && static_cast<int>(blockIdx.z) * per >= n_chunks) return;
   const int* table = block_table + static_cast<size_t>(seq_of_token[t0]) * table_stride;
 
   const bool live = active && c < ntok;
@@ -444,10 +479,8 @@ __global__ __launch_bounds__(kThreads) void attn_biased_tile16_kernel(
   const int keep = window > 0 ? keep_first : 0;
   const float* bias_row = bias ? bias + static_cast<size_t>(head) * (far + 1) : nullptr;
   for (int i = tid; i < tab_lds; i += kThreads) tab_s[i] = table[i];
-  if (bias && bias_lds) {
+  if (bias && bias_lds)
     for (int i = lane; i <= far; i += 64) bias_s[wave * (far + 1) + i] = bias_row[i];
-    bias_row = bias_s + wave * (far + 1);
-  }
   const uint4 zero4 = {0u, 0u, 0u, 0u};
   {  // this wave's queries: Qs[wave][token][d], zeros where there is no token or no element
     bf16* mine = Qs + wave * 32 * ldk;
@@ -466,69 +499,92 @@ __global__ __launch_bounds__(kThreads) void attn_biased_tile16_kernel(
     for (int i = 0; i < 16; ++i) o[dt][i] = 0.f;
   float m = -INFINITY, l = 0.f;
 
-  const int lo_all = first_seen(pos0, window, chunk);
   const int hi_all = pos0 + ntok - 1;
-  const int kept_end = min(keep, lo_all);
-  const int n_first = kept_end > 0 ? (kept_end - 1) / kKeys + 1 : 0;
-  const int chunk_b = max(lo_all / kKeys, n_first);
-  const int n_chunks = n_first + (hi_all / kKeys - chunk_b + 1);
-  // the next chunk's keys and values are asked for (into registers) before the current chunk is multiplied, and go
-  // to LDS when every wave is done with it
-  constexpr int KI = kKeys * (kTileMaxKeyHead / 8) / kThreads, VI = (kKeys * 4 * NV + kThreads - 1) / kThreads;
-  uint4 kreg[KI], vreg[VI];
+  const int it_begin = part ? static_cast<int>(blockIdx.z) * per : 0,
+            it_end = part && blockIdx.z + 1 < gridDim.z ? min(it_begin + per, n_chunks) : n_chunks;
+  // The next chunk's keys and values are asked for (into registers) before the current chunk is multiplied, and go to LDS
+  // when every wave is done with it. A thread brings pieces of eight elements: of keys up to two, each of one key; of
+  // values NV / 4 times (at least once) the same piece of two neighbouring keys, whose elements go to LDS in pairs. Loads are
+  // nothing but loads: what is not there is read from somewhere inside the cache and replaced by zeros on its way to LDS.
+  constexpr int KI = kKeys * (kTileMaxKeyHead / 8) / kThreads, VP = (16 * 4 * NV + kThreads - 1) / kThreads;
+  const int kg = dkp / 8, page_size = 1 << page_shift;
+  int k_key[KI], k_at[KI], v_pair[VP], v_at[VP];
+  bool k_mine[KI], v_mine[VP];
+#pragma unroll
+  for (int k = 0; k < KI; ++k) {
+    const int i = tid + k * kThreads;
+    k_key[k] = i / kg, k_at[k] = 8 * (i % kg);
+    k_mine[k] = k_key[k] < kKeys && k_at[k] < dk;
+  }
+#pragma unroll
+  for (int k = 0; k < VP; ++k) {
+    const int i = tid + k * kThreads;
+    v_pair[k] = i & 15, v_at[k] = 8 * (i >> 4);
+    v_mine[k] = v_at[k] < dv;
+  }
+  uint4 kreg[KI], vreg[VP][2];
+  unsigned there = 0;  // which of them are: bit k for keys, bits 8 + 2 k and 9 + 2 k for values
   auto chunk_key0 = [&](int it) { return (it < n_first ? it : chunk_b + (it - n_first)) * kKeys; };
-  auto page_of = [&](int key) {
-    const int entry = key / page_size;
-    if (key > hi_all || entry >= table_stride) return -1;
-    return entry < tab_lds ? tab_s[entry] : table[entry];
+  auto row_of = [&](int key, bool mine, bool& is) {  // the key's row among the cache's rows of this head
+    const int entry = key >> page_shift;
+    int page;
+    const bool asked = mine & (key <= hi_all) & (entry < table_stride);
+    if constexpr (TAB) page = tab_s[asked ? entry : 0];
+    else page = table[asked ? entry : 0];
+    is = asked & (page >= 0);
+    return ((static_cast<size_t>(max(page, 0)) * nkv + kvh) << page_shift) + (key & (page_size - 1));
   };
   auto ask = [&](int it) {
-    const int key0 = chunk_key0(it), kg = dkp / 8;
-    if (tid < kKeys) page_s[it & 1][tid] = page_of(key0 + tid);
+    const int key0 = chunk_key0(it);
+    there = 0;
 #pragma unroll
     for (int k = 0; k < KI; ++k) {
-      const int i = tid + k * kThreads, key = key0 + i / kg, d = 8 * (i % kg);
-      const int page = i < kKeys * kg ? page_of(key) : -1;
-      kreg[k] = zero4;
-      if (page >= 0 && d < dk)
-        kreg[k] = *reinterpret_cast<const uint4*>(k_cache + ((static_cast<size_t>(page) * nkv + kvh) * page_size + key % page_size) * dk + d);
+      bool is;
+      const size_t row = row_of(key0 + k_key[k], k_mine[k], is);
+      kreg[k] = *reinterpret_cast<const uint4*>(k_cache + row * dk + (k_mine[k] ? k_at[k] : 0));
+      there |= is ? 1u << k : 0u;
     }
 #pragma unroll
-    for (int k = 0; k < VI; ++k) {
-      const int i = tid + k * kThreads, key = key0 + i / (4 * NV), d = 8 * (i % (4 * NV));
-      const int page = i < kKeys * 4 * NV ? page_of(key) : -1;
-      vreg[k] = zero4;
-      if (page >= 0 && d < dv)
-        vreg[k] = *reinterpret_cast<const uint4*>(v_cache + ((static_cast<size_t>(page) * nkv + kvh) * page_size + key % page_size) * dv + d);
-    }
+    for (int k = 0; k < VP; ++k)
+#pragma unroll
+      for (int e = 0; e < 2; ++e) {
+        bool is;
+        const size_t row = row_of(key0 + 2 * v_pair[k] + e, v_mine[k], is);
+        vreg[k][e] = *reinterpret_cast<const uint4*>(v_cache + row * dv + (v_mine[k] ? v_at[k] : 0));
+        there |= is ? 1u << (8 + 2 * k + e) : 0u;
+      }
+  };
+  auto kept = [&](uint4 v, int bit) {  // v, or zeros
+    const uint32_t w = there >> bit & 1u ? ~0u : 0u;
+    return uint4{v.x & w, v.y & w, v.z & w, v.w & w};
   };
   auto stash = [&]() {
-    const int kg = dkp / 8;
 #pragma unroll
-    for (int k = 0; k < KI; ++k) {
-      const int i = tid + k * kThreads, key = i / kg, d = 8 * (i % kg);
-      if (i < kKeys * kg) *reinterpret_cast<uint4*>(Ks + key * ldk + d) = kreg[k];
-    }
+    for (int k = 0; k < KI; ++k)
+      if (k_key[k] < kKeys) *reinterpret_cast<uint4*>(Ks + k_key[k] * ldk + k_at[k]) = kept(kreg[k], k);
 #pragma unroll
-    for (int k = 0; k < VI; ++k) {
-      const int i = tid + k * kThreads, key = i / (4 * NV), d = 8 * (i % (4 * NV));
-      if (i < kKeys * 4 * NV) {
-        const uint32_t w[4] = {vreg[k].x, vreg[k].y, vreg[k].z, vreg[k].w};
-        const int slot = vt_slot(key);
+    for (int k = 0; k < VP; ++k) {
+      if (v_at[k] >= 32 * NV) continue;
+      const uint4 a = kept(vreg[k][0], 8 + 2 * k), b = kept(vreg[k][1], 9 + 2 * k);
+      const uint32_t wa[4] = {a.x, a.y, a.z, a.w}, wb[4] = {b.x, b.y, b.z, b.w};
+      uint32_t* dst = reinterpret_cast<uint32_t*>(Vt + v_at[k] * ldv) + vt_pair(v_pair[k]);
 #pragma unroll
-        for (int u = 0; u < 8; ++u) Vt[(d + u) * ldv + slot].bits = static_cast<uint16_t>(u & 1 ? w[u >> 1] >> 16 : w[u >> 1] & 0xffffu);
+      for (int u = 0; u < 4; ++u) {  // element 2 u and 2 u + 1 of both keys
+        dst[2 * u * (ldv / 2)] = (wa[u] & 0xffffu) | (wb[u] << 16);
+        dst[(2 * u + 1) * (ldv / 2)] = (wa[u] >> 16) | (wb[u] & 0xffff0000u);
       }
     }
   };
   __syncthreads();  // the table and the biases are in LDS
-  ask(0);
-  for (int it = 0; it < n_chunks; ++it) {
+  ask(it_begin);
+  // cap tanh(s scale / cap) log2(e), or s scale log2(e): tanh(x) = sign(x) (1 - e) / (1 + e), e = exp(-2 |x|)
+  const float to2 = scale * kLog2e, cap2 = cap * kLog2e, bend = cap > 0.f ? -2.f * to2 / cap : 0.f;
+  for (int it = it_begin; it < it_end; ++it) {
     const int key0 = chunk_key0(it);
-    const int* pages = page_s[it & 1];
     __syncthreads();  // the previous chunk has been read by every wave (and the queries are written)
     stash();
     __syncthreads();
-    if (it + 1 < n_chunks) ask(it + 1);
+    if (it + 1 < it_end) ask(it + 1);
     if (!active) continue;
 
     f32x16 s;
@@ -543,41 +599,63 @@ __global__ __launch_bounds__(kThreads) void attn_biased_tile16_kernel(
     }
 
     // element i of s: key key0 + 8 (i / 4) + 4 h + i % 4, token c
-    float bv[16];
+    if (cap > 0.f) {
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const int key = key0 + 8 * (i >> 2) + 4 * h + (i & 3);
-      bv[i] = bias_row ? bias_row[min(max(hi - key, 0), far)] : 0.f;
-    }
-    float mx = -INFINITY;
+      for (int i = 0; i < 16; ++i) {
+        const float e = __builtin_amdgcn_exp2f(bend * fabsf(s[i]));
+        s[i] = copysignf((1.f - e) * __builtin_amdgcn_rcpf(1.f + e) * cap2, s[i]);
+      }
+    } else {
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const int kk = 8 * (i >> 2) + 4 * h + (i & 3), key = key0 + kk;
-      const bool seen = key <= hi && (key >= lo || key < keep) && pages[kk] >= 0;
-      const float shaped = shaped_score(s[i], scale, cap, nullptr, 0, 0) + bv[i];
-      s[i] = seen ? shaped : -INFINITY;
-      mx = fmaxf(mx, s[i]);
+      for (int i = 0; i < 16; ++i) s[i] *= to2;
     }
+    if (bias) {  // the biases of the lane's sixteen distances (a key that is not seen reads a distance that is there)
+      float bv[16];
+      if (bias_lds) {
+#pragma unroll
+        for (int i = 0; i < 16; ++i)
+          bv[i] = bias_s[wave * (far + 1) + min(max(hi - (key0 + 8 * (i >> 2) + 4 * h + (i & 3)), 0), far)];
+      } else {
+#pragma unroll
+        for (int i = 0; i < 16; ++i) bv[i] = bias_row[min(max(hi - (key0 + 8 * (i >> 2) + 4 * h + (i & 3)), 0), far)];
+      }
+#pragma unroll
+      for (int i = 0; i < 16; ++i) s[i] = fmaf(bv[i], kLog2e, s[i]);
+    }
+    const int first = key0 + 4 * h;  // the lane's first key
+    if (key0 < lo || key0 + kKeys - 1 > hi) {  // some key of the chunk is hidden from this lane's token
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int key = first + 8 * (i >> 2) + (i & 3);
+        const bool seen = (key <= hi) & ((key >= lo) | (key < keep));
+        s[i] = seen ? s[i] : -INFINITY;
+      }
+    }
+    float mx = s[0];
+#pragma unroll
+    for (int i = 1; i < 16; ++i) mx = fmaxf(mx, s[i]);
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
     const float m_new = fmaxf(m, mx);
     const float m_use = m_new == -INFINITY ? 0.f : m_new;
-    const float alpha = expf(m - m_use);
+    if (__any(m_new > m)) {  // no maximum of the wave's tokens rises in most chunks: nothing to scale down then
+      const float alpha = __builtin_amdgcn_exp2f(m - m_use);
+      l *= alpha;
+#pragma unroll
+      for (int dt = 0; dt < NV; ++dt)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) o[dt][i] *= alpha;
+    }
     m = m_new;
     float sum = 0.f;
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
-      s[i] = expf(s[i] - m_use);
+      s[i] = __builtin_amdgcn_exp2f(s[i] - m_use);
       sum += s[i];
     }
-    l = l * alpha + sum;
-#pragma unroll
-    for (int dt = 0; dt < NV; ++dt)
-#pragma unroll
-      for (int i = 0; i < 16; ++i) o[dt][i] *= alpha;
-    // the weights in three bfloat16 pieces each; piece[a]: the lane's eight keys of instruction a (s[8 a .. 8 a + 7])
-    uint4 piece[3][2];
+    l += sum;
 #pragma unroll
     for (int a = 0; a < 2; ++a) {
+      // the weights of the lane's eight keys of instruction a (s[8 a .. 8 a + 7]) in three bfloat16 pieces each
       uint32_t w1[4], w2[4], w3[4];
 #pragma unroll
       for (int u = 0; u < 4; ++u) {
@@ -587,25 +665,40 @@ __global__ __launch_bounds__(kThreads) void attn_biased_tile16_kernel(
         w2[u] = pack_bf16x2(r0, r1);
         w3[u] = pack_bf16x2(r0 - __uint_as_float(w2[u] << 16), r1 - __uint_as_float(w2[u] & 0xffff0000u));
       }
-      piece[0][a] = uint4{w1[0], w1[1], w1[2], w1[3]};
-      piece[1][a] = uint4{w2[0], w2[1], w2[2], w2[3]};
-      piece[2][a] = uint4{w3[0], w3[1], w3[2], w3[3]};
-    }
+      const bf16x8 p1 = __builtin_bit_cast(bf16x8, uint4{w1[0], w1[1], w1[2], w1[3]});
+      const bf16x8 p2 = __builtin_bit_cast(bf16x8, uint4{w2[0], w2[1], w2[2], w2[3]});
+      const bf16x8 p3 = __builtin_bit_cast(bf16x8, uint4{w3[0], w3[1], w3[2], w3[3]});
 #pragma unroll
-    for (int dt = 0; dt < NV; ++dt)
+      for (int d0 = 0; d0 < NV; d0 += 4) {  // four tiles of the output at a time: their chains of products overlap
+        bf16x8 v8[4];
 #pragma unroll
-      for (int a = 0; a < 2; ++a) {
-        const bf16x8 v8 = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(Vt + (32 * dt + c) * ldv + 16 * a + 8 * h));
+        for (int dt = d0; dt < NV && dt < d0 + 4; ++dt)
+          v8[dt - d0] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(Vt + (32 * dt + c) * ldv + 16 * a + 8 * h));
 #pragma unroll
         for (int pc = 2; pc >= 0; --pc)  // the smallest pieces first
-          o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8, __builtin_bit_cast(bf16x8, piece[pc][a]), o[dt], 0, 0, 0);
+#pragma unroll
+          for (int dt = d0; dt < NV && dt < d0 + 4; ++dt)
+            o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v8[dt - d0], pc == 2 ? p3 : pc == 1 ? p2 : p1, o[dt], 0, 0, 0);
       }
+    }
   }
 
   if (!active) return;
   l += __shfl_xor(l, 32, 64);
   if (!live) return;
-  float f = softmax_factor(m, l, sink, head) * out_scale;
+  if (part && n_chunks > per) {  // the tile's other chunks are other blocks'
+    float* dst = part + ((static_cast<size_t>(t0 + c) * nq + head) * gridDim.z + blockIdx.z) * (dv + 4);
+#pragma unroll
+    for (int dt = 0; dt < NV; ++dt)
+#pragma unroll
+      for (int a = 0; a < 4; ++a) {
+        const int d = 32 * dt + 8 * a + 4 * h;
+        if (d < dv) *reinterpret_cast<float4*>(dst + d) = float4{o[dt][4 * a], o[dt][4 * a + 1], o[dt][4 * a + 2], o[dt][4 * a + 3]};
+      }
+    if (h == 0) dst[dv] = m, dst[dv + 1] = l;
+    return;
+  }
+  float f = softmax_factor2(m, l, sink, head) * out_scale;
   const float* grow = gate ? gate + (static_cast<size_t>(t0 + c) * nq + head) * gate_dim : nullptr;
   if (gate && gate_dim == 1) f *= grow[0];
   bf16* dst = out + static_cast<size_t>(t0 + c) * out_ld + head * dv;
@@ -616,6 +709,42 @@ __global__ __launch_bounds__(kThreads) void attn_biased_tile16_kernel(
       const int d = 32 * dt + 8 * (i >> 2) + 4 * h + (i & 3);
       if (d < dv) dst[d] = from_float<bf16>(o[dt][i] * (gate_dim > 1 && gate ? f * grow[d] : f));
     }
+}
+
+// What the blocks of a long tile left, added up in the order of its chunks: a block per tile and head.
+__global__ __launch_bounds__(kThreads) void attn_tile_join_kernel(
+    const float* __restrict__ part, bf16* __restrict__ out, int out_ld, const float* __restrict__ gate, float out_scale,
+    const int* __restrict__ tiles, const int* __restrict__ positions, int nq, int dv, int window, int keep_first, int chunk,
+    int splits, int per, const float* __restrict__ sink, int gate_dim) {
+  const int t0 = tiles[2 * blockIdx.x], ntok = tiles[2 * blockIdx.x + 1], head = blockIdx.y;
+  if (ntok <= 0) return;
+  const int pieces = min((tile_chunks(positions[t0], ntok, window, keep_first, chunk).n_chunks + per - 1) / per, splits);
+  if (pieces <= 1) return;  // finished where it was made
+  const int quads = dv / 4;
+  for (int i = threadIdx.x; i < ntok * quads; i += kThreads) {
+    const int n = t0 + i / quads, d = 4 * (i % quads);
+    const float* src = part + (static_cast<size_t>(n) * nq + head) * splits * (dv + 4);
+    float M = sink ? sink[head] * kLog2e : -INFINITY;
+    for (int p = 0; p < pieces; ++p) M = fmaxf(M, src[p * (dv + 4) + dv]);
+    float l = sink ? __builtin_amdgcn_exp2f(sink[head] * kLog2e - M) : 0.f;
+    float4 o = {0.f, 0.f, 0.f, 0.f};
+    for (int p = 0; p < pieces; ++p) {
+      const float w = __builtin_amdgcn_exp2f(src[p * (dv + 4) + dv] - M);  // (a piece whose keys a token does not see: 0)
+      const float4 v = *reinterpret_cast<const float4*>(src + p * (dv + 4) + d);
+      l = fmaf(src[p * (dv + 4) + dv + 1], w, l);
+      o = float4{fmaf(v.x, w, o.x), fmaf(v.y, w, o.y), fmaf(v.z, w, o.z), fmaf(v.w, w, o.w)};
+    }
+    float f = (l > 0.f ? 1.f / l : 0.f) * out_scale;
+    float4 g = {f, f, f, f};
+    if (gate) {
+      const float* grow = gate + (static_cast<size_t>(n) * nq + head) * gate_dim;
+      if (gate_dim > 1) g = float4{f * grow[d], f * grow[d + 1], f * grow[d + 2], f * grow[d + 3]};
+      else g = float4{f * grow[0], f * grow[0], f * grow[0], f * grow[0]};
+    }
+    bf16* dst = out + static_cast<size_t>(n) * out_ld + head * dv + d;
+    dst[0] = from_float<bf16>(o.x * g.x), dst[1] = from_float<bf16>(o.y * g.y);
+    dst[2] = from_float<bf16>(o.z * g.z), dst[3] = from_float<bf16>(o.w * g.w);
+  }
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -829,11 +958,14 @@ extern "C" int pyre_attn_biased_tile(const void* q, void* out, int out_ld, int d
                                      const int* positions, const int* seq_of_token, const int* block_table,
                                      int table_stride, int nq, int nkv, int dk, int dv, int page_size, float scale,
                                      float cap, const float* bias, int far, int window, int keep_first, int chunk,
-                                     const float* sink, int gate_dim, hipStream_t stream) {
+                                     const float* sink, int gate_dim, float* part, int splits, int per,
+                                     hipStream_t stream) {
   if (check_geometry("attn_biased_tile", nq, nkv, dk, dv, page_size)) return 1;
   PYRE_REQUIRE(gate_dim == 1 || gate_dim == dv, "attn_biased_tile: a gate per head or per element, not per %d", gate_dim);
   PYRE_REQUIRE(known_dtype(dt) && table_stride > 0 && window >= 0 && keep_first >= 0 && far >= 0 && chunk >= 0, "attn_biased_tile: bad arguments");
   PYRE_REQUIRE(dk <= kTileMaxKeyHead, "attn_biased_tile: key heads of %d elements are more than %d", dk, kTileMaxKeyHead);
+  PYRE_REQUIRE(!part || (splits >= 1 && splits <= 65535 && per >= 1 && reinterpret_cast<uintptr_t>(part) % 16 == 0),
+               "attn_biased_tile: %d blocks of %d chunks a tile are not a launch", splits, per);
   if (n_tiles <= 0) return 0;
   const int hgroups = (nq / nkv + 3) / 4;
   PYRE_REQUIRE(nkv * hgroups <= 65535, "attn_biased_tile: grid too large");
@@ -870,28 +1002,37 @@ extern "C" int pyre_attn_biased_tile(const void* q, void* out, int out_ld, int d
   }
   const bool vec = dk % 8 == 0 && dv % 8 == 0 && reinterpret_cast<uintptr_t>(k_cache) % 16 == 0 &&
                    reinterpret_cast<uintptr_t>(v_cache) % 16 == 0 && reinterpret_cast<uintptr_t>(q) % 16 == 0;
-  if (dt == kBF16 && vec) {  // the 16-bit instruction, scores and weights in 32 bits all the same
+  const bool pow2_pages = (page_size & (page_size - 1)) == 0;
+  if (dt == kBF16 && vec && pow2_pages) {  // the 16-bit instruction, scores and weights in 32 bits all the same
     const int ldk = dkp + kPad16, ldv = kKeys + kPad16;
+    const int page_shift = __builtin_ctz(page_size);
+    float* pieces = part && splits > 1 ? part : nullptr;
+    const dim3 grid16(n_tiles, nkv * hgroups, pieces ? splits : 1);
     size_t lds16 = sizeof(bf16) * (static_cast<size_t>(kKeys + 4 * 32) * ldk + 32 * nvp * ldv);
     lds16 = (lds16 + 15) / 16 * 16;
     const int tab16 = lds16 + sizeof(int) * table_stride <= 48 * 1024 ? table_stride : 0;
     lds16 += sizeof(int) * tab16;
     const int bias16 = bias && lds16 + sizeof(float) * 4 * (far + 1) <= 52 * 1024 ? 1 : 0;
     lds16 += bias16 ? sizeof(float) * 4 * (far + 1) : 0;
-#define PYRE_TILE16(NV)                                                                                                  \
+#define PYRE_TILE16(NV)              \
+  do {                               \
+    if (tab16) PYRE_TILE16T(NV, true); \
+    else PYRE_TILE16T(NV, false);    \
+  } while (0)
+#define PYRE_TILE16T(NV, TAB)                                                                                            \
   do {                                                                                                                   \
     static size_t raised = 64 * 1024;                                                                                    \
     if (lds16 > raised) {                                                                                                \
-      if (hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_biased_tile16_kernel<NV>),                             \
+      if (hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_biased_tile16_kernel<NV, TAB>),                        \
                               hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds16)) != hipSuccess)        \
         return fail("attn_biased_tile: the device refuses %zu bytes of LDS", lds16);                                     \
       raised = lds16;                                                                                                    \
     }                                                                                                                    \
-    hipLaunchKernelGGL((attn_biased_tile16_kernel<NV>), grid, dim3(kThreads), lds16, stream, static_cast<const bf16*>(q), \
+    hipLaunchKernelGGL((attn_biased_tile16_kernel<NV, TAB>), grid16, dim3(kThreads), lds16, stream, static_cast<const bf16*>(q), \
                        static_cast<const bf16*>(k_cache), static_cast<const bf16*>(v_cache), static_cast<bf16*>(out),    \
                        out_ld, gate, out_scale, tiles, positions, seq_of_token, block_table, table_stride, nq, nkv, dk,  \
-                       dkp, dv, page_size, scale, cap, bias, far, window, keep_first, chunk, tab16, bias16, sink,         \
-                       gate_dim);                                                                                        \
+                       dkp, dv, page_shift, scale, cap, bias, far, window, keep_first, chunk, tab16, bias16,   \
+                       sink, gate_dim, pieces, per);                                                                     \
   } while (0)
     switch (nvp) {
       case 1: PYRE_TILE16(1); break;
@@ -900,7 +1041,12 @@ extern "C" int pyre_attn_biased_tile(const void* q, void* out, int out_ld, int d
       default: PYRE_TILE16(8); break;
     }
 #undef PYRE_TILE16
-    return check_launch("attn_biased_tile");
+#undef PYRE_TILE16T
+    if (check_launch("attn_biased_tile")) return 1;
+    if (pieces)
+      hipLaunchKernelGGL(attn_tile_join_kernel, dim3(n_tiles, nq), dim3(kThreads), 0, stream, pieces, static_cast<bf16*>(out), out_ld,
+                         gate, out_scale, tiles, positions, nq, dv, window, keep_first, chunk, splits, per, sink, gate_dim);
+    return check_launch("attn_tile_join");
   }
   if (dt == kF32) {
     if (vec) { PYRE_TILE_NV(float, true) } else { PYRE_TILE_NV(float, false) }

@@ -259,7 +259,8 @@ int pyre_attn_biased_tile(const void* q, void* out, int out_ld, int dt, const vo
                           const int* positions, const int* seq_of_token, const int* block_table,
                           int table_stride, int nq, int nkv, int dk, int dv, int page_size, float scale,
                           float cap, const float* bias, int far, int window, int keep_first, int chunk,
-                          const float* sink, int gate_dim, hipStream_t stream);
+                          const float* sink, int gate_dim, float* part, int splits,
+                          int per, hipStream_t stream);
 // tokens: the n tokens of the flat batch to attend for (null: 0..n-1), a block per token and head.
 int pyre_attn_biased_single(const void* q, void* out, int out_ld, int dt, const void* k_cache,
                             const void* v_cache, const float* gate, float out_scale, const int* tokens,

@@ -61,7 +61,7 @@ _SIGNATURES = {
     "pyre_stream_norm": [P, I, P, I, P, I, I, L, P, P, P, P, P, I, F, P, I, P, I, I, P],
     "pyre_poly_norm": [P, I, I, L, P, F, P, I, I, I, P],
     "pyre_unit_qkv_write": [P, I, I, L, I, I, P, I, P, P, I, P, P, I, I, I, I, I, I, I, F, I, P],
-    "pyre_attn_biased_tile": [P, P, I, I, P, P, P, F, P, I, P, P, P, I, I, I, I, I, I, F, F, P, I, I, I, I, P, I, P],
+    "pyre_attn_biased_tile": [P, P, I, I, P, P, P, F, P, I, P, P, P, I, I, I, I, I, I, F, F, P, I, I, I, I, P, I, P, I, I, P],
     "pyre_attn_biased_single": [P, P, I, I, P, P, P, F, P, I, P, P, P, I, I, I, I, I, I, F, F, P, I, I, I, I, P, I, P, I, P],
     "pyre_attn_biased_spans": [I, I, I, I],
     "pyre_gla_prepare": [P, I, I, L, I, I, P, I, P, I, F, P, I, I, I, I, I, P],

@@ -17,6 +17,9 @@ from pyre_amd.hip.lib import KernelError, call
 
 _DT = {torch.float32: 0, torch.bfloat16: 1}
 
+#: compute units that launch plans are made for when nobody names a device (an MI355X)
+DEFAULT_UNITS = 256
+
 
 def dtype_code(t: torch.Tensor | torch.dtype) -> int:
     dt = t if isinstance(t, torch.dtype) else t.dtype
@@ -310,20 +313,49 @@ def _attn_biased_common(q, out, k_cache, v_cache, gate, positions, seq_of_token,
         raise KernelError(f"attn_biased: the bias by distance is float32 [{nq}, {far + 1}]")
 
 
+ATTN_TILE_SPLITS = 8     #: the most blocks that a tile's keys are dealt to
+ATTN_TILE_MIN_CHUNKS = 6  #: the fewest chunks of 32 keys that are worth a block of their own
+
+
+def attn_biased_tile_plan(n_tiles: int, nq: int, nkv: int, max_keys: int, window: int = 0, keep_first: int = 0, chunk: int = 0,
+                          units: int = DEFAULT_UNITS) -> tuple[int, int]:
+    """(splits, chunks a block) for a launch of the 16-bit tile kernel whose longest tile sees ``max_keys`` keys: as many
+    blocks as give every compute unit six (three share one at a time), since a short prompt's tiles of few heads leave the
+    chip to the few blocks that see the most keys. (1, ..): whole tiles."""
+    keys = max_keys
+    if window > 0:
+        keys = min(keys, window + keep_first + 64)
+    if chunk > 0:
+        keys = min(keys, chunk + 64)
+    chunks = -(-max(keys, 1) // 32)
+    blocks = max(1, n_tiles * nkv * -(-(nq // nkv) // 4))
+    splits = max(1, min(ATTN_TILE_SPLITS, 6 * units // blocks, chunks // ATTN_TILE_MIN_CHUNKS))
+    return splits, -(-chunks // splits)
+
+
 def attn_biased_tile(q, out, k_cache, v_cache, gate, out_scale, tiles, n_tiles, positions, seq_of_token,
                      block_table, nq, nkv, dk, dv, page_size, scale, cap, bias, far, window, keep_first, chunk: int = 0,
-                     sink: torch.Tensor | None = None, gate_dim: int = 1) -> None:
+                     sink: torch.Tensor | None = None, gate_dim: int = 1, scratch: torch.Tensor | None = None,
+                     splits: int = 1, per: int = 1) -> None:
     """Prompt portions of the capped, biased attention; ``tiles`` is int32 [n_tiles, 2] = (first token, count <= 32).
     ``sink`` (float32 [nq]): exp(sink) of the head joins the softmax's denominator, a key without a value.
-    ``gate_dim`` = dv: ``gate`` is [N, nq*dv], a gate per element of the output."""
+    ``gate_dim`` = dv: ``gate`` is [N, nq*dv], a gate per element of the output. ``scratch`` (float32, N * nq * splits *
+    (dv + 4) elements): in the 16-bit form a tile's chunks of 32 keys are dealt to ``splits`` blocks, ``per`` chunks each
+    (the last takes what is left; :func:`attn_biased_tile_plan`), whose results a second kernel joins."""
     _attn_biased_common(q, out, k_cache, v_cache, gate, positions, seq_of_token, block_table, bias, far,
                         nq, nkv, dk, dv, page_size, sink, gate_dim)
     _i32("tiles", tiles, 2 * n_tiles)
+    if scratch is not None:
+        _dev(scratch)
+        rows = q.numel() // (nq * dk)
+        if scratch.dtype != torch.float32 or not scratch.is_contiguous() or scratch.numel() < rows * nq * splits * (dv + 4) or \
+                splits < 1 or per < 1:
+            raise KernelError(f"attn_biased_tile: scratch of {rows * nq * splits * (dv + 4)} float32 elements needed")
     call("pyre_attn_biased_tile", q.data_ptr(), out.data_ptr(), out.stride(0), dtype_code(q), k_cache.data_ptr(),
          v_cache.data_ptr(), _ptr(gate), float(out_scale), tiles.data_ptr(), n_tiles, positions.data_ptr(),
          seq_of_token.data_ptr(), block_table.data_ptr(), block_table.stride(0), nq, nkv, dk, dv, page_size,
          float(scale), float(cap), _ptr(bias), int(far), int(window), int(keep_first), int(chunk), _ptr(sink),
-         int(gate_dim), _stream())
+         int(gate_dim), _ptr(scratch), int(splits), int(per), _stream())
 
 
 def attn_biased_spans(table_width: int, page_size: int, window: int, keep_first: int, chunk: int = 0) -> int:
@@ -560,9 +592,6 @@ def gemm_generic(a: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None, ou
 
 
 F32_KSPLIT_MAX = 8
-
-#: compute units that launch plans are made for when nobody names a device (an MI355X)
-DEFAULT_UNITS = 256
 
 
 def compute_units(device=None) -> int:

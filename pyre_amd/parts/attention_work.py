@@ -229,3 +229,22 @@ def prefill_slots(work: np.ndarray) -> int:
     """Partial slots that a work list of :func:`prefill_work` uses."""
     shared = work[:, 6] > 1
     return int((work[shared, 4] + work[shared, 6]).max()) if shared.any() else 0
+
+
+def biased_tile_scratch(ctx, n_tiles: int, heads: int, kv_heads: int, value_dim: int, window: int = 0, keep_first: int = 0,
+                        chunk: int = 0) -> dict:
+    """The arguments by which :func:`pyre_amd.hip.ops.attn_biased_tile` deals long tiles of a 16-bit step to several
+    blocks (none where whole tiles fill the chip): what :func:`~pyre_amd.hip.ops.attn_biased_tile_plan` says, and scratch
+    for the blocks' results."""
+    import torch
+
+    from pyre_amd.hip import ops
+
+    if ctx.dtype != torch.bfloat16:
+        return {}
+    splits, per = ops.attn_biased_tile_plan(n_tiles, heads, kv_heads, int(ctx.host.ctx_len.max()), window, keep_first, chunk,
+                                            ctx.runtime.compute_units)
+    if splits <= 1:
+        return {}
+    scratch = ctx.workspace.get("attn.tile_parts", (ctx.n_tokens * heads * splits * (value_dim + 4),), torch.float32)
+    return dict(scratch=scratch, splits=splits, per=per)

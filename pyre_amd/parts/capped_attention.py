@@ -10,6 +10,7 @@ import torch
 
 from pyre_amd.hip import ops
 from pyre_amd.parts.attention import STEP_ARRAYS
+from pyre_amd.parts.attention_work import biased_tile_scratch
 from pyre_amd.parts.base import (CappedAttentionSpec, PagedCacheSpec, PagedTensorSpec, TensorSpec, take)
 from pyre_amd.parts.branch import BranchMixer
 
@@ -111,7 +112,8 @@ class CappedAttention(BranchMixer):
             return
         if len(tiles):
             ops.attn_biased_tile(q, o, k_pages, v_pages, gate, scale, ctx.arrays["attention.prefill_tiles"], len(tiles),
-                                 ctx.positions, ctx.seq_of_token, cache.table, *shape)
+                                 ctx.positions, ctx.seq_of_token, cache.table, *shape,
+                                 **biased_tile_scratch(ctx, len(tiles), s.num_heads, s.num_kv_heads, s.value_dim, s.window, s.keep_first))
         if len(singles):
             # a block per span of 128 keys, joined by a second kernel: a step of few tokens fills the chip that way
             spans = ops.attn_biased_spans(cache.table.shape[1], cache.page_size, s.window, s.keep_first)

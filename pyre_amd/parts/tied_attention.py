@@ -6,6 +6,7 @@ import torch
 
 from pyre_amd.hip import ops
 from pyre_amd.parts.attention import STEP_ARRAYS
+from pyre_amd.parts.attention_work import biased_tile_scratch
 from pyre_amd.parts.base import Mixer, PagedCacheSpec, PagedTensorSpec, TensorSpec, TiedAttentionSpec, make_part, take
 from pyre_amd.parts.linear import Linear
 
@@ -28,7 +29,8 @@ def attend_pages(ctx, q, o, k_pages, v_pages, cache, nq: int, nkv: int, dk: int,
         return
     if len(tiles):
         ops.attn_biased_tile(q, o, k_pages, v_pages, None, 1.0, ctx.arrays["attention.prefill_tiles"], len(tiles),
-                             ctx.positions, ctx.seq_of_token, cache.table, *shape, chunk=chunk)
+                             ctx.positions, ctx.seq_of_token, cache.table, *shape, chunk=chunk,
+                             **biased_tile_scratch(ctx, len(tiles), nq, nkv, dv, chunk=chunk))
     if len(singles):
         spans = ops.attn_biased_spans(cache.table.shape[1], cache.page_size, 0, 0, chunk)
         scratch = None

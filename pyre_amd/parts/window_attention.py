@@ -7,6 +7,7 @@ import torch
 
 from pyre_amd.hip import ops
 from pyre_amd.parts.attention import STEP_ARRAYS
+from pyre_amd.parts.attention_work import biased_tile_scratch
 from pyre_amd.parts.base import PagedCacheSpec, PagedTensorSpec, TensorSpec, WindowAttentionSpec, make_part, take
 from pyre_amd.parts.branch import BranchMixer
 
@@ -107,7 +108,8 @@ class WindowAttention(BranchMixer):
             return
         if len(tiles):
             ops.attn_biased_tile(q, o, k_pages, v_pages, None, scale, ctx.arrays["attention.prefill_tiles"], len(tiles),
-                                 ctx.positions, ctx.seq_of_token, pages.table, *shape, **extra)
+                                 ctx.positions, ctx.seq_of_token, pages.table, *shape, **extra,
+                                 **biased_tile_scratch(ctx, len(tiles), s.num_heads, s.num_kv_heads, s.value_dim, s.window))
         if len(singles):
             # a block per span of 128 keys, joined by a second kernel: a step of few tokens fills the chip that way
             spans = ops.attn_biased_spans(pages.table.shape[1], pages.page_size, s.window, 0)

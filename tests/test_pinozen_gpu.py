@@ -622,6 +622,72 @@ def test_a_convolutions_state_in_a_step_of_single_tokens(dk, dv, taps):
             assert close(got[0][3][slot], torch.cat([state[slot, 1:].double(), u[s:s + 1]]).cpu(), 1e-6)
 
 
+@pytest.mark.parametrize("nq,nkv,dk,dv,window,keep,cap,with_sink,gate_dim", [
+    (6, 2, 64, 40, 0, 0, 20.0, True, 0), (5, 1, 128, 128, 0, 0, 0.0, True, 0), (4, 4, 24, 64, 300, 5, 5.0, False, 1), (3, 1, 96, 16, 40, 0, 0.0, True, 2),
+    (9, 1, 32, 136, 0, 0, 3.0, False, 2)])
+def test_tiles_whose_keys_are_dealt_to_several_blocks(nq, nkv, dk, dv, window, keep, cap, with_sink, gate_dim):
+    """The 16-bit tile kernel whole and in parts against float64 on the same values, to the rounding of the output; two
+    requests, one that goes on behind earlier keys, tiles that are not full, parts that hold all, some or one chunk."""
+    from pyre_amd.hip import ops
+
+    g = torch.Generator().manual_seed(nq * dk + window)
+    page, lens, first = 16, (700, 90), (0, 61)          # the second request brings its tokens 61 .. 89
+    rows = [(r, t) for r in (0, 1) for t in range(first[r], lens[r])]
+    n = len(rows)
+    ks, vs = [torch.randn(m, nkv, dk, generator=g).bfloat16() for m in lens], [torch.randn(m, nkv, dv, generator=g).bfloat16() for m in lens]
+    q = torch.randn(n, nq, dk, generator=g).bfloat16()
+    pages = [-(-m // page) for m in lens]
+    order = torch.randperm(sum(pages) + 3, generator=g)
+    kc, vc = (torch.full((sum(pages) + 3, nkv, page, d), float("nan"), dtype=torch.bfloat16) for d in (dk, dv))
+    table = torch.full((2, pages[0]), -1, dtype=torch.int32)
+    for r in (0, 1):
+        table[r, :pages[r]] = order[r * pages[0]:r * pages[0] + pages[r]].int()
+        for t in range(lens[r]):
+            kc[table[r, t // page], :, t % page], vc[table[r, t // page], :, t % page] = ks[r][t], vs[r][t]
+    sink = torch.randn(nq, generator=g) + 2
+    gate = torch.rand(n, nq * (dv if gate_dim == 2 else 1), generator=g) if gate_dim else None
+    scale = 2.0 / dk ** 0.5
+    want, at = torch.zeros(n, nq, dv, dtype=torch.float64), 0
+    for r in (0, 1):
+        i, j = torch.arange(first[r], lens[r])[:, None], torch.arange(lens[r])[None]
+        seen = (j <= i) & (((i - j < window) | (j < keep)) if window else torch.ones(1, dtype=torch.bool))
+        for head in range(nq):
+            m = lens[r] - first[r]
+            x = q[at:at + m, head].double() @ ks[r][:, head // (nq // nkv)].double().T * scale
+            x = (cap * torch.tanh(x / cap) if cap else x).masked_fill(~seen, -math.inf)
+            if with_sink:
+                x = torch.cat([x, sink[head].double().expand(m, 1)], 1)
+            want[at:at + m, head] = torch.softmax(x, -1)[:, :lens[r]] @ vs[r][:, head // (nq // nkv)].double()
+        at += lens[r] - first[r]
+    if gate is not None:
+        want = want * gate.double().view(n, nq, -1)
+    want = (want * 0.5).reshape(n, -1)
+    tiles = [(t, min(32, 700 - t)) for t in range(0, 700, 32)] + [(700, 5), (705, 24)]
+    d = lambda t: None if t is None else t.contiguous().to(DEV)  # noqa: E731
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=DEV)  # noqa: E731
+    args = (i32(tiles), len(tiles), i32([t for _, t in rows]), i32([r for r, _ in rows]), d(table), nq, nkv, dk, dv, page, scale, cap, None, 0, window, keep)
+    ulp = 2.0 ** -8
+    for splits, per in ((1, 1), (2, 11), (3, 4), (8, 3), (8, 1), (5, 40)):
+        out = torch.zeros(n, nq * dv + 8, device=DEV, dtype=torch.bfloat16)
+        scratch = torch.full((n * nq * splits * (dv + 4),), float("nan"), device=DEV) if splits > 1 else None
+        ops.attn_biased_tile(d(q.view(n, -1)), out, d(kc), d(vc), d(gate), 0.5, *args, sink=d(sink) if with_sink else None,
+                             gate_dim=dv if gate_dim == 2 else 1, scratch=scratch, splits=splits, per=per)
+        got = out[:, :nq * dv].cpu().double()
+        assert bool(((got - want).abs() <= ulp * want.abs() + 4e-6).all()), (splits, per, float(((got - want).abs() - ulp * want.abs()).max()))
+        assert not bool(out[:, nq * dv:].any())
+
+
+def test_the_plan_of_a_tiles_parts():
+    from pyre_amd.hip.ops import attn_biased_tile_plan
+
+    for args in ((64, 14, 2, 2048), (1, 4, 2, 33), (3, 8, 8, 100000), (64, 28, 4, 32768), (64, 14, 2, 2048, 1024, 4), (5, 3, 1, 700, 0, 0, 64)):
+        splits, per = attn_biased_tile_plan(*args, units=256)
+        assert splits >= 1 and per >= 1 and (splits - 1) * per < -(-args[3] // 32)
+    assert attn_biased_tile_plan(64, 14, 2, 2048, units=256) == (6, 11)
+    assert attn_biased_tile_plan(2048, 14, 2, 2048, units=256)[0] == 1        # many tiles fill the chip whole
+    assert attn_biased_tile_plan(1, 4, 2, 33, units=256)[0] == 1              # nothing to deal
+
+
 @pytest.mark.parametrize("rank,padded,parts", [(5, 8, 1), (16, 16, 3), (1, 8, 2), (24, 24, 1)])
 def test_operands_of_the_step_sizes_product(rank, padded, parts):
     from pyre_amd.hip import ops
