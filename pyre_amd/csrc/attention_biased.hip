@@ -21,7 +21,8 @@
 //                 heads of a key/value head per block, chunks of 32 keys through LDS, both products on
 //                 the matrix cores' float32 instruction (scores and weights stay float32).
 // attn_biased_single  single tokens: a block per (token, up to eight query heads of a key/value head), the keys in
-//                 spans of 128 that the block's heads read together.
+//                 spans of 128 that the block's heads read together; in bfloat16 on the matrix cores, up to sixteen heads a
+//                 block, a wave per 32 keys of a span.
 //
 // Chunks start at multiples of 32 keys and spans at the token's first visible key, so the order of
 // every sum of a token depends on its own bounds alone.
@@ -432,7 +433,7 @@ __device__ inline TileChunks tile_chunks(int pos0, int ntok, int window, int kee
   r.n_chunks = r.n_first + ((pos0 + ntok - 1) / kKeys - r.chunk_b + 1);
   return r;
 }
-constexpr float kLog2e = 1.44269504088896340736f;
+constexpr float kLog2e = 1.44269504088896340736f, kLn2 = 0.69314718055994530942f;
 // The same for a maximum and a sink in powers of two.
 __device__ inline float softmax_factor2(float m, float l, const float* sink, int head) {
   if (!sink) return l > 0.f ? 1.f / l : 0.f;
@@ -887,30 +888,211 @@ __global__ __launch_bounds__(kThreads) void attn_biased_single_kernel(
   }
 }
 
-// out = gate * out_scale * sum_s acc_s e^(m_s - M) / sum_s l_s e^(m_s - M) over the token's spans, in their order.
+// The same for bfloat16 queries and caches on the matrix cores: up to sixteen query heads of a key/value head are the columns
+// of 16 x 16 tiles, and a wave takes 32 keys of its block's span of 128 on its own. Scores S^T = K Q^T on the 16-bit
+// instruction (products of two bfloat16 values are exact in float32); a lane then holds its head's scores of eight keys in
+// the layout in which the float32 instruction wants the weights of O^T = V^T P^T, so weights stay float32 and go nowhere.
+// Row r of tile e of the output is element 8 r + e of the head (of each 128 elements): a lane's operands of eight tiles are
+// one 16-byte piece of a value, and a value's pieces are read side by side. The waves join their sums through LDS.
+// DKS: steps of 32 elements of the key head; EV: runs of 128 elements of the value head. Head sizes are multiples of
+// eight, the pages' size a power of two, the caches start on 16 bytes.
+constexpr int kCols = 16;
+template <int DKS, int EV>
+__global__ __launch_bounds__(kThreads) void attn_biased_single16_kernel(
+    const bf16* __restrict__ q, const bf16* __restrict__ k_cache, const bf16* __restrict__ v_cache, bf16* __restrict__ out,
+    int out_ld, const float* __restrict__ gate, float out_scale, const int* __restrict__ tokens,
+    const int* __restrict__ positions, const int* __restrict__ seq_of_token, const int* __restrict__ block_table,
+    int table_stride, int nq, int nkv, int dk, int dv, int page_shift, float scale, float cap, const float* __restrict__ bias,
+    int far, int window, int keep_first, int chunk, float* __restrict__ part, const float* __restrict__ sink, int gate_dim) {
+  extern __shared__ __attribute__((aligned(16))) float acc_s[];  // [4 waves][heads of the block][128 EV + 4]
+  __shared__ float m_s[4][kCols], l_s[4][kCols];
+  constexpr int kLd = 128 * EV + 4;
+  const int n = tokens ? tokens[blockIdx.x] : blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int r = lane & 15, g = lane >> 4;
+  const int rep = nq / nkv, hgroups = (rep + kCols - 1) / kCols;
+  const int kvh = blockIdx.y / hgroups, first = (blockIdx.y % hgroups) * kCols, nh = min(kCols, rep - first);
+  const int h0 = kvh * rep + first;
+  const int pos = positions[n];
+  const int* table = block_table + static_cast<size_t>(seq_of_token[n]) * table_stride;
+  const int lo = first_seen(pos, window, chunk);
+  const int kept_end = window > 0 ? min(keep_first, lo) : 0;
+  const int spans_first = (kept_end + kSpan - 1) / kSpan, span = blockIdx.z;
+  if (span >= spans_first + (pos - lo) / kSpan + 1) return;
+  const int base = span < spans_first ? span * kSpan : lo + (span - spans_first) * kSpan;
+  const int end = min(base + kSpan, span < spans_first ? kept_end : pos + 1);
+  const int key0 = base + 32 * wave;  // the wave's keys are key0 .. key0 + 31, those before `end`
+
+  // lane j < 32 finds key j's row in the cache
+  int row = -1;
+  if (lane < 32 && key0 + lane < end) {
+    const int key = key0 + lane, page = table[key >> page_shift];
+    if (page >= 0) row = (page << page_shift) | (key & ((1 << page_shift) - 1));
+  }
+  auto cache_row = [&](int row_) {  // rows of this head: [page][nkv][page size]
+    const int page = row_ >> page_shift, off = row_ & ((1 << page_shift) - 1);
+    return ((static_cast<size_t>(page) * nkv + kvh) << page_shift) + off;
+  };
+  const uint4 zero4 = {0u, 0u, 0u, 0u};
+  uint4 kr[2][DKS], vr[2][4][EV], qr[DKS];
+#pragma unroll
+  for (int st = 0; st < DKS; ++st) {
+    const int e = 32 * st + 8 * g;
+    qr[st] = r < nh && e < dk ? *reinterpret_cast<const uint4*>(q + (static_cast<size_t>(n) * nq + h0 + r) * dk + e) : zero4;
+  }
+#pragma unroll
+  for (int t = 0; t < 2; ++t) {
+    const size_t at = cache_row(max(__shfl(row, 16 * t + r, 64), 0)) * dk;  // a key that is not there: some key, hidden below
+#pragma unroll
+    for (int st = 0; st < DKS; ++st) kr[t][st] = *reinterpret_cast<const uint4*>(k_cache + at + (32 * st + 8 * g < dk ? 32 * st + 8 * g : 0));
+  }
+  unsigned there = 0;  // bit 4 t + i: key 16 t + 4 g + i
+#pragma unroll
+  for (int t = 0; t < 2; ++t)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int vrow = __shfl(row, 16 * t + 4 * g + i, 64);
+      there |= vrow >= 0 ? 1u << (4 * t + i) : 0u;
+      const size_t at = cache_row(max(vrow, 0)) * dv;
+#pragma unroll
+      for (int e = 0; e < EV; ++e) vr[t][i][e] = *reinterpret_cast<const uint4*>(v_cache + at + (128 * e + 8 * r < dv ? 128 * e + 8 * r : 0));
+    }
+  f32x4 s[2];
+#pragma unroll
+  for (int t = 0; t < 2; ++t) {
+    s[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int st = 0; st < DKS; ++st) {
+      const uint32_t w = 32 * st + 8 * g < dk ? ~0u : 0u;
+      const uint4 k4 = {kr[t][st].x & w, kr[t][st].y & w, kr[t][st].z & w, kr[t][st].w & w};
+      s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, k4), __builtin_bit_cast(bf16x8, qr[st]), s[t], 0, 0, 0);
+    }
+  }
+  // element i of s[t]: key key0 + 16 t + 4 g + i, head r; scores times log2(e)
+  const float to2 = scale * kLog2e, cap2 = cap * kLog2e, bend = cap > 0.f ? -2.f * to2 / cap : 0.f;
+  const float* bias_row = bias && r < nh ? bias + static_cast<size_t>(h0 + r) * (far + 1) : nullptr;
+  float m = -INFINITY;
+#pragma unroll
+  for (int t = 0; t < 2; ++t)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      float x;
+      if (cap > 0.f) {
+        const float e = __builtin_amdgcn_exp2f(bend * fabsf(s[t][i]));
+        x = copysignf((1.f - e) * __builtin_amdgcn_rcpf(1.f + e) * cap2, s[t][i]);
+      } else {
+        x = s[t][i] * to2;
+      }
+      if (bias_row) x = fmaf(bias_row[min(max(pos - (key0 + 16 * t + 4 * g + i), 0), far)], kLog2e, x);
+      s[t][i] = there >> (4 * t + i) & 1u ? x : -INFINITY;
+      m = fmaxf(m, s[t][i]);
+    }
+  m = fmaxf(m, __shfl_xor(m, 16, 64));
+  m = fmaxf(m, __shfl_xor(m, 32, 64));
+  const float m_use = m == -INFINITY ? 0.f : m;
+  float l = 0.f;
+#pragma unroll
+  for (int t = 0; t < 2; ++t)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      s[t][i] = __builtin_amdgcn_exp2f(s[t][i] - m_use);
+      l += s[t][i];
+    }
+  l += __shfl_xor(l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  f32x4 o[8 * EV];
+#pragma unroll
+  for (int e = 0; e < 8 * EV; ++e) o[e] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int t = 0; t < 2; ++t)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const uint32_t w = there >> (4 * t + i) & 1u ? ~0u : 0u;  // what a page held before is no number to multiply with
+#pragma unroll
+      for (int e = 0; e < EV; ++e) {
+        const uint32_t v[4] = {vr[t][i][e].x & w, vr[t][i][e].y & w, vr[t][i][e].z & w, vr[t][i][e].w & w};
+#pragma unroll
+        for (int u = 0; u < 8; ++u)
+          o[8 * e + u] = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(u & 1 ? v[u >> 1] & 0xffff0000u : v[u >> 1] << 16), s[t][i],
+                                                              o[8 * e + u], 0, 0, 0);
+      }
+    }
+  if (g == 0) m_s[wave][r] = m, l_s[wave][r] = l;
+  if (r < nh) {  // element i of o[8 e + u]: element 128 e + 8 (4 g + i) + u of head r
+    float* dst = acc_s + (wave * nh + r) * kLd;
+#pragma unroll
+    for (int e = 0; e < EV; ++e)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = 128 * e + 8 * (4 * g + i);
+        *reinterpret_cast<f32x4*>(dst + d) = f32x4{o[8 * e][i], o[8 * e + 1][i], o[8 * e + 2][i], o[8 * e + 3][i]};
+        *reinterpret_cast<f32x4*>(dst + d + 4) = f32x4{o[8 * e + 4][i], o[8 * e + 5][i], o[8 * e + 6][i], o[8 * e + 7][i]};
+      }
+  }
+  __syncthreads();
+  for (int i = tid; i < nh * dv; i += kThreads) {
+    const int a = i / dv, d = i % dv, hd = h0 + a;
+    const float M = fmaxf(fmaxf(m_s[0][a], m_s[1][a]), fmaxf(m_s[2][a], m_s[3][a]));
+    const float M_use = M == -INFINITY ? 0.f : M;
+    float total = 0.f, sum = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const float f = __builtin_amdgcn_exp2f(m_s[w][a] - M_use);
+      total = fmaf(acc_s[(w * nh + a) * kLd + d], f, total);
+      sum = fmaf(l_s[w][a], f, sum);
+    }
+    if (part) {  // as the kernel above leaves it: the maximum of the scores themselves
+      float* dst = part + ((static_cast<size_t>(blockIdx.x) * nq + hd) * gridDim.z + blockIdx.z) * (dv + 2);
+      dst[d] = total;
+      if (d == 0) dst[dv] = M * kLn2, dst[dv + 1] = sum;
+      continue;
+    }
+    float f = softmax_factor2(M, sum, sink, hd) * out_scale;
+    if (gate) f *= gate[(static_cast<size_t>(n) * nq + hd) * gate_dim + (gate_dim > 1 ? d : 0)];
+    out[static_cast<size_t>(n) * out_ld + hd * dv + d] = from_float<bf16>(total * f);
+  }
+}
+
+// out = gate * out_scale * sum_s acc_s e^(m_s - M) / sum_s l_s e^(m_s - M) over the token's spans: a block per token and head,
+// kThreads / dv groups of threads that take the spans in turn (eight of them asked for together), joined in their order.
 template <typename T>
 __global__ __launch_bounds__(kThreads) void attn_biased_join_kernel(
     const float* __restrict__ part, T* __restrict__ out, int out_ld, const float* __restrict__ gate, float out_scale,
     const int* __restrict__ tokens, const int* __restrict__ positions, int nq, int dv, int window, int keep_first,
     int chunk, int max_spans, const float* __restrict__ sink, int gate_dim) {
+  __shared__ float total_s[kThreads], scratch[16];
   const int n = tokens ? tokens[blockIdx.x] : blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int pos = positions[n];
   const int lo = first_seen(pos, window, chunk);
   const int kept_end = window > 0 ? min(keep_first, lo) : 0;
   const int spans = min(max_spans, (kept_end + kSpan - 1) / kSpan + (pos - lo) / kSpan + 1);
   const float* src = part + (static_cast<size_t>(blockIdx.x) * nq + h) * max_spans * (dv + 2);
-  float M = -INFINITY;
-  for (int s = 0; s < spans; ++s) M = fmaxf(M, src[s * (dv + 2) + dv]);
-  if (sink) M = fmaxf(M, sink[h]);
+  float M = sink ? sink[h] : -INFINITY;
+  for (int s = tid; s < spans; s += kThreads) M = fmaxf(M, src[static_cast<size_t>(s) * (dv + 2) + dv]);
+  M = block_max(M, scratch);
   const float m_use = M == -INFINITY ? 0.f : M;
-  if (tid < dv) {
-    float total = 0.f, l = 0.f;
-    for (int s = 0; s < spans; ++s) {
-      const float w = expf(src[s * (dv + 2) + dv] - m_use);
-      total = fmaf(src[s * (dv + 2) + tid], w, total);
-      l = fmaf(src[s * (dv + 2) + dv + 1], w, l);
+  float l = 0.f;
+  for (int s = tid; s < spans; s += kThreads)
+    l = fmaf(src[static_cast<size_t>(s) * (dv + 2) + dv + 1], expf(src[static_cast<size_t>(s) * (dv + 2) + dv] - m_use), l);
+  l = block_sum(l, scratch);
+  if (sink) l += expf(sink[h] - m_use);
+  const int groups = kThreads / dv, grp = tid / dv, d = tid % dv;
+  float total = 0.f;
+  if (grp < groups)
+    for (int s0 = grp; s0 < spans; s0 += 8 * groups) {
+      float v[8], mm[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const float* p = src + static_cast<size_t>(min(s0 + u * groups, spans - 1)) * (dv + 2);
+        v[u] = p[d], mm[u] = p[dv];
+      }
+#pragma unroll
+      for (int u = 0; u < 8; ++u)
+        if (s0 + u * groups < spans) total = fmaf(v[u], expf(mm[u] - m_use), total);
     }
-    if (sink) l += expf(sink[h] - m_use);
+  total_s[tid] = total;
+  __syncthreads();
+  if (tid < dv) {
+    for (int a = 1; a < groups; ++a) total += total_s[a * dv + tid];
     float f = (l > 0.f ? 1.f / l : 0.f) * out_scale;
     if (gate) f *= gate[(static_cast<size_t>(n) * nq + h) * gate_dim + (gate_dim > 1 ? tid : 0)];
     out[static_cast<size_t>(n) * out_ld + h * dv + tid] = from_float<T>(total * f);
@@ -1010,9 +1192,10 @@ extern "C" int pyre_attn_biased_tile(const void* q, void* out, int out_ld, int d
     const dim3 grid16(n_tiles, nkv * hgroups, pieces ? splits : 1);
     size_t lds16 = sizeof(bf16) * (static_cast<size_t>(kKeys + 4 * 32) * ldk + 32 * nvp * ldv);
     lds16 = (lds16 + 15) / 16 * 16;
-    const int tab16 = lds16 + sizeof(int) * table_stride <= 48 * 1024 ? table_stride : 0;
+    const size_t budget16 = nvp <= 4 ? 78 * 1024 : 150 * 1024;  // two blocks share a compute unit, or one has it alone
+    const int tab16 = lds16 + sizeof(int) * table_stride <= budget16 ? table_stride : 0;
     lds16 += sizeof(int) * tab16;
-    const int bias16 = bias && lds16 + sizeof(float) * 4 * (far + 1) <= 52 * 1024 ? 1 : 0;
+    const int bias16 = bias && lds16 + sizeof(float) * 4 * (far + 1) <= budget16 ? 1 : 0;
     lds16 += bias16 ? sizeof(float) * 4 * (far + 1) : 0;
 #define PYRE_TILE16(NV)              \
   do {                               \
@@ -1078,6 +1261,41 @@ extern "C" int pyre_attn_biased_single(const void* q, void* out, int out_ld, int
   PYRE_REQUIRE(known_dtype(dt) && table_stride > 0 && window >= 0 && keep_first >= 0 && far >= 0 && chunk >= 0, "attn_biased_single: bad arguments");
   PYRE_REQUIRE(!part || (max_spans >= 1 && max_spans <= 65535), "attn_biased_single: %d spans are not a launch", max_spans);
   if (n <= 0) return 0;
+  // bfloat16 on the matrix cores, a block per span (a token of one span needs no scratch)
+  const auto a16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  const int col_groups = (nq / nkv + kCols - 1) / kCols;
+  if (dt == kBF16 && (part || max_spans == 1) && dk % 8 == 0 && dv % 8 == 0 && (page_size & (page_size - 1)) == 0 && a16(q) && a16(k_cache) &&
+      a16(v_cache) && static_cast<long>(nkv) * col_groups <= 65535) {
+    const int nh = nq / nkv < kCols ? nq / nkv : kCols, ev = dv <= 128 ? 1 : 2, dks = dk <= 32 ? 1 : dk <= 64 ? 2 : dk <= 128 ? 4 : 8;
+    const size_t lds = sizeof(float) * 4 * nh * (128 * ev + 4);
+#define PYRE_SINGLE16(DKS, EV)                                                                                           \
+  do {                                                                                                                   \
+    static size_t raised = 64 * 1024;                                                                                    \
+    if (lds > raised) {                                                                                                  \
+      if (hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_biased_single16_kernel<DKS, EV>),                      \
+                              hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)) != hipSuccess)          \
+        return fail("attn_biased_single: the device refuses %zu bytes of LDS", lds);                                     \
+      raised = lds;                                                                                                      \
+    }                                                                                                                    \
+    hipLaunchKernelGGL((attn_biased_single16_kernel<DKS, EV>), dim3(n, nkv * col_groups, part ? max_spans : 1), dim3(kThreads), lds, \
+                       stream, static_cast<const bf16*>(q), static_cast<const bf16*>(k_cache), static_cast<const bf16*>(v_cache), \
+                       static_cast<bf16*>(out), out_ld, gate, out_scale, tokens, positions, seq_of_token, block_table,   \
+                       table_stride, nq, nkv, dk, dv, __builtin_ctz(page_size), scale, cap, bias, far, window, keep_first, chunk, \
+                       part, sink, gate_dim);                                                                            \
+  } while (0)
+    if (dks == 1 && ev == 1) PYRE_SINGLE16(1, 1);
+    else if (dks == 2 && ev == 1) PYRE_SINGLE16(2, 1);
+    else if (dks == 4 && ev == 1) PYRE_SINGLE16(4, 1);
+    else if (dks == 8 && ev == 1) PYRE_SINGLE16(8, 1);
+    else if (dks <= 4) PYRE_SINGLE16(4, 2);
+    else PYRE_SINGLE16(8, 2);
+#undef PYRE_SINGLE16
+    if (check_launch("attn_biased_single")) return 1;
+    if (part)
+      hipLaunchKernelGGL(attn_biased_join_kernel<bf16>, dim3(n, nq), dim3(kThreads), 0, stream, part, static_cast<bf16*>(out),
+                         out_ld, gate, out_scale, tokens, positions, nq, dv, window, keep_first, chunk, max_spans, sink, gate_dim);
+    return check_launch("attn_biased_single");
+  }
   // the query heads of a key/value head in blocks of up to kGroup heads, which read the keys and values once for all of
   // them: as many heads a block as still leave two blocks for every compute unit (a head's sums do not depend on its
   // block-mates), equally many in each

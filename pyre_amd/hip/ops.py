@@ -377,10 +377,9 @@ def attn_biased_single(q, out, k_cache, v_cache, gate, out_scale, tokens, n, pos
                         nq, nkv, dk, dv, page_size, sink, gate_dim)
     if tokens is not None:
         _dev(tokens), _i32("tokens", tokens, n)
-    spans = 0
+    spans = attn_biased_spans(block_table.shape[1], page_size, window, keep_first, chunk)
     if scratch is not None:
         _dev(scratch)
-        spans = attn_biased_spans(block_table.shape[1], page_size, window, keep_first, chunk)
         if scratch.dtype != torch.float32 or not scratch.is_contiguous() or scratch.numel() < n * nq * spans * (dv + 2):
             raise KernelError(f"attn_biased_single: scratch of {n * nq * spans * (dv + 2)} float32 elements needed")
     call("pyre_attn_biased_single", q.data_ptr(), out.data_ptr(), out.stride(0), dtype_code(q), k_cache.data_ptr(),
