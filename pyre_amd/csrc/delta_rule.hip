@@ -242,9 +242,10 @@ __global__ __launch_bounds__(2 * kWave) void gdr_scan_lanes_kernel(const float* 
   constexpr int kItems = kGroup * kPieces;
   constexpr int kMine = (kItems + kWave - 1) / kWave;
   __shared__ __attribute__((aligned(16))) float ring[2][kGroup * kTok];
-  const int seq = blockIdx.x, hd = blockIdx.y, lane = threadIdx.x & (kWave - 1);
+  // one request's blocks lie together in the grid: a long prompt beside many single tokens is then spread over all dies
+  const int seq = blockIdx.z, hd = blockIdx.x, lane = threadIdx.x & (kWave - 1);
   const bool fetches = threadIdx.x >= kWave;
-  const int col0 = blockIdx.z * kCols, g = hd / (s.H / s.G);
+  const int col0 = blockIdx.y * kCols, g = hd / (s.H / s.G);
   const int t_begin = q_start[seq], t_end = q_start[seq + 1], width = s.width();
   const int groups = (t_end - t_begin + kGroup - 1) / kGroup;
   if (groups <= 0) return;
@@ -433,13 +434,13 @@ extern "C" int pyre_gdr_scan(const float* x, float* state, float* o, const int* 
                              int max_tokens, int H, int G, int dk, int dv, hipStream_t stream) {
   const Geometry s{H, G, dk, dv};
   PYRE_REQUIRE(good(s) && H <= 65535, "gdr_scan: heads %d / %d of %d / %d elements are not taken", H, G, dk, dv);
-  PYRE_REQUIRE(x && state && o && q_start && state_slots, "gdr_scan: rows, state and the step's arrays are needed");
+  PYRE_REQUIRE(x && state && o && q_start && state_slots && n_seqs <= 65535, "gdr_scan: rows, state and the step's arrays (of at most 65,535 requests) are needed");
   if (n_seqs <= 0) return 0;
   if (dk % 16 == 0 && dk <= 128 && dv % 4 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0) {
     // eight lanes a column where that leaves each a multiple of four rows, else four
 #define PYRE_LANES(DR, LPC)                                                                                             \
   do {                                                                                                                  \
-    const dim3 lanes_grid(n_seqs, H, (dv + kWave / LPC - 1) / (kWave / LPC));                                           \
+    const dim3 lanes_grid(H, (dv + kWave / LPC - 1) / (kWave / LPC), n_seqs);                                           \
     if (max_tokens > 0 && max_tokens <= 2)                                                                              \
       hipLaunchKernelGGL((gdr_scan_lanes_kernel<DR, LPC, 2>), lanes_grid, dim3(2 * kWave), 0, stream, x, state, o, q_start, \
                          state_slots, s);                                                                               \

@@ -244,8 +244,12 @@ __global__ __launch_bounds__(kWave) void gla_chunk_walk_kernel(
     ChunkScratch sc, float* __restrict__ state, float* __restrict__ o, const int* __restrict__ q_start,
     const int* __restrict__ state_slots, int heads, int dk, int dv, int dvp, float qscale) {
   constexpr int dkp = 16 * DT;
-  const int s = blockIdx.x, hd = blockIdx.y, lane = threadIdx.x, g = lane >> 4, c = lane & 15;
-  const int col = blockIdx.z * 16 + c;
+  // the blocks of one request lie together in the grid and not those of one head: neighbours go to different dies, and a
+  // long prompt beside many single tokens is then not one die's alone. Heads are padded to a multiple of eight, so that the
+  // blocks of a head, which read the same operands, share a die and its cache
+  const int s = blockIdx.z, hd = blockIdx.x, lane = threadIdx.x, g = lane >> 4, c = lane & 15;
+  if (hd >= heads) return;
+  const int col = blockIdx.y * 16 + c;
   const bool has_col = col < dv;
   const int t_begin = q_start[s], t_end = q_start[s + 1], hv = heads * dv;
   float* st = state + (static_cast<size_t>(state_slots[s]) * heads + hd) * dk * dv;
@@ -523,7 +527,7 @@ extern "C" int pyre_gla_chunks(const float* x, float* scratch, float* state, flo
   hipLaunchKernelGGL(gla_chunk_prep_kernel, dim3((max_tokens + kChunk - 1) / kChunk, heads, n_seqs), dim3(kThreads),
                      sizeof(float) * 3 * kChunk * dk, stream, x, sc, q_start, heads, dk, dv, dkp, dvp);
   if (check_launch("gla_chunk_prep")) return 1;
-  const dim3 grid(n_seqs, heads, (dv + 15) / 16);
+  const dim3 grid((heads + 7) / 8 * 8, (dv + 15) / 16, n_seqs);
 #define PYRE_WALK(DT)                                                                                                  \
   hipLaunchKernelGGL(gla_chunk_walk_kernel<DT>, grid, dim3(kWave), 0, stream, sc, state, o, q_start, state_slots, heads, \
                      dk, dv, dvp, qscale)
