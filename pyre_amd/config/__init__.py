@@ -8,6 +8,5 @@ from pyre_amd.config.presets import PRESETS, preset
 from pyre_amd.config.rukosun import RukosunConfig
 from pyre_amd.config.zorulix import ZorulixConfig
 
-__all__ = ["ConfigError", "DurelixConfig", "EngineConfig", "MafuraxConfig", "ModelConfig", "NurasunConfig", "PinozenConfig", "Qwen2Config", "PRESETS", "preset",
-           "RukosunConfig",
-           "ZorulixConfig"]
+__all__ = ["ConfigError", "DurelixConfig", "EngineConfig", "MafuraxConfig", "ModelConfig", "NurasunConfig", "PinozenConfig",
+           "Qwen2Config", "PRESETS", "preset", "RukosunConfig", "ZorulixConfig"]
